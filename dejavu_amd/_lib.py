@@ -9,7 +9,7 @@ from __future__ import annotations
 import ctypes
 import os
 
-import torch  # noqa: F401  (loads the HIP runtime that the library binds to)
+from ._binding import DejavuHipError, load_library  # noqa: F401
 
 _PKG_DIR = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_PKG_DIR, "libdejavu_hip.so")
@@ -144,25 +144,7 @@ SIGNATURES = {
 }
 
 
-class DejavuHipError(RuntimeError):
-    """A libdejavu_hip.so entry point returned a non-zero status."""
-
-
-def _load() -> ctypes.CDLL:
-    if not os.path.exists(LIB_PATH):
-        raise ImportError(
-            f"{LIB_PATH} is missing: build it with `python -m dejavu_amd.build` "
-            "(there is no fallback implementation)"
-        )
-    lib = ctypes.CDLL(LIB_PATH)
-    for name, (restype, argtypes) in SIGNATURES.items():
-        fn = getattr(lib, name)
-        fn.restype = restype
-        fn.argtypes = argtypes
-    return lib
-
-
-lib = _load()
+lib = load_library(LIB_PATH, SIGNATURES)
 
 
 def check(code: int, what: str) -> None:

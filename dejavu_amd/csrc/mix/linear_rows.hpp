@@ -1,0 +1,168 @@
+// One activation row times a weight matrix (the products of a decode step), with what comes before and after the
+// product inside the launch:
+//   before: nothing, an RMS norm of the row, or a per-head RMS norm with an output gate;
+//   after : plain store, the clamped gated unit, a short convolution with its state, or dynamic tanh + residual add
+//           + the next dynamic tanh.
+// A wave owns R consecutive rows of W at a time; the row x is staged in LDS once per workgroup.
+#pragma once
+#include "elem.hpp"
+#include "stream.hpp"
+
+namespace dv {
+
+using RowsArgs = dvRowArgs;
+
+// Short convolution of one channel's newest value with its state; returns the filtered value.
+__device__ __forceinline__ float conv_step(float u, const float* __restrict__ w, float* __restrict__ st, int taps) {
+  float y = w[taps - 1] * u;
+  for (int j = 0; j < taps - 1; ++j) {
+    const float old = st[j];
+    y = __builtin_fmaf(w[j], old, y);
+    if (j > 0) st[j - 1] = old;
+  }
+  if (taps > 1) st[taps - 2] = u;
+  return y;
+}
+
+template <typename T, int BEFORE>
+__device__ __forceinline__ void stage_row(const RowsArgs& a, T* xs, float* red) {
+  const int tid = threadIdx.x, K = a.K;
+  if constexpr (BEFORE == DV_ROW_PLAIN) {
+    const T* x = reinterpret_cast<const T*>(a.x);
+    for (int i = tid * 8; i < K; i += 256 * 8) {
+      Pack8<T> v;
+      v.load(x + i);
+      *reinterpret_cast<Pack8<T>*>(xs + i) = v;
+    }
+  } else if constexpr (BEFORE == DV_ROW_RMS) {
+    const float* x = reinterpret_cast<const float*>(a.x);
+    float ss = 0.f;
+    for (int i = tid; i < a.norm_dim; i += 256) ss = __builtin_fmaf(x[i], x[i], ss);
+    ss = wave_sum(ss);
+    if ((tid & 63) == 0) red[tid >> 6] = ss;
+    __syncthreads();
+    const float s = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / a.norm_dim + a.eps);
+    for (int i = tid; i < K; i += 256) xs[i] = from_f<T>(x[i] * s * a.xw[i]);
+  } else {
+    // one head per wave at a time
+    const float* x = reinterpret_cast<const float*>(a.x);
+    const int heads = K / a.head_stride, lane = tid & 63;
+    for (int h = tid >> 6; h < heads; h += 4) {
+      const float* xh = x + (int64_t)h * a.head_stride;
+      float ss = 0.f;
+      for (int c = lane; c < a.norm_dim; c += 64) ss = __builtin_fmaf(xh[c], xh[c], ss);
+      const float s = 1.f / sqrtf(wave_sum(ss) / a.norm_dim + a.eps);
+      for (int c = lane; c < a.head_stride; c += 64)
+        xs[h * a.head_stride + c] = from_f<T>(xh[c] * s * a.xw[c] * a.gate[(int64_t)h * a.head_stride + c]);
+    }
+  }
+  __syncthreads();
+}
+
+template <typename T, int BEFORE, int AFTER, int R, int U>
+__global__ __launch_bounds__(256) void linear_rows_kernel(RowsArgs a) {
+  extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
+  T* xs = reinterpret_cast<T*>(smem_raw);
+  __shared__ float red[4];
+  const int lane = threadIdx.x & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  int nblocks = gridDim.x;
+  if (a.side_x) {
+    --nblocks;
+    if ((int)blockIdx.x == nblocks) {
+      float ss = 0.f;
+      for (int i = threadIdx.x; i < a.side_dim; i += 256) ss = __builtin_fmaf(a.side_x[i], a.side_x[i], ss);
+      ss = wave_sum(ss);
+      if (lane == 0) red[wave] = ss;
+      __syncthreads();
+      const float s = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / a.side_dim + a.eps);
+      T* o = reinterpret_cast<T*>(a.side_out) + (int64_t)seq_position(a.pos_dev, a.pos_host) * a.side_ld;
+      for (int i = threadIdx.x; i < a.side_padded; i += 256) o[i] = from_f<T>(a.side_x[i] * s * a.side_w[i]);
+      return;
+    }
+  }
+  constexpr int CH = 8 * kWave;
+  const T* W = reinterpret_cast<const T*>(a.W);
+  const int K = a.K, ntasks = (a.M + R - 1) / R;
+  int t = blockIdx.x * 4 + wave;
+  Pack8<T> w[U][R];
+  const T* wr[R];
+  auto rows_of = [&](int task) {
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      const int row = task * R + r;
+      wr[r] = W + (int64_t)(row < a.M ? row : 0) * a.ldw + lane * 8;
+    }
+  };
+  auto load_w = [&](int base) {
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+        if (base + u * CH + lane * 8 < K) w[u][r].load_stream(wr[r] + base + u * CH);
+        else w[u][r].zero();
+      }
+  };
+  if (t < ntasks) {  // the first weights are requested before x is there
+    rows_of(t);
+    load_w(0);
+  }
+  stage_row<T, BEFORE>(a, xs, red);
+  for (; t < ntasks; t += nblocks * 4) {
+    float acc[R];
+#pragma unroll
+    for (int r = 0; r < R; ++r) acc[r] = 0.f;
+    for (int base = 0; base < K; base += U * CH) {
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int k = base + u * CH + lane * 8;
+        if (k < K) {
+          Pack8<T> xv;
+          xv = *reinterpret_cast<const Pack8<T>*>(xs + k);
+#pragma unroll
+          for (int r = 0; r < R; ++r)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) acc[r] = __builtin_fmaf(w[u][r].get(e), xv.get(e), acc[r]);
+        }
+      }
+      if (base + U * CH < K) load_w(base + U * CH);
+    }
+#pragma unroll
+    for (int r = 0; r < R; ++r) acc[r] = wave_sum(acc[r]);
+    const int row0 = t * R;
+    if (t + nblocks * 4 < ntasks) {
+      rows_of(t + nblocks * 4);
+      load_w(0);
+    }
+    if constexpr (AFTER == DV_OUT_GLU) {
+      static_assert(R % 2 == 0, "gate / up rows come in pairs");
+#pragma unroll
+      for (int r = 0; r < R; r += 2)
+        if (lane == r && row0 + r + 1 < a.M)
+          reinterpret_cast<T*>(a.out)[(row0 + r) >> 1] = from_f<T>(clamped_glu_f(acc[r], acc[r + 1], a.limit));
+    } else {
+      float v = 0.f;
+#pragma unroll
+      for (int r = 0; r < R; ++r)
+        if (lane == r) v = acc[r];
+      const int row = row0 + lane;
+      if (lane < R && row < a.M) {
+        if constexpr (AFTER == DV_OUT_F32) {
+          reinterpret_cast<float*>(a.out)[row] = v;
+        } else if constexpr (AFTER == DV_OUT_T) {
+          reinterpret_cast<T*>(a.out)[row] = from_f<T>(v);
+        } else if constexpr (AFTER == DV_OUT_CONV) {
+          if (row < a.conv_rows) {
+            v = conv_step(v, a.conv_w + (int64_t)row * a.taps, a.conv_state + (int64_t)row * (a.taps - 1), a.taps);
+            if (a.silu) v = silu_f(v);
+          }
+          reinterpret_cast<float*>(a.out)[row] = v;
+        } else {
+          residual_apply<T>(a.res, row, row, v);
+        }
+      }
+    }
+  }
+}
+
+}  // namespace dv

@@ -1,0 +1,404 @@
+// C ABI of libdejavu_mixers.so (include/dejavu_mixers.h): argument checks on the host, then launches.
+#include "../../include/dejavu_mixers.h"
+
+#include <hip/hip_runtime.h>
+
+#include <atomic>
+
+#include "mix/attn_rows.hpp"
+#include "mix/attn_tiles.hpp"
+#include "mix/delta_rule.hpp"
+#include "mix/linear_rows.hpp"
+#include "mix/linear_tiles.hpp"
+#include "mix/short_conv.hpp"
+#include "mix/stream.hpp"
+
+using namespace dv;
+
+namespace {
+
+inline bool al16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15u) == 0; }
+inline int launched() { return hipGetLastError() == hipSuccess ? DV_OK : DV_ERR_LAUNCH; }
+inline hipStream_t st(void* s) { return reinterpret_cast<hipStream_t>(s); }
+inline bool dtype_ok(int d) { return d == DV_BF16 || d == DV_F32; }
+inline unsigned blocks_of(int64_t work, int64_t per) { return (unsigned)((work + per - 1) / per); }
+
+// Dynamic LDS above 48 KiB is granted per kernel and device.
+template <auto KERNEL>
+int grant(size_t bytes) {
+  static std::atomic<size_t> granted[64];
+  if (bytes <= 48 * 1024) return DV_OK;
+  if (bytes > 158 * 1024) return DV_ERR_UNSUPPORTED;
+  int dev = 0;
+  if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev >= 64) return DV_ERR_UNSUPPORTED;
+  if (bytes <= granted[dev].load(std::memory_order_relaxed)) return DV_OK;
+  if (hipFuncSetAttribute(reinterpret_cast<const void*>(KERNEL), hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes) !=
+      hipSuccess)
+    return DV_ERR_UNSUPPORTED;
+  granted[dev].store(bytes, std::memory_order_relaxed);
+  return DV_OK;
+}
+
+template <auto KERNEL, typename... A>
+int launch_lds(dim3 grid, dim3 block, size_t lds, hipStream_t s, A... args) {
+  const int rc = grant<KERNEL>(lds);
+  if (rc != DV_OK) return rc;
+  hipLaunchKernelGGL(KERNEL, grid, block, lds, s, args...);
+  return launched();
+}
+
+// ---- one row ---------------------------------------------------------------
+template <typename T, int BEFORE, int AFTER>
+int linear_row(const RowsArgs& a, hipStream_t s) {
+  constexpr int R = AFTER == DV_OUT_GLU ? 2 : 2, U = sizeof(T) == 2 ? 4 : 2;
+  const int ntasks = (a.M + R - 1) / R;
+  int blocks = (ntasks + 3) / 4;
+  if (blocks > 2048) blocks = 2048;
+  if (a.side_x) ++blocks;
+  return launch_lds<linear_rows_kernel<T, BEFORE, AFTER, R, U>>(dim3(blocks), dim3(256), (size_t)a.K * sizeof(T), s, a);
+}
+template <typename T>
+int linear_row_any(int before, int after, const RowsArgs& a, hipStream_t s) {
+  if (before == DV_ROW_PLAIN) {
+    switch (after) {
+      case DV_OUT_F32: return linear_row<T, DV_ROW_PLAIN, DV_OUT_F32>(a, s);
+      case DV_OUT_T: return linear_row<T, DV_ROW_PLAIN, DV_OUT_T>(a, s);
+      case DV_OUT_GLU: return linear_row<T, DV_ROW_PLAIN, DV_OUT_GLU>(a, s);
+      case DV_OUT_RESIDUAL: return linear_row<T, DV_ROW_PLAIN, DV_OUT_RESIDUAL>(a, s);
+      case DV_OUT_CONV: return linear_row<T, DV_ROW_PLAIN, DV_OUT_CONV>(a, s);
+    }
+  } else if (before == DV_ROW_RMS && after == DV_OUT_F32) {
+    return linear_row<T, DV_ROW_RMS, DV_OUT_F32>(a, s);
+  } else if (before == DV_ROW_HEADS && after == DV_OUT_RESIDUAL) {
+    return linear_row<T, DV_ROW_HEADS, DV_OUT_RESIDUAL>(a, s);
+  }
+  return DV_ERR_UNSUPPORTED;
+}
+
+// ---- attention rows --------------------------------------------------------
+template <typename T, typename TQ, int RH>
+int attn_rows_rh(const AttnArgs& a, hipStream_t s) {
+  const int rep = a.H / a.G;
+  const dim3 grid(a.splits, a.G * ((rep + RH - 1) / RH), a.n);
+  const size_t lds = (size_t)RH * a.dim_s * 4 + 256 * 8 * 4;
+  return launch_lds<attn_rows_kernel<T, TQ, RH>>(grid, dim3(256), lds, s, a);
+}
+template <typename T, typename TQ>
+int attn_rows_any(const AttnArgs& a, hipStream_t s) {
+  const int rep = a.H / a.G;
+  if (rep >= 8) return attn_rows_rh<T, TQ, 8>(a, s);
+  if (rep >= 3) return attn_rows_rh<T, TQ, 4>(a, s);
+  if (rep == 2) return attn_rows_rh<T, TQ, 2>(a, s);
+  return attn_rows_rh<T, TQ, 1>(a, s);
+}
+
+int attn_args_ok(const AttnArgs* a) {
+  if (!a || !a->q || !a->k || !a->v || a->n < 1 || a->H < 1 || a->G < 1 || a->H % a->G || a->dim_s < 8 ||
+      a->vdim_s < 8 || a->splits < 1 || (a->splits > 1 && !a->part) || (a->splits == 1 && !a->out) ||
+      (!a->fresh_k != !a->fresh_v))
+    return DV_ERR_INVALID_ARG;
+  if (a->dim_s % 8 || a->vdim_s % 8 || a->ldk % 8 || a->ldv % 8 || a->k_head % 8 || a->v_head % 8 || !al16(a->k) ||
+      !al16(a->v) || !al16(a->q))
+    return DV_ERR_ALIGNMENT;
+  if (a->vdim_s > 2048 || a->n > 65535 || (int64_t)a->H > 65535) return DV_ERR_UNSUPPORTED;
+  return DV_OK;
+}
+
+template <int DT, int VT>
+int attn_tiles_launch(const AttnArgs& a, int keys, hipStream_t s) {
+  hipLaunchKernelGGL((attn_tiles_kernel<DT, VT>), dim3((unsigned)((int64_t)a.H * ((a.n + kTileQ - 1) / kTileQ))), dim3(256), 0, s, a, keys);
+  return launched();
+}
+
+}  // namespace
+
+extern "C" {
+
+int dv_mix_embed(int dtype, const void* tokens, int64_t vocab, const void* embed, int n, int width, float* x, float* x0,
+                 const dvDynTanh* norm, void* h, void* stream) {
+  if (!dtype_ok(dtype) || !tokens || !embed || n < 1 || width < 1 || !x || !norm || !norm->w || !norm->b || !h)
+    return DV_ERR_INVALID_ARG;
+  const int64_t* t = reinterpret_cast<const int64_t*>(tokens);
+  if (dtype == DV_BF16)
+    hipLaunchKernelGGL((embed_norm_kernel<bf16_t>), dim3(n), dim3(256), 0, st(stream), t, vocab, (const bf16_t*)embed,
+                       width, x, x0, *norm, (bf16_t*)h);
+  else
+    hipLaunchKernelGGL((embed_norm_kernel<float>), dim3(n), dim3(256), 0, st(stream), t, vocab, (const float*)embed,
+                       width, x, x0, *norm, (float*)h);
+  return launched();
+}
+
+int dv_mix_residual(int dtype, const void* y, int64_t n, int width, const dvResidual* r, void* stream) {
+  if (!dtype_ok(dtype) || n < 1 || width < 1 || !r || !r->x || (y && (!r->post.w || !r->post.b)) ||
+      (r->h && (!r->pre.w || !r->pre.b)))
+    return DV_ERR_INVALID_ARG;
+  const int64_t count = n * width;
+  unsigned grid = blocks_of(count, 256);
+  if (grid > 16384) grid = 16384;
+  if (dtype == DV_BF16)
+    hipLaunchKernelGGL((residual_norm_kernel<bf16_t>), dim3(grid), dim3(256), 0, st(stream), (const bf16_t*)y, count, width, *r);
+  else
+    hipLaunchKernelGGL((residual_norm_kernel<float>), dim3(grid), dim3(256), 0, st(stream), (const float*)y, count, width, *r);
+  return launched();
+}
+
+int dv_mix_clamped_glu(int dtype, const void* gu, int64_t count, float limit, void* y, void* stream) {
+  if (!dtype_ok(dtype) || !gu || !y || count < 4) return DV_ERR_INVALID_ARG;
+  if (count % 4 || !al16(gu)) return DV_ERR_ALIGNMENT;
+  const dim3 grid(blocks_of(count, 1024));
+  if (dtype == DV_BF16)
+    hipLaunchKernelGGL((clamped_glu_kernel<bf16_t>), grid, dim3(256), 0, st(stream), (const bf16_t*)gu, count, limit, (bf16_t*)y);
+  else
+    hipLaunchKernelGGL((clamped_glu_kernel<float>), grid, dim3(256), 0, st(stream), (const float*)gu, count, limit, (float*)y);
+  return launched();
+}
+
+int dv_mix_rms_rows(int dtype, const void* x, int64_t ldx, int64_t rows, int dim, int padded, const float* w, float eps,
+                    void* y, int64_t ldy, void* stream) {
+  if (!dtype_ok(dtype) || !x || !w || !y || rows < 1 || dim < 1 || padded < dim) return DV_ERR_INVALID_ARG;
+  const dim3 grid(blocks_of(rows, 4));
+  if (dtype == DV_BF16)
+    hipLaunchKernelGGL((rms_rows_kernel<bf16_t>), grid, dim3(256), 0, st(stream), (const bf16_t*)x, ldx, rows, dim, padded, w, eps, (bf16_t*)y, ldy);
+  else
+    hipLaunchKernelGGL((rms_rows_kernel<float>), grid, dim3(256), 0, st(stream), (const float*)x, ldx, rows, dim, padded, w, eps, (float*)y, ldy);
+  return launched();
+}
+
+int dv_mix_gated_head_norm(int dtype, const float* o, const void* gate, int64_t ldg, int64_t rows, int heads, int vdim,
+                           int padded, const float* w, float eps, void* y, void* stream) {
+  if (!dtype_ok(dtype) || !o || !gate || !w || !y || rows < 1 || heads < 1 || vdim < 1 || padded < vdim)
+    return DV_ERR_INVALID_ARG;
+  const dim3 grid(blocks_of(rows * heads, 4));
+  if (dtype == DV_BF16)
+    hipLaunchKernelGGL((gated_head_norm_kernel<bf16_t>), grid, dim3(256), 0, st(stream), o, (const bf16_t*)gate, ldg, rows, heads, vdim, padded, w, eps, (bf16_t*)y);
+  else
+    hipLaunchKernelGGL((gated_head_norm_kernel<float>), grid, dim3(256), 0, st(stream), o, (const float*)gate, ldg, rows, heads, vdim, padded, w, eps, (float*)y);
+  return launched();
+}
+
+int dv_mix_linear_row(int dtype, int before, int after, const dvRowArgs* a, void* stream) {
+  if (!dtype_ok(dtype) || !a || !a->x || !a->W || a->M < 1 || a->K < 8) return DV_ERR_INVALID_ARG;
+  if (a->K % 8 || a->ldw % 8 || !al16(a->W) || !al16(a->x)) return DV_ERR_ALIGNMENT;
+  if (after != DV_OUT_RESIDUAL && !a->out) return DV_ERR_INVALID_ARG;
+  if (after == DV_OUT_GLU && a->M % 2) return DV_ERR_INVALID_ARG;
+  if (after == DV_OUT_RESIDUAL && (!a->res.x || !a->res.post.w || (a->res.h && !a->res.pre.w))) return DV_ERR_INVALID_ARG;
+  if (after == DV_OUT_CONV && (!a->conv_w || a->taps < 1 || (a->taps > 1 && !a->conv_state) || a->conv_rows > a->M))
+    return DV_ERR_INVALID_ARG;
+  if (before == DV_ROW_RMS && (!a->xw || a->norm_dim < 1 || a->norm_dim > a->K)) return DV_ERR_INVALID_ARG;
+  if (before == DV_ROW_HEADS && (!a->xw || !a->gate || a->head_stride < 1 || a->K % a->head_stride ||
+                                 a->norm_dim < 1 || a->norm_dim > a->head_stride))
+    return DV_ERR_INVALID_ARG;
+  if (a->side_x && (!a->side_w || !a->side_out || a->side_dim < 1)) return DV_ERR_INVALID_ARG;
+  return dtype == DV_BF16 ? linear_row_any<bf16_t>(before, after, *a, st(stream))
+                          : linear_row_any<float>(before, after, *a, st(stream));
+}
+
+int dv_mix_linear_tiles(int after, const dvTileArgs* a, void* stream) {
+  if (!a || !a->x || !a->W || a->n < 1 || a->M < 1 || a->K < 8) return DV_ERR_INVALID_ARG;
+  if (a->K % 8 || a->ldw % 8 || a->ldx % 8 || !al16(a->W) || !al16(a->x)) return DV_ERR_ALIGNMENT;
+  if (after != DV_OUT_RESIDUAL && !a->out) return DV_ERR_INVALID_ARG;
+  if (after == DV_OUT_GLU && a->M % 2) return DV_ERR_INVALID_ARG;
+  if (after == DV_OUT_RESIDUAL && (!a->res.x || !a->res.post.w || (a->res.h && !a->res.pre.w))) return DV_ERR_INVALID_ARG;
+  const int nt = a->n <= 16 ? 1 : (a->n <= 32 ? 2 : 4);
+  const dim3 grid((a->M + 31) / 32, (a->n + 16 * nt - 1) / (16 * nt));
+  if (grid.y > 65535) return DV_ERR_UNSUPPORTED;
+#define DV_TILE(AFTER)                                                                                              \
+  do {                                                                                                              \
+    if (nt == 1) hipLaunchKernelGGL((linear_tiles_kernel<AFTER, 1>), grid, dim3(256), 0, st(stream), *a);            \
+    else if (nt == 2) hipLaunchKernelGGL((linear_tiles_kernel<AFTER, 2>), grid, dim3(256), 0, st(stream), *a);       \
+    else hipLaunchKernelGGL((linear_tiles_kernel<AFTER, 4>), grid, dim3(256), 0, st(stream), *a);                    \
+  } while (0)
+  switch (after) {
+    case DV_OUT_F32: DV_TILE(DV_OUT_F32); break;
+    case DV_OUT_T: DV_TILE(DV_OUT_T); break;
+    case DV_OUT_GLU: DV_TILE(DV_OUT_GLU); break;
+    case DV_OUT_RESIDUAL: DV_TILE(DV_OUT_RESIDUAL); break;
+    default: return DV_ERR_UNSUPPORTED;
+  }
+#undef DV_TILE
+  return launched();
+}
+
+int dv_mix_short_conv(int dtype, int out_f32, const dvConvArgs* a, void* stream) {
+  if (!dtype_ok(dtype) || !a || !a->in || a->n < 1 || a->taps < 1 || !a->w || (a->taps > 1 && !a->state))
+    return DV_ERR_INVALID_ARG;
+  int heads = 0, widest = 0;
+  for (const dvConvGroup& g : a->g) {
+    if (g.heads < 0 || (g.heads > 0 && (!g.out || g.stride < 1 || g.dim < 1))) return DV_ERR_INVALID_ARG;
+    heads += g.heads;
+    if (g.heads > 0 && g.stride > widest) widest = g.stride;
+  }
+  if (heads == 0) return DV_ERR_INVALID_ARG;
+  if (widest > 1024) return DV_ERR_UNSUPPORTED;
+  const dim3 grid(blocks_of((int64_t)a->n * heads, 4));
+#define DV_CONV(T, TO)                                                                                       \
+  do {                                                                                                       \
+    if (widest <= 128) hipLaunchKernelGGL((short_conv_kernel<T, TO, 2>), grid, dim3(256), 0, st(stream), *a); \
+    else if (widest <= 256) hipLaunchKernelGGL((short_conv_kernel<T, TO, 4>), grid, dim3(256), 0, st(stream), *a); \
+    else hipLaunchKernelGGL((short_conv_kernel<T, TO, 16>), grid, dim3(256), 0, st(stream), *a);             \
+  } while (0)
+  if (dtype == DV_F32) DV_CONV(float, float);
+  else if (out_f32) DV_CONV(bf16_t, float);
+  else DV_CONV(bf16_t, bf16_t);
+#undef DV_CONV
+  return launched();
+}
+
+int dv_mix_conv_state(int dtype, const void* in, int64_t ldi, int n, int channels, int taps, float* state, void* stream) {
+  if (!dtype_ok(dtype) || !in || n < 1 || channels < 1 || taps < 1 || (taps > 1 && !state)) return DV_ERR_INVALID_ARG;
+  if (taps == 1) return DV_OK;
+  const dim3 grid(blocks_of(channels, 256));
+  if (dtype == DV_BF16)
+    hipLaunchKernelGGL((conv_state_kernel<bf16_t>), grid, dim3(256), 0, st(stream), (const bf16_t*)in, ldi, n, channels, taps, state);
+  else
+    hipLaunchKernelGGL((conv_state_kernel<float>), grid, dim3(256), 0, st(stream), (const float*)in, ldi, n, channels, taps, state);
+  return launched();
+}
+
+int dv_mix_ring_copy(int dtype, void* buf, int64_t ldb, void* ring, int cap, int64_t ldr, int first, int count, int width,
+                     int to_ring, void* stream) {
+  if (!dtype_ok(dtype) || !buf || !ring || cap < 1 || first < 0 || count < 0 || count > cap || width < 8)
+    return DV_ERR_INVALID_ARG;
+  if (width % 8 || ldb % 8 || ldr % 8 || !al16(buf) || !al16(ring)) return DV_ERR_ALIGNMENT;
+  if (count == 0) return DV_OK;
+  unsigned grid = blocks_of((int64_t)count * (width / 8), 256);
+  if (grid > 4096) grid = 4096;
+  if (dtype == DV_BF16)
+    hipLaunchKernelGGL((ring_copy_kernel<bf16_t>), dim3(grid), dim3(256), 0, st(stream), (bf16_t*)buf, ldb, (bf16_t*)ring, cap, ldr, first, count, width, to_ring);
+  else
+    hipLaunchKernelGGL((ring_copy_kernel<float>), dim3(grid), dim3(256), 0, st(stream), (float*)buf, ldb, (float*)ring, cap, ldr, first, count, width, to_ring);
+  return launched();
+}
+
+int dv_mix_attn_rows(int dtype, int q_f32, const dvAttnArgs* a, void* stream) {
+  if (!dtype_ok(dtype)) return DV_ERR_INVALID_ARG;
+  int rc = attn_args_ok(a);
+  if (rc != DV_OK) return rc;
+  if (!a->out) return DV_ERR_INVALID_ARG;
+  if (dtype == DV_F32) rc = attn_rows_any<float, float>(*a, st(stream));
+  else if (q_f32) rc = attn_rows_any<bf16_t, float>(*a, st(stream));
+  else rc = attn_rows_any<bf16_t, bf16_t>(*a, st(stream));
+  if (rc != DV_OK || a->splits == 1) return rc;
+  const dim3 grid(a->H, a->n);
+  if (dtype == DV_F32) hipLaunchKernelGGL((attn_merge_kernel<float, float>), grid, dim3(256), 0, st(stream), *a);
+  else if (q_f32) hipLaunchKernelGGL((attn_merge_kernel<bf16_t, float>), grid, dim3(256), 0, st(stream), *a);
+  else hipLaunchKernelGGL((attn_merge_kernel<bf16_t, bf16_t>), grid, dim3(256), 0, st(stream), *a);
+  return launched();
+}
+
+int dv_mix_attn_tiles(const dvAttnArgs* a, int keys, void* stream) {
+  int rc = attn_args_ok(a);
+  if (rc != DV_OK) return rc;
+  if (!a->out || a->ring > 0 || a->fresh_k || a->norm_dim > 0 || a->pos_dev || keys < 1 ||
+      a->pos_host - a->base < 0 || a->pos_host - a->base + a->n > keys)
+    return DV_ERR_INVALID_ARG;
+  if (a->ldq % 8) return DV_ERR_ALIGNMENT;
+  const int dt = (a->dim_s + 15) / 16, vt = (a->vdim_s + 31) / 32;
+#define DV_TILES_V(DT)                                                        \
+  do {                                                                        \
+    if (vt <= 2) return attn_tiles_launch<DT, 2>(*a, keys, st(stream));       \
+    if (vt <= 4) return attn_tiles_launch<DT, 4>(*a, keys, st(stream));       \
+    if (vt <= 8) return attn_tiles_launch<DT, 8>(*a, keys, st(stream));       \
+    return DV_ERR_UNSUPPORTED;                                                \
+  } while (0)
+  if (dt <= 4) DV_TILES_V(4);
+  if (dt <= 8) DV_TILES_V(8);
+  if (dt <= 12) DV_TILES_V(12);
+  if (dt <= 16) DV_TILES_V(16);
+#undef DV_TILES_V
+  return DV_ERR_UNSUPPORTED;
+}
+
+int dv_mix_latent_absorb(int dtype, const float* q, const void* W, int H, int dim_s, int rank, float* out, void* stream) {
+  if (!dtype_ok(dtype) || !q || !W || !out || H < 1 || dim_s < 1 || rank < 8) return DV_ERR_INVALID_ARG;
+  if (rank % 8 || !al16(W)) return DV_ERR_ALIGNMENT;
+  const dim3 grid(H, (rank + 127) / 128);
+  if (dtype == DV_BF16)
+    hipLaunchKernelGGL((latent_absorb_kernel<bf16_t>), grid, dim3(256), 0, st(stream), q, (const bf16_t*)W, dim_s, rank, out);
+  else
+    hipLaunchKernelGGL((latent_absorb_kernel<float>), grid, dim3(256), 0, st(stream), q, (const float*)W, dim_s, rank, out);
+  return launched();
+}
+
+int dv_mix_latent_attn(int dtype, const dvAttnArgs* a, const void* W, int vrows, void* out, void* stream) {
+  if (!dtype_ok(dtype) || !W || !out || vrows < 1 || !a || a->n != 1 || a->G != 1 || !a->part) return DV_ERR_INVALID_ARG;
+  dvAttnArgs b = *a;
+  // one split also goes through the partial sums: the value product reads them
+  const int splits = b.splits;
+  if (splits < 2) return DV_ERR_INVALID_ARG;
+  int rc = attn_args_ok(&b);
+  if (rc != DV_OK) return rc;
+  if (!al16(W)) return DV_ERR_ALIGNMENT;
+  rc = dtype == DV_BF16 ? attn_rows_any<bf16_t, float>(b, st(stream)) : attn_rows_any<float, float>(b, st(stream));
+  if (rc != DV_OK) return rc;
+  const dim3 grid(b.H, vrows <= 16 ? 1 : (vrows <= 64 ? 2 : 8));
+  const size_t lds = (size_t)b.vdim_s * 4;
+  if (dtype == DV_BF16)
+    hipLaunchKernelGGL((latent_out_kernel<bf16_t>), grid, dim3(256), lds, st(stream), b, (const bf16_t*)W, vrows, (bf16_t*)out);
+  else
+    hipLaunchKernelGGL((latent_out_kernel<float>), grid, dim3(256), lds, st(stream), b, (const float*)W, vrows, (float*)out);
+  return launched();
+}
+
+int dv_mix_delta_gates(int dtype, const void* z, int64_t ldz, const void* b, int64_t ldb, const float* A_log,
+                       const float* dt_bias, int n, int heads, int dim_s, float* g, float* beta, void* stream) {
+  if (!dtype_ok(dtype) || !z || !b || !A_log || !dt_bias || n < 1 || heads < 1 || dim_s < 1 || !g || !beta)
+    return DV_ERR_INVALID_ARG;
+  const dim3 grid(blocks_of((int64_t)n * heads * dim_s, 256));
+  if (dtype == DV_BF16)
+    hipLaunchKernelGGL((delta_gates_kernel<bf16_t>), grid, dim3(256), 0, st(stream), (const bf16_t*)z, ldz, (const bf16_t*)b, ldb, A_log, dt_bias, n, heads, dim_s, g, beta);
+  else
+    hipLaunchKernelGGL((delta_gates_kernel<float>), grid, dim3(256), 0, st(stream), (const float*)z, ldz, (const float*)b, ldb, A_log, dt_bias, n, heads, dim_s, g, beta);
+  return launched();
+}
+
+int dv_mix_delta_scan(const dvDeltaArgs* a, void* stream) {
+  if (!a || !a->q || !a->k || !a->v || !a->g || !a->beta || !a->S || !a->o || a->n < 1 || a->heads < 1 ||
+      a->kv_heads < 1 || a->heads % a->kv_heads || a->dim_s < 8 || a->vdim_s < 1)
+    return DV_ERR_INVALID_ARG;
+  if (a->dim_s % 8 || !al16(a->q) || !al16(a->k) || !al16(a->g) || !al16(a->S)) return DV_ERR_ALIGNMENT;
+  const dim3 grid((unsigned)(a->heads * ((a->vdim_s + kDeltaCols - 1) / kDeltaCols)));
+  if (a->dim_s <= 64) hipLaunchKernelGGL((delta_scan_kernel<4>), grid, dim3(256), 0, st(stream), *a);
+  else if (a->dim_s <= 128) hipLaunchKernelGGL((delta_scan_kernel<8>), grid, dim3(256), 0, st(stream), *a);
+  else if (a->dim_s <= 192) hipLaunchKernelGGL((delta_scan_kernel<12>), grid, dim3(256), 0, st(stream), *a);
+  else if (a->dim_s <= 256) hipLaunchKernelGGL((delta_scan_kernel<16>), grid, dim3(256), 0, st(stream), *a);
+  else return DV_ERR_UNSUPPORTED;
+  return launched();
+}
+
+int dv_mix_delta_step(int dtype, const dvDeltaStepArgs* a, void* stream) {
+  if (!dtype_ok(dtype) || !a || !a->p || !a->Wa || !a->Wg || !a->A_log || !a->dt_bias || !a->S || !a->o || !a->gate ||
+      a->heads < 1 || a->kv_heads < 1 || a->heads % a->kv_heads || a->dim < 1 || a->dim_s < a->dim || a->vdim_s < 1 ||
+      a->rank_a < 8 || a->rank_g < 8)
+    return DV_ERR_INVALID_ARG;
+  if (a->dim_s % 8 || a->rank_a % 8 || a->rank_g % 8 || !al16(a->Wa) || !al16(a->Wg) || !al16(a->S)) return DV_ERR_ALIGNMENT;
+  const dim3 grid((unsigned)(a->heads * ((a->vdim_s + kDeltaCols - 1) / kDeltaCols)));
+  const size_t lds = (size_t)(a->rank_a + a->rank_g) * 4;
+  if (lds > 40 * 1024) return DV_ERR_UNSUPPORTED;
+#define DV_STEP(T)                                                                                                  \
+  do {                                                                                                              \
+    if (a->dim_s <= 64) hipLaunchKernelGGL((delta_decode_kernel<T, 4>), grid, dim3(256), lds, st(stream), *a);       \
+    else if (a->dim_s <= 128) hipLaunchKernelGGL((delta_decode_kernel<T, 8>), grid, dim3(256), lds, st(stream), *a); \
+    else if (a->dim_s <= 192) hipLaunchKernelGGL((delta_decode_kernel<T, 12>), grid, dim3(256), lds, st(stream), *a); \
+    else if (a->dim_s <= 256) hipLaunchKernelGGL((delta_decode_kernel<T, 16>), grid, dim3(256), lds, st(stream), *a); \
+    else return DV_ERR_UNSUPPORTED;                                                                                 \
+  } while (0)
+  if (dtype == DV_BF16) DV_STEP(bf16_t);
+  else DV_STEP(float);
+#undef DV_STEP
+  return launched();
+}
+
+int dv_mix_greedy_advance(const float* logits, int vocab, void* token, void* position, void* seq_pos, void* sequences,
+                          int64_t seq_capacity, void* out_index, float* scores, int64_t score_ld, int64_t score_rows,
+                          void* score_index, void* stream) {
+  if (!logits || vocab < 1 || !token || !position || !seq_pos || !sequences || !out_index || seq_capacity < 0 ||
+      (scores && (!score_index || score_ld < vocab || score_rows < 0)))
+    return DV_ERR_INVALID_ARG;
+  hipLaunchKernelGGL(greedy_advance_f32_kernel, dim3(1), dim3(1024), 0, st(stream), logits, vocab, (int64_t*)token,
+                     (int64_t*)position, (int*)seq_pos, (int64_t*)sequences, (int64_t*)out_index, scores, score_ld,
+                     (int64_t*)score_index, seq_capacity, score_rows);
+  return launched();
+}
+
+}  // extern "C"

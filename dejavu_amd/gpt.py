@@ -8,21 +8,12 @@ block, a final add + LayerNorm and an lm_head tied to the word embeddings.  The
 first block receives no prediction and therefore runs dense, as in the
 reference.
 
-``generate`` restates the greedy loop the reference reaches through
-``model.generate`` (flash-attention v0.2.8 ``flash_attn/utils/generation.py``,
-call site Dejavu/benchmarks/benchmark_generation_opt_dejavu.py:187-196).  With
-``cg=True`` a decode step (all layers, lm_head, argmax and the bookkeeping of
-token / position / sequence length) is replayed from HIP graphs: the values that
-change from token to token live in device buffers, and the one host-side
-quantity a step depends on, the position inside the 16-token back-fill window,
-selects the graph: one graph holds a whole window (16 tokens per launch), and 16
-single-position graphs serve the tokens before the first and after the last whole
-window.
+``generate`` is the shared greedy loop (generation.py); a decode step's host-side state is the position inside the
+16-token back-fill window, so a captured period is one window.
 """
 from __future__ import annotations
 
 import math
-from collections import namedtuple
 from dataclasses import dataclass, field
 from functools import partial
 from typing import List, Optional
@@ -34,11 +25,9 @@ import torch.nn.functional as F
 from . import modules as dv_modules
 from . import fused_layer, ops
 from .block import BlockDejavu, BlockMlpAttSparse
-from .modules import (InferenceParams, ParallelFusedMLPDejavu, ParallelMHADejavu, ParallelMHASparseAttMlp,
-                      decode_linear)
-
-CausalLMOutput = namedtuple("CausalLMOutput", ["logits"])
-GreedySearchDecoderOnlyOutput = namedtuple("GreedySearchDecoderOnlyOutput", ["sequences", "scores"])
+from .generation import (CausalLMOutput, GreedyDecoding,  # noqa: F401
+                         GreedySearchDecoderOnlyOutput)
+from .modules import ParallelFusedMLPDejavu, ParallelMHADejavu, ParallelMHASparseAttMlp, decode_linear
 
 
 @dataclass
@@ -217,26 +206,10 @@ class GPTModel(nn.Module):
         return hidden_states
 
 
-class _DecodingCache:
-    """Buffers and graphs of a generation session (batch 1), kept on the model between
-    ``generate`` calls of the same maximum length."""
+class GPTLMHeadModel(GreedyDecoding, nn.Module):
+    decode_period = ParallelMHASparseAttMlp.WINDOW
+    decode_warm_steps = ParallelMHASparseAttMlp.WINDOW
 
-    def __init__(self, model, max_length, device, dtype):
-        self.max_length = max_length
-        self.inference_params = InferenceParams(max_sequence_len=max_length, max_batch_size=1)
-        # device-resident per-token state
-        self.token = torch.zeros(1, 1, dtype=torch.long, device=device)
-        self.position = torch.zeros(1, 1, dtype=torch.long, device=device)
-        self.seq_pos = torch.zeros(1, dtype=torch.int32, device=device)  # == lengths_per_sample
-        self.out_index = torch.zeros(1, dtype=torch.long, device=device)    # column of `sequences` to write
-        self.score_index = torch.zeros(1, dtype=torch.long, device=device)  # row of `scores` to write
-        self.sequences = torch.zeros(1, max_length, dtype=torch.long, device=device)
-        self.scores = None
-        self.graphs = {}
-        self.counters_after = {}
-
-
-class GPTLMHeadModel(nn.Module):
     def __init__(self, config, process_group=None, device=None, dtype=None):
         super().__init__()
         assert process_group is None, "this build runs the model on one GPU"
@@ -246,7 +219,6 @@ class GPTLMHeadModel(nn.Module):
         vocab_size = math.ceil(config.vocab_size / pad) * pad
         self.lm_head = nn.Linear(config.hidden_size, vocab_size, bias=False, device=device, dtype=dtype)
         self.tie_weights()
-        self._decoding_cache = None
 
     def tie_weights(self):
         self.lm_head.weight = self.transformer.embeddings.word_embeddings.weight
@@ -263,112 +235,26 @@ class GPTLMHeadModel(nn.Module):
     def _sparse_mixers(self):
         return [layer.mixer for layer in self.transformer.layers if isinstance(layer.mixer, ParallelMHASparseAttMlp)]
 
-    def _decode_step(self, cache: _DecodingCache, vocab_size: Optional[int]):
-        """One token: forward at the device-resident position, argmax, bookkeeping.
-        Everything is enqueued; nothing is read back."""
-        logits = self(cache.token, position_ids=cache.position, inference_params=cache.inference_params).logits[:, -1]
-        if vocab_size is not None:
-            logits = logits[..., :vocab_size]
-        ops.greedy_advance(logits[0].contiguous(), cache.token, cache.position, cache.seq_pos, cache.sequences,
-                           cache.out_index, cache.scores, cache.score_index)
+    def max_positions(self):
+        return self.transformer.embeddings.max_position_embeddings
 
-    @torch.no_grad()
-    def generate(self, input_ids, max_length, top_k=1, top_p=0.0, temperature=1.0, fused_ft_kernel=True, cg=False,
-                 vocab_size=None, return_dict_in_generate=False, output_scores=False, timing=False, **kwargs):
-        """Greedy decoding of ``max_length - input_ids.shape[1]`` tokens (batch 1).
+    def vocab_rows(self):
+        return self.lm_head.weight.shape[0]
 
-        Returns the (1, max_length) sequences, or GreedySearchDecoderOnlyOutput(sequences,
-        scores) with ``return_dict_in_generate``; scores is a (new tokens, vocab) tensor
-        when ``output_scores``."""
-        assert top_k == 1 and top_p == 0.0, "greedy decoding only"
-        assert fused_ft_kernel, "the decode kernels work on the packed cache layouts"
-        batch_size, seqlen_og = input_ids.shape
-        assert batch_size == 1, "head-sparse decoding keeps one back-fill window: batch size 1"
-        assert seqlen_og < max_length <= self.transformer.embeddings.max_position_embeddings
-        device, dtype = input_ids.device, self.lm_head.weight.dtype
-        cache = self._decoding_cache
-        if cache is None or cache.max_length != max_length:
-            cache = self._decoding_cache = _DecodingCache(self, max_length, device, dtype)
-        n_new = max_length - seqlen_og
-        vocab = self.lm_head.weight.shape[0] if vocab_size is None else vocab_size
-        if output_scores and (cache.scores is None or cache.scores.shape != (max_length, vocab)):
-            # sized for the longest run so that captured steps do not depend on the prompt length
-            cache.scores = torch.zeros(max_length, vocab, dtype=dtype, device=device)
-            cache.graphs.clear()
-        elif not output_scores and cache.scores is not None:
-            cache.scores = None
-            cache.graphs.clear()
-        if getattr(cache, "graph_key", None) != (vocab_size, bool(output_scores)):
-            cache.graphs.clear()  # captured steps hold the logits slice and the score buffer of their run
-            cache.graph_key = (vocab_size, bool(output_scores))
-        ip = cache.inference_params
+    @property
+    def score_dtype(self):
+        return self.lm_head.weight.dtype
 
-        # prompt: dense, fills the caches
-        ip.sequence_len_offset = 0
-        ip.lengths_per_sample = None
-        logits = self(input_ids, inference_params=ip, last_token_only=True).logits[:, -1]
-        if vocab_size is not None:
-            logits = logits[..., :vocab_size]
-        cache.sequences[:, :seqlen_og] = input_ids
-        next_token = logits.argmax(dim=-1, keepdim=True)
-        cache.token.copy_(next_token)
-        cache.sequences[:, seqlen_og:seqlen_og + 1] = next_token
-        if cache.scores is not None:
-            cache.scores[0] = logits[0]
-        cache.position.fill_(seqlen_og)
-        cache.seq_pos.fill_(seqlen_og)
-        cache.out_index.fill_(seqlen_og + 1)
-        cache.score_index.fill_(1)
-        ip.sequence_len_offset = seqlen_og
-        ip.lengths_per_sample = cache.seq_pos
+    def advance(self, logits_row, cache):
+        ops.greedy_advance(logits_row, cache.token, cache.position, cache.seq_pos, cache.sequences, cache.out_index,
+                           cache.scores, cache.score_index)
 
-        mixers = self._sparse_mixers()
-        window = ParallelMHASparseAttMlp.WINDOW
-        total = n_new - 1
-        step = 0
-        while step < total:
-            c = step % window  # position inside the back-fill window (== every sparse mixer's counter)
-            if cg and c == 0 and total - step >= window and (step >= window or "window" in cache.graphs):
-                # A whole back-fill window (16 tokens) is one graph: the gap between two graph
-                # launches is paid once per window instead of once per token.  Captured once every
-                # position has run eagerly (workspaces exist then); nothing in it depends on the
-                # host: token, position and sequence length live on the device.
-                if "window" not in cache.graphs:
-                    offset = ip.sequence_len_offset
-                    g = torch.cuda.CUDAGraph()
-                    with torch.cuda.graph(g):
-                        for _ in range(window):
-                            self._decode_step(cache, vocab_size)
-                            dv_modules.join_side_stream()
-                            ip.sequence_len_offset += 1
-                    ip.sequence_len_offset = offset
-                    cache.graphs["window"] = g
-                    cache.counters_after["window"] = [m.counter for m in mixers]
-                cache.graphs["window"].replay()
-                for m, v in zip(mixers, cache.counters_after["window"]):
-                    m.counter = v
-                ip.sequence_len_offset += window
-                step += window
-                continue
-            if cg and (step >= window or c in cache.graphs):
-                # a window position is captured once it has run eagerly (workspaces exist then);
-                # later generations replay the graphs from their first decode step on
-                if c not in cache.graphs:
-                    g = torch.cuda.CUDAGraph()
-                    with torch.cuda.graph(g):
-                        self._decode_step(cache, vocab_size)
-                        dv_modules.join_side_stream()
-                    cache.graphs[c] = g
-                    cache.counters_after[c] = [m.counter for m in mixers]
-                cache.graphs[c].replay()
-                for m, v in zip(mixers, cache.counters_after[c]):
-                    m.counter = v
-            else:
-                self._decode_step(cache, vocab_size)
-            ip.sequence_len_offset += 1
-            step += 1
-        sequences = cache.sequences.clone()
-        if return_dict_in_generate:
-            return GreedySearchDecoderOnlyOutput(sequences=sequences,
-                                                 scores=None if cache.scores is None else cache.scores[:n_new].clone())
-        return sequences
+    def host_state(self):
+        return [m.counter for m in self._sparse_mixers()]
+
+    def set_host_state(self, state):
+        for m, v in zip(self._sparse_mixers(), state):
+            m.counter = v
+
+    def end_of_step(self):
+        dv_modules.join_side_stream()

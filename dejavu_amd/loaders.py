@@ -1,4 +1,4 @@
-"""Checkpoint formats: HuggingFace OPT weights and trained sparsity predictors.
+"""Checkpoint formats: HuggingFace OPT weights, trained sparsity predictors, Vimulorn weights.
 
 Mirrors what the reference does before ``model.load_state_dict``
 (Dejavu/src/utils/dejavu_util.py:12-234 ``remap_state_dict_opt`` / ``shard_state_dict_tp``,
@@ -11,6 +11,7 @@ Decentralized_FM_alpha/modules/hf_opt_sparse_mlp_attention.py:430-445), which be
 from __future__ import annotations
 
 import math
+import os
 import re
 from collections import OrderedDict
 from typing import Mapping, Optional, Sequence
@@ -141,3 +142,103 @@ def add_predictors(state_dict: dict, mlp_predictors: Optional[Sequence] = None,
 def load_checkpoint_file(path: str) -> dict:
     """Reads a tensor-only checkpoint without executing anything stored in the file."""
     return torch.load(path, map_location="cpu", weights_only=True)
+
+
+def load_checkpoint_folder(folder: str) -> dict:
+    """The tensors of a model folder: model.safetensors, else pytorch_model.bin."""
+    path = os.path.join(folder, "model.safetensors")
+    if os.path.exists(path):
+        from safetensors.torch import load_file
+
+        return load_file(path)
+    return load_checkpoint_file(os.path.join(folder, "pytorch_model.bin"))
+
+
+# ---- Vimulorn ---------------------------------------------------------------------
+def _pad(x: torch.Tensor, *sizes: int) -> torch.Tensor:
+    """Zero padding at the end of the leading dimensions up to ``sizes``."""
+    out = x.new_zeros(*sizes, *x.shape[len(sizes):])
+    out[tuple(slice(0, n) for n in x.shape[:len(sizes)])] = x
+    return out
+
+
+def remap_state_dict_vimulorn(state_dict: Mapping[str, torch.Tensor], config) -> "OrderedDict[str, torch.Tensor]":
+    """Vimulorn checkpoint names -> parameters of ``dejavu_amd.hybrid.HybridLMHeadModel``.
+
+    * the projections that read a mixer's input become one matrix (rows in the order the mixer documents), the short
+      convolutions of q, k, v one table; gate and up rows of the feed-forward alternate
+    * every size along a vectorised dimension is padded to a multiple of 8 with zeros, per head where there are heads
+    """
+    from .mixer_ops import padded
+
+    t = dict(state_dict)
+    out: "OrderedDict[str, torch.Tensor]" = OrderedDict()
+    width = config.width
+    ws = padded(width)
+
+    def cols(x):  # an input of the model's width
+        return _pad(x.t(), ws).t()
+
+    def head_rows(x, heads, dim):  # (heads * dim, ...) -> rows padded per head
+        return _pad(x.reshape(heads, dim, *x.shape[1:]), heads, padded(dim)).reshape(heads * padded(dim), *x.shape[1:])
+
+    def head_cols(x, heads, dim):
+        return head_rows(x.t(), heads, dim).t()
+
+    def norm(src, dst):
+        out[dst + ".weight"] = _pad(t.pop(src).float(), ws)
+        out[dst + ".bias"] = _pad(t.pop(src + ".b").float(), ws)
+        out[dst + ".alpha"] = t.pop(src + ".alpha").float().reshape(1)
+
+    def conv(parts):  # tables of (channels, taps); the newest token's tap is the last one
+        taps = max(p.shape[1] for p in parts)
+        return torch.cat([F.pad(p.float(), (taps - p.shape[1], 0)) for p in parts])
+
+    out["embeddings"] = cols(t.pop("embed"))
+    out["lm_head"] = cols(t.pop("head"))
+    norm("final.norm", "final_norm")
+    for i, spec in enumerate(config.layers):
+        src, dst, m = f"l{i}.", f"layers.{i}.", spec.mixer
+
+        def take(name, src=src):
+            return t.pop(src + "mix." + name)
+
+        norm(src + "norm1", dst + "norm1")
+        norm(src + "norm1b", dst + "norm1b")
+        H, dim, vdim, mix = m["heads"], m["dim"], m["vdim"], dst + "mixer."
+        if spec.type == "latent_attention":
+            qr, kr = padded(m["q_rank"]), padded(m["kv_rank"])
+            out[mix + "in_proj"] = cols(torch.cat([_pad(take("dq"), qr), _pad(take("dkv"), kr), _pad(take("g"), padded(H))]))
+            out[mix + "q_norm"] = _pad(take("dq.norm").float(), qr)
+            out[mix + "kv_norm"] = _pad(take("dkv.norm").float(), kr)
+            out[mix + "q_up"] = _pad(head_rows(take("uq"), H, dim).t(), qr).t()
+            out[mix + "k_up"] = _pad(head_rows(take("uk"), H, dim).t(), kr).t()
+            out[mix + "v_up"] = _pad(head_rows(take("uv"), H, vdim).t(), kr).t()
+        elif spec.type == "attention":
+            G = m["kv_heads"]
+            groups = (("q", H, dim), ("k", G, dim), ("v", G, vdim))
+            out[mix + "in_proj"] = cols(torch.cat([head_rows(take(n), h, d) for n, h, d in groups]))
+            out[mix + "conv"] = conv([head_rows(take(n + ".conv"), h, d) for n, h, d in groups])
+            out[mix + "sink"] = take("sink").float()
+        else:
+            G, ra, rg = m["kv_heads"], padded(m["decay_rank"]), padded(m["gate_rank"])
+            groups = (("q", G, dim), ("k", G, dim), ("v", H, vdim))
+            out[mix + "in_proj"] = cols(torch.cat([head_rows(take(n), h, d) for n, h, d in groups] +
+                                                  [_pad(take("b"), padded(H)), _pad(take("a1"), ra), _pad(take("g1"), rg)]))
+            out[mix + "conv"] = conv([head_rows(take(n + ".conv"), h, d) for n, h, d in groups])
+            out[mix + "decay_up"] = _pad(head_rows(take("a2"), H, dim).t(), ra).t()
+            out[mix + "gate_up"] = _pad(head_rows(take("g2"), H, vdim).t(), rg).t()
+            out[mix + "A_log"] = take("A_log").float()
+            out[mix + "dt_bias"] = head_rows(take("dt_bias").float(), H, dim)
+            out[mix + "norm"] = _pad(take("norm").float(), padded(vdim))
+        out[mix + "out_proj"] = _pad(head_cols(take("o"), H, vdim), ws)
+        if spec.mlp is not None:
+            norm(src + "norm2", dst + "norm2")
+            norm(src + "norm2b", dst + "norm2b")
+            fs = padded(spec.mlp["ff"])
+            gate, up = (_pad(cols(t.pop(f"{src}mlp.{n}")), fs) for n in ("gate", "up"))
+            out[dst + "mlp.gate_up"] = torch.stack([gate, up], dim=1).reshape(2 * fs, ws)
+            out[dst + "mlp.down"] = _pad(_pad(t.pop(f"{src}mlp.down"), ws).t(), fs).t()
+    for name in t:  # what is left has no place in this family: reported by the caller
+        out[name] = t[name]
+    return out

@@ -16,7 +16,6 @@ the library GEMM / attention of PyTorch, as the reference's do through cuBLAS.
 """
 from __future__ import annotations
 
-from dataclasses import dataclass, field
 from typing import Optional
 
 import torch
@@ -25,6 +24,7 @@ import torch.nn.functional as F
 
 from . import ops
 from ._lib import check, lib
+from .inference import InferenceParams  # noqa: F401  (part of this module's interface)
 
 
 # Side-stream overlap of predictor / top-k work with the main kernels (the reference's
@@ -129,20 +129,6 @@ def _world_size(process_group) -> int:
     if size != 1:
         raise NotImplementedError("this build runs the sparse decode path on one GPU (tensor parallel size 1)")
     return size
-
-
-@dataclass
-class InferenceParams:
-    """Decode-time state shared by the layers (same fields as the
-    ``inference_params`` object the reference's modules read)."""
-
-    max_sequence_len: int
-    max_batch_size: int
-    sequence_len_offset: int = 0
-    batch_size_offset: int = 0
-    key_value_memory_dict: dict = field(default_factory=dict)
-    fused_ft_kernel: bool = True
-    lengths_per_sample: Optional[torch.Tensor] = None
 
 
 class ParallelSP(nn.Module):
