@@ -641,6 +641,275 @@ def mlp_bench(args):
         "batches": results}))
 
 
+def vimulorn_kernels(torch, model, prompt, context):
+    """Every kernel of the design at the sizes of ``model`` beside the like kernel of the OPT layers at the same sizes:
+    time per launch (HIP graph of launches over several sets of weights, so that no cache holds them), the bytes or
+    flops that have to be moved or done, and the fraction of the peak.  ``like``: the OPT side."""
+    import torch.nn.functional as F
+
+    from dejavu_amd import mixer_ops as mo
+    from dejavu_amd import ops
+    from dejavu_amd.mixers import ChannelDelta, LatentAttention, StepInfo, WindowAttention
+
+    dev, bf, table = "cuda", torch.bfloat16, {}
+    width = model.embeddings.shape[1]
+    gen = torch.Generator(device=dev)
+    gen.manual_seed(3)
+
+    def rnd(*shape, dtype=bf):
+        return torch.randn(*shape, dtype=torch.float32, device=dev, generator=gen).to(dtype)
+
+    def copies(W, least=600e6):
+        count = max(2, min(24, int(least // (W.numel() * W.element_size())) + 1))
+        return [W.detach().clone() for _ in range(count)]
+
+    def put(name, us, like_us, nbytes=0, flops=0, like=None, like_bytes=None, like_flops=None):
+        def entry(t, b, f):
+            e = {"us": round(t, 2)}
+            if f:
+                e.update(TFLOPS=round(f / t / 1e6, 1), frac=round(f / t / 1e6 / MFMA_PEAK_TFLOPS, 4))
+            else:
+                e.update({"GB/s": round(b / t / 1e3, 1), "frac": round(b / t / 1e3 / HBM_PEAK_GBPS, 4)})
+            return e
+        row = entry(us, nbytes, flops)
+        if like_us is not None:
+            row["like"] = dict(entry(like_us, like_bytes or nbytes, like_flops if like_flops is not None else flops), kernel=like)
+        table[name] = row
+
+    def norm_stream(n):
+        return mo.ResidualStream(rnd(n, width, dtype=torch.float32), None, bf)
+
+    norm = model.final_norm
+    by_type = {}
+    for layer in model.layers:
+        by_type.setdefault(type(layer.mixer), layer)
+    lat, dlt, win = (by_type[t].mixer for t in (LatentAttention, ChannelDelta, WindowAttention))
+    mlp = by_type[LatentAttention].mlp
+
+    # ---- one token: products ----
+    def row_product(name, W, fn, x=None):
+        Ws = copies(W)
+        us = time_kernel(torch, fn, Ws)
+        xh = rnd(1, W.shape[1], dtype=torch.float16)
+        Wh = [w.half() for w in Ws]
+        like_us = time_kernel(torch, lambda w: ops.gather_gemv(xh, w, None, None, "relu"), Wh)
+        put(name, us, like_us, nbytes=W.numel() * 2, like="gather_rows_kernel, all rows")
+
+    x1, xf = rnd(1, width), rnd(1, mlp.down.shape[1])
+    s1 = norm_stream(1)
+    wst = win.new_state(context)
+    row_product("decode: projections + short convolution", win.in_proj,
+                lambda w: mo.row_conv(x1, w, win.conv, wst["conv"], False))
+    row_product("decode: latent projections", lat.in_proj, lambda w: mo.linear(x1, w, f32=True))
+    xq = rnd(1, lat.in_proj.shape[0], dtype=torch.float32)
+    row_product("decode: RMS norm + query up-projection", lat.q_up,
+                lambda w: mo.row_rms_linear(xq, lat.q_norm, lat.q_rank, 1e-5, w))
+    row_product("decode: gate / up + clamped gated unit", mlp.gate_up, lambda w: mo.clamped_glu(x1, w, 7.0))
+    row_product("decode: down + norm + residual + norm", mlp.down, lambda w: mo.linear_residual(xf, w, s1, norm, norm))
+    xo = rnd(1, win.out_proj.shape[1])
+    row_product("decode: output projection + norm + residual + norm", win.out_proj,
+                lambda w: mo.linear_residual(xo, w, s1, norm, norm))
+    go, gg = rnd(1, dlt.out_proj.shape[1], dtype=torch.float32), torch.rand(dlt.out_proj.shape[1], device=dev)
+    gh = mo.GatedHeads(go, gg, dlt.norm, dlt.vdim, 1e-5)
+    row_product("decode: gated head norm + output projection + norm + residual + norm", dlt.out_proj,
+                lambda w: gh.linear_residual(w, s1, norm, norm))
+    row_product("decode: head", model.lm_head, lambda w: mo.linear(x1, w, f32=True))
+
+    # ---- one token: attention and delta rule ----
+    def like_attention(nbytes):
+        H, hd = 32, 128
+        S = max(64, int(nbytes // (H * hd * 4)) // 64 * 64)
+        caches = [(rnd(1, H, hd // 8, S, 8, dtype=torch.float16), rnd(1, H, S, hd, dtype=torch.float16))
+                  for _ in range(max(2, min(24, int(600e6 // nbytes))))]
+        q = rnd(1, H, hd, dtype=torch.float16)
+        us = time_kernel(torch, lambda c: ops.single_query_attention(q, None, None, c[0], c[1], None, S - 1), caches)
+        return us, H * hd * S * 4
+
+    q = rnd(1, lat.heads * lat.dim_s, dtype=torch.float32)
+    gate = rnd(lat.heads, dtype=torch.float32)
+    for ctx in (context, 8 * context):
+        nb = ctx * lat.kv_rank_s * 2 + (lat.k_up.numel() + lat.v_up.numel()) * 2
+        sets = [(rnd(ctx, lat.kv_rank_s), lat.k_up.clone(), lat.v_up.clone()) for _ in range(max(2, min(24, int(600e6 // nb))))]
+        us = time_kernel(torch, lambda c: mo.latent_attention_row(q, c[1], c[2], c[0], lat.heads, lat.scale, gate, None, ctx - 1), sets)
+        like_us, like_b = like_attention(nb)
+        put(f"decode: latent attention with up-projections, {ctx} tokens", us, like_us, nbytes=nb,
+            like="decode_attn_kernel of the same bytes", like_bytes=like_b)
+    row = rnd(1, win.channels, dtype=torch.float32)
+    wst = [win.new_state(context) for _ in range(24)]
+    nb = (wst[0]["k"].numel() + wst[0]["v"].numel()) * 2
+    us = time_kernel(torch, lambda st: mo.window_attention_row(row, st["k"], st["v"], win.heads, win.kv_heads, win.dim,
+                                                               win.scale, 1e-5, win.sink, win.window, None, context - 1), wst)
+    like_us, like_b = like_attention(nb)
+    put(f"decode: windowed attention, window {win.window}", us, like_us, nbytes=nb,
+        like="decode_attn_kernel of the same bytes", like_bytes=like_b)
+    row = rnd(1, dlt.in_proj.shape[0], dtype=torch.float32)
+    dst = [(dlt.new_state(1)["S"], dlt.decay_up.clone(), dlt.gate_up.clone()) for _ in range(24)]
+    nb = dst[0][0].numel() * 8 + (dlt.decay_up.numel() + dlt.gate_up.numel()) * 2
+    us = time_kernel(torch, lambda st: mo.delta_row(row, dlt.offsets, dlt.heads, dlt.kv_heads, dlt.dim, st[1], st[2],
+                                                    dlt.A_log, dlt.dt_bias, st[0]), dst)
+    like_us, like_b = like_attention(nb)
+    put("decode: delta rule step with its low-rank products", us, like_us, nbytes=nb,
+        like="decode_attn_kernel of the same bytes", like_bytes=like_b)
+
+    # ---- portions: products of a few rows ----
+    for n in (16, 64):
+        for name, W, fn in (("gate / up + clamped gated unit", mlp.gate_up, lambda xx, w: mo.clamped_glu(xx, w, 7.0)),
+                            ("plain product", win.in_proj, lambda xx, w: mo.linear(xx, w))):
+            xn, xh = rnd(n, width), rnd(n, width, dtype=torch.float16)
+            Ws = copies(W)
+            us = time_kernel(torch, lambda w: fn(xn, w), Ws)
+            Wh = [w.half() for w in Ws]
+            like_us = time_kernel(torch, lambda w: ops.dense_linear(xh, w), Wh)
+            put(f"portion of {n}: {name}", us, like_us, nbytes=W.numel() * 2, like="gemm_tiled_mfma_kernel")
+
+    # ---- prompt ----
+    n, H, hd = prompt, lat.heads, lat.dim_s
+    qkv = [rnd(n, H * hd) for _ in range(3)]
+    causal = 2.0 * H * hd * n * n  # two products over half the pairs
+    us = time_kernel(torch, lambda a: mo.portion_attention(qkv[0], qkv[1], qkv[2], H, H, lat.scale, 0, 0, gate=qkv[0]), [0], launches=10)
+    qh = [rnd(1, H, n, hd, dtype=torch.float16) for _ in range(3)]
+    like_us = time_kernel(torch, lambda a: F.scaled_dot_product_attention(*qh, is_causal=True), [0], launches=10)
+    put(f"prompt of {n}: latent attention (keys and values expanded)", us, like_us, flops=causal,
+        like="library attention, the OPT layers' above 192 tokens")
+    G, W = win.kv_heads, min(win.window, n)
+    pairs = W * n - W * (W - 1) / 2.0
+    kw, vw = rnd(n, G * hd), rnd(n, G * hd)
+    us = time_kernel(torch, lambda a: mo.portion_attention(qkv[0], kw, vw, H, G, win.scale, 0, 0, sink=win.sink, window=win.window), [0], launches=10)
+    put(f"prompt of {n}: windowed attention, window {win.window}", us, like_us, flops=4.0 * H * hd * pairs,
+        like="library attention, causal", like_flops=causal)
+    m = 160
+    qs = [rnd(m, H * hd) for _ in range(3)]
+    us = time_kernel(torch, lambda a: mo.portion_attention(qs[0], qs[1], qs[2], H, H, lat.scale, 0, 0), [0])
+    pq = rnd(1, m, 3, H, hd, dtype=torch.float16)
+    like_us = time_kernel(torch, lambda a: ops.prefill_attention(pq, None, None, 0, lat.scale), [0])
+    put(f"prompt of {m}: latent attention", us, like_us, flops=2.0 * H * hd * m * m, like="prefill_attn_kernel")
+
+    hh = rnd(n, width, dtype=torch.float16)
+    res, lw = rnd(n, width, dtype=torch.float16), torch.ones(width, dtype=torch.float16, device=dev)
+    like_us = time_kernel(torch, lambda a: ops.add_layer_norm(hh, res, lw, lw), [0])
+    like_b, like = n * width * 8, "add_layer_norm_kernel"
+
+    def elementwise(name, fn, nbytes):
+        put(f"prompt of {n}: {name}", time_kernel(torch, fn, [0]), like_us, nbytes=nbytes, like=like, like_bytes=like_b)
+
+    y, st = rnd(n, width), norm_stream(n)
+    elementwise("norm + residual + norm", lambda a: mo.residual(y, st, norm, norm), n * width * 12)
+    gu = rnd(n, mlp.gate_up.shape[0])
+    out = torch.empty(n, mlp.gate_up.shape[0] // 2, dtype=bf, device=dev)
+    elementwise("clamped gated unit", lambda a: mo.lib.dv_mix_clamped_glu(
+        0, gu.data_ptr(), out.numel(), 7.0, out.data_ptr(), mo._stream()), gu.numel() * 3)
+    p = rnd(n, win.channels)
+    k, v, qq = torch.empty(n, G * hd, dtype=bf, device=dev), torch.empty(n, G * hd, dtype=bf, device=dev), torch.empty(n, H * hd, dtype=bf, device=dev)
+    cst = win.new_state(context)["conv"]
+    elementwise("short convolution + head RMS norm", lambda a: mo.short_conv(
+        p, win.conv, cst, [(H, hd, hd, 1, 1e-5, 1.0, qq), (G, hd, hd, 1, 1e-5, 1.0, k), (G, hd, hd, 0, 0.0, 1.0, v)], False),
+        n * win.channels * 4)
+    ck = rnd(n, lat.in_proj.shape[0])
+    elementwise("latent RMS norm", lambda a: mo.rms_rows(ck[:, :lat.q_rank_s], lat.q_norm, lat.q_rank, 1e-5), n * lat.q_rank_s * 4)
+    dh, dg, dv_, ds = dlt.heads, dlt.kv_heads, dlt.vdim_s, dlt.dim_s
+    f32 = torch.float32
+    q, k2 = (F.normalize(rnd(n * dg, ds, dtype=f32), dim=-1).view(n, dg * ds) for _ in range(2))
+    v = rnd(n, dh * dv_, dtype=f32)
+    z, b = rnd(n, dh * ds), rnd(n, 64)
+    g, beta = mo.delta_gates(z, b, dlt.A_log, dlt.dt_bias, dh)
+    elementwise("decays of the delta rule", lambda a: mo.delta_gates(z, b, dlt.A_log, dlt.dt_bias, dh), n * dh * ds * 6)
+    S = dlt.new_state(1)["S"]
+    o = mo.delta_scan(q, k2, v, g, beta, S, dh, dg)
+    elementwise("delta rule scan", lambda a: mo.delta_scan(q, k2, v, g, beta, S, dh, dg),
+                4 * (2 * n * dg * ds + 2 * n * dh * dv_ + n * dh * ds))
+    gt = rnd(n, dh * dv_)
+    elementwise("gated head norm", lambda a: mo.gated_head_norm(o, gt, dlt.norm, dv_, 1e-5), n * dh * dv_ * 8)
+    return table
+
+
+def vimulorn_bench(args):
+    """Vimulorn at the layer sizes of real models (random weights): prompt and decode throughput beside an OPT-shaped
+    sparse model of the same width, layers and feed-forward weights, and every kernel beside its like.  A step is one
+    generated token; prints its own JSON line."""
+    import torch
+
+    from dejavu_amd.block import init_block_synthetic
+    from dejavu_amd.gpt import GPTLMHeadModel, SparseGPTConfig
+    from dejavu_amd.hybrid import HybridConfig, HybridLMHeadModel
+    from dejavu_amd.workloads import VIMULORN_CONFIGS, init_vimulorn_synthetic
+
+    torch.cuda.set_device(0)
+    new_tokens, decode_prompt = args.steps, 1024
+    prompts = (128, 2048, 8192)
+
+    def throughput(model, vocab, prompts):
+        ids = torch.randint(0, vocab, (1, max(prompts + (decode_prompt,))), device="cuda")
+
+        def run(n, length, cg):
+            torch.cuda.synchronize()
+            t0 = time.perf_counter()
+            model.generate(ids[:, :n], max_length=length, cg=cg)
+            torch.cuda.synchronize()
+            return time.perf_counter() - t0
+
+        length = decode_prompt + new_tokens
+        for _ in range(max(1, args.warmup)):
+            run(decode_prompt, length, True)
+        total = min(run(decode_prompt, length, True) for _ in range(3))
+        out = {"prompt_ms": {}, "prompt_tokens_per_s": {}}
+        for n in prompts:
+            run(n, n + 1, False)
+            t = min(run(n, n + 1, False) for _ in range(3))
+            out["prompt_ms"][str(n)] = round(t * 1e3, 3)
+            out["prompt_tokens_per_s"][str(n)] = round(n / t)
+        run(decode_prompt, decode_prompt + 1, False)
+        t_prompt = min(run(decode_prompt, decode_prompt + 1, False) for _ in range(3))
+        out["decode_tokens_per_s"] = round((new_tokens - 1) / (total - t_prompt), 1)
+        out["decode_ms_per_token"] = round((total - t_prompt) / (new_tokens - 1) * 1e3, 4)
+        return out
+
+    results = {}
+    with torch.no_grad():
+        for name in args.vimulorn:
+            cfg = VIMULORN_CONFIGS[name]
+            model = HybridLMHeadModel(HybridConfig.from_dict(cfg), device="cuda", dtype=torch.bfloat16).eval()
+            init_vimulorn_synthetic(model, 1)
+            r = throughput(model, cfg["vocab"], prompts)
+            runs = [model.layers[i] for i, _ in model.runs]
+            nbytes = model.lm_head.numel() * 2 + sum(
+                p.numel() * 2 for layer in runs for p in layer.parameters() if p.dtype == torch.bfloat16)
+            r["weight_MB_per_token"] = round(nbytes / 1e6, 1)
+            r["weight_frac_of_hbm_peak"] = round(nbytes / r["decode_ms_per_token"] / 1e6 / HBM_PEAK_GBPS, 4)
+            if not args.no_kernels:
+                r["kernels"] = vimulorn_kernels(torch, model, 2048, 4096)
+            width, layers = cfg["width"], len(runs)
+            del model, runs
+            ffn, heads = 4 * width, width // 128
+            conf = SparseGPTConfig(hidden_size=width, num_attention_heads=heads, num_hidden_layers=layers,
+                                   vocab_size=cfg["vocab"], n_inner=ffn, max_position_embeddings=8448, mlp_K=ffn // 4,
+                                   mlp_sp_dim=1000, att_K=[heads // 2, heads // 2], att_sp_dim=1000)
+            opt = GPTLMHeadModel(conf, device="cuda", dtype=torch.float16).eval()
+            for l, blk in enumerate(opt.transformer.layers):
+                init_block_synthetic(blk, seed=100 + l)
+            for emb in (opt.transformer.embeddings.word_embeddings, opt.transformer.embeddings.position_embeddings):
+                emb.weight.normal_(0.0, 0.02)
+            opt.tie_weights()
+            o = throughput(opt, cfg["vocab"], prompts)
+            d, hd, K, Hk, rk = width, 128, ffn // 4, heads // 2, 1000
+            pred = (2 * d * rk + rk * ffn + rk * heads) * 2
+            nb = (4 * d * d + 2 * d * ffn) * 2 + pred + (layers - 1) * ((4 * Hk * hd * d + 2 * K * d) * 2 + pred) + cfg["vocab"] * d * 2
+            o["weight_MB_per_token"] = round(nb / 1e6, 1)
+            o["weight_frac_of_hbm_peak"] = round(nb / o["decode_ms_per_token"] / 1e6 / HBM_PEAK_GBPS, 4)
+            o["shape"] = f"{layers} blocks, first dense, {K} of {ffn} neurons, {Hk} of {heads} heads"
+            r["opt_of_equal_size"] = o
+            results[name] = r
+            del opt
+            torch.cuda.empty_cache()
+    lead = results[args.vimulorn[0]]
+    print(json.dumps({
+        "metric": f"tokens_per_s, greedy decode, {args.vimulorn[0]}, batch 1", "value": lead["decode_tokens_per_s"],
+        "unit": "tokens/s", "n_gpus": 1, "steps": new_tokens, "warmup": args.warmup,
+        "ms_per_step": lead["decode_ms_per_token"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+        "dtype": "bf16", "data": "synthetic", "config": {"workload": "vimulorn", "models": args.vimulorn,
+                                                        "decode_prompt": decode_prompt, "prompts": prompts},
+        "models": results}))
+
+
 def holds_gpu():
     """True when this process already has the GPU's device node open (the compute driver's /dev/kfd)."""
     try:
@@ -759,9 +1028,13 @@ def main():
                     help="batch sizes of --workload mlp")
     ap.add_argument("--K", type=int, default=None,
                     help="--workload mlp: active neurons (default: the configuration's K; K = ffn is the dense block)")
-    ap.add_argument("--workload", default="layer", choices=["layer", "decode", "mlp"],
+    ap.add_argument("--workload", default="layer", choices=["layer", "decode", "mlp", "vimulorn"],
                     help="layer: the headline sparse decode layer; decode: end-to-end greedy generation "
-                         "(40-layer OPT-13B shape, --steps = new tokens, default 256)")
+                         "(40-layer OPT-13B shape, --steps = new tokens, default 256); vimulorn: prompt and decode "
+                         "throughput and the kernels of Vimulorn models beside OPT ones of equal size")
+    ap.add_argument("--vimulorn", nargs="+", default=["vimulorn-4k", "vimulorn-2k"],
+                    help="model sizes of --workload vimulorn (workloads.VIMULORN_CONFIGS)")
+    ap.add_argument("--no-kernels", action="store_true", help="--workload vimulorn: throughput only")
     ap.add_argument("--decode-layers", type=int, default=40)
     ap.add_argument("--no-other-workloads", action="store_true",
                     help="default run only: skip the batched-layer (batch 8 / 16 / 32) and greedy-decode legs")
@@ -795,6 +1068,10 @@ def main():
     from dejavu_amd.workloads import CONFIGS
 
     dv_modules.USE_SIDE_STREAM = args.side_stream
+    if args.workload == "vimulorn":
+        args.steps = 256 if args.steps is None else args.steps
+        args.warmup = 1 if args.warmup is None else args.warmup
+        return vimulorn_bench(args)
     if args.workload == "decode":
         args.steps = 256 if args.steps is None else args.steps
         args.warmup = 1 if args.warmup is None else args.warmup

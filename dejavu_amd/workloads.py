@@ -68,3 +68,46 @@ def pack_k_cache(k_bhsd: torch.Tensor) -> torch.Tensor:
     """(B, H, S, hd) -> (B, H, hd/8, S, 8), the packed key-cache layout."""
     B, H, S, hd = k_bhsd.shape
     return k_bhsd.view(B, H, S, hd // 8, 8).permute(0, 1, 3, 2, 4).contiguous()
+
+
+# Vimulorn decoders with the layer sizes of real models: [latent attention, delta rule, windowed attention] twice, the
+# second three run twice (nine layer runs)
+def vimulorn_config(width: int, ff: int, heads: int, q_rank: int, kv_rank: int, window: int, vocab: int = 32768) -> dict:
+    hd = 128
+    mlp = {"kind": "dense", "ff": ff, "limit": 7.0}
+    trio = [
+        {"type": "latent_attention", "mlp": mlp,
+         "mixer": dict(heads=heads, dim=hd, vdim=hd, q_rank=q_rank, kv_rank=kv_rank, scale=hd ** -0.5)},
+        {"type": "channel_delta", "mlp": mlp,
+         "mixer": dict(heads=heads, kv_heads=heads // 2, dim=hd, vdim=hd, conv=4, decay_rank=hd, gate_rank=hd)},
+        {"type": "attention", "mlp": mlp,
+         "mixer": dict(heads=heads, kv_heads=heads // 4, dim=hd, vdim=hd, conv=4, mask={"size": window},
+                       scale=hd ** -0.5)}]
+    return {"architecture": "Vimulorn", "width": width, "vocab": vocab, "norm": {"eps": 1e-5}, "layers": trio * 2,
+            "loop": {"start": 3, "stop": 6, "times": 2}}
+
+
+VIMULORN_CONFIGS = {
+    "vimulorn-4k": vimulorn_config(4096, 11008, 32, 1536, 512, 1024),
+    "vimulorn-2k": vimulorn_config(2048, 5632, 16, 768, 256, 512),
+}
+
+
+@torch.no_grad()
+def init_vimulorn_synthetic(model, seed: int = 0) -> None:
+    """Seeded random weights in place: matrices ~ N(0, 1 / columns), norm weights 1, everything else small."""
+    dev = next(model.parameters()).device
+    gen = torch.Generator(device=dev)
+    gen.manual_seed(seed)
+    for name, p in model.named_parameters():
+        tmp = torch.empty(p.shape, dtype=torch.float32, device=dev)
+        leaf = name.rsplit(".", 1)[-1]
+        if leaf in ("weight", "norm", "q_norm", "kv_norm"):
+            tmp.fill_(1.0)
+        elif leaf == "alpha":
+            tmp.fill_(0.5)
+        elif leaf == "A_log":
+            tmp.fill_(-2.0)
+        else:
+            tmp.normal_(0.0, p.shape[-1] ** -0.5 if p.dim() == 2 else 0.1, generator=gen)
+        p.copy_(tmp)
