@@ -64,7 +64,7 @@ SIGNATURES = {
     "dv_mix_attn_rows": (_i, [_i, _i, _P(AttnArgs), _p]),
     "dv_mix_attn_tiles": (_i, [_P(AttnArgs), _i, _p]),
     "dv_mix_latent_absorb": (_i, [_i, _p, _p, _i, _i, _i, _p, _p]),
-    "dv_mix_latent_attn": (_i, [_i, _P(AttnArgs), _p, _i, _p, _p]),
+    "dv_mix_latent_attn": (_i, [_i, _P(AttnArgs), _p, _p, _i, _p, _p]),
     "dv_mix_delta_gates": (_i, [_i, _p, _l, _p, _l, _p, _p, _i, _i, _i, _p, _p, _p]),
     "dv_mix_delta_scan": (_i, [_P(DeltaArgs), _p]),
     "dv_mix_delta_step": (_i, [_i, _P(DeltaStepArgs), _p]),

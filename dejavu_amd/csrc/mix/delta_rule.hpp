@@ -12,32 +12,45 @@
 
 namespace dv {
 
-// The state of a lane: E key channels of one column.
+// What a lane needs of one token: its E key channels of q, k and the decays, and the scalars of its column.
 template <int E>
-__device__ __forceinline__ float delta_step(float (&S)[E], const float* __restrict__ q, const float* __restrict__ k,
-                                            const float* __restrict__ g, int sub, float v, float beta, float kq) {
-  float dk[4] = {0.f, 0.f, 0.f, 0.f}, dq[4] = {0.f, 0.f, 0.f, 0.f};
-  float4_t kv[E / 4];
+struct DeltaToken {
+  float4_t q[E / 4], k[E / 4], g[E / 4];
+  float v, beta, kq;
+  __device__ __forceinline__ void load(const float* qp, const float* kp, const float* gp, int sub, float v_, float beta_,
+                                       float kq_) {
 #pragma unroll
-  for (int c = 0; c < E / 4; ++c) {
-    const float4_t gv = *reinterpret_cast<const float4_t*>(g + c * 64 + sub * 4);
-    const float4_t qv = *reinterpret_cast<const float4_t*>(q + c * 64 + sub * 4);
-    kv[c] = *reinterpret_cast<const float4_t*>(k + c * 64 + sub * 4);
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      S[c * 4 + e] *= gv[e];
-      dk[e] = __builtin_fmaf(S[c * 4 + e], kv[c][e], dk[e]);
-      dq[e] = __builtin_fmaf(S[c * 4 + e], qv[e], dq[e]);
+    for (int c = 0; c < E / 4; ++c) {
+      k[c] = *reinterpret_cast<const float4_t*>(kp + c * 64 + sub * 4);
+      g[c] = *reinterpret_cast<const float4_t*>(gp + c * 64 + sub * 4);
+      q[c] = *reinterpret_cast<const float4_t*>(qp + c * 64 + sub * 4);
     }
+    v = v_;
+    beta = beta_;
+    kq = kq_;
   }
-  const float sk = row16_sum((dk[0] + dk[1]) + (dk[2] + dk[3]));
-  const float sq = row16_sum((dq[0] + dq[1]) + (dq[2] + dq[3]));
-  const float u = beta * (v - sk);
+};
+
+// One token; S: the E key channels of the lane's column.  Returns the read-out of the column.
+template <int E>
+__device__ __forceinline__ float delta_step(float (&S)[E], const DeltaToken<E>& t) {
+  float dk[4] = {0.f, 0.f, 0.f, 0.f}, dq[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int c = 0; c < E / 4; ++c)
 #pragma unroll
-    for (int e = 0; e < 4; ++e) S[c * 4 + e] = __builtin_fmaf(kv[c][e], u, S[c * 4 + e]);
-  return __builtin_fmaf(kq, u, sq);
+    for (int e = 0; e < 4; ++e) {
+      S[c * 4 + e] *= t.g[c][e];
+      dk[e] = __builtin_fmaf(S[c * 4 + e], t.k[c][e], dk[e]);
+      dq[e] = __builtin_fmaf(S[c * 4 + e], t.q[c][e], dq[e]);
+    }
+  const float sk = row16_sum((dk[0] + dk[1]) + (dk[2] + dk[3]));
+  const float sq = row16_sum((dq[0] + dq[1]) + (dq[2] + dq[3]));
+  const float u = t.beta * (t.v - sk);
+#pragma unroll
+  for (int c = 0; c < E / 4; ++c)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) S[c * 4 + e] = __builtin_fmaf(t.k[c][e], u, S[c * 4 + e]);
+  return __builtin_fmaf(t.kq, u, sq);
 }
 
 using DeltaArgs = dvDeltaArgs;
@@ -134,15 +147,32 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaArgs a) {
     if (more) fetch(t0 + TC);
     const int cnt = a.n - t0 < TC ? a.n - t0 : TC;
     float mine = 0.f;  // lane s keeps the read-out of token s
-    auto token = [&](int t) {
-      const float o = delta_step<E>(S, sq[buf][t], sk[buf][t], sg[buf][t], sub, sv[buf][t][colw], sb[buf][t], skq[buf][t]);
+    DeltaToken<E> cur, nxt;
+    auto get = [&](DeltaToken<E>& d, int t) {
+      d.load(sq[buf][t], sk[buf][t], sg[buf][t], sub, sv[buf][t][colw], sb[buf][t], skq[buf][t]);
+    };
+    auto run = [&](const DeltaToken<E>& d, int t) {
+      const float o = delta_step<E>(S, d);
       if (sub == t) mine = o;
     };
-    if (cnt == TC) {
+    get(cur, 0);
+    if (cnt == TC) {  // the operands of a token are requested one token ahead
 #pragma unroll
-      for (int t = 0; t < TC; ++t) token(t);
+      for (int t = 0; t < TC; t += 2) {
+        get(nxt, t + 1);
+        __builtin_amdgcn_sched_barrier(0);
+        run(cur, t);
+        __builtin_amdgcn_sched_barrier(0);
+        if (t + 2 < TC) get(cur, t + 2);
+        __builtin_amdgcn_sched_barrier(0);
+        run(nxt, t + 1);
+        __builtin_amdgcn_sched_barrier(0);
+      }
     } else {
-      for (int t = 0; t < cnt; ++t) token(t);
+      for (int t = 0; t < cnt; ++t) {
+        get(cur, t);
+        run(cur, t);
+      }
     }
     if (col_ok && sub < cnt) a.o[((int64_t)(t0 + sub) * a.heads + head) * a.vdim_s + col] = mine;
     if (more) {
@@ -157,18 +187,25 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaArgs a) {
   store_state<E>(S, sp, sub, a.dim_s, col_ok);
 }
 
-// g = exp(-exp(A_log) softplus(z + dt_bias)), beta = sigmoid(b).
+// g = exp(-exp(A_log) softplus(z + dt_bias)), beta = sigmoid(b).  Four channels of a head per thread (dim_s % 4 == 0).
 template <typename T>
 __global__ __launch_bounds__(256) void delta_gates_kernel(const T* __restrict__ z, int64_t ldz, const T* __restrict__ b,
                                                           int64_t ldb, const float* __restrict__ A_log,
-                                                          const float* __restrict__ dt_bias, int n, int heads,
+                                                          const float* __restrict__ dt_bias, int64_t n, int heads,
                                                           int dim_s, float* __restrict__ g, float* __restrict__ beta) {
-  const int per = heads * dim_s;
+  typedef T quad_t __attribute__((ext_vector_type(4)));
+  const int per = heads * dim_s / 4;
   const int64_t at = (int64_t)blockIdx.x * 256 + threadIdx.x;
-  if (at >= (int64_t)n * per) return;
+  if (at >= n * per) return;
   const int64_t t = at / per;
-  const int c = (int)(at % per), h = c / dim_s;
-  g[at] = expf(-expf(A_log[h]) * softplus_f(to_f(z[t * ldz + c]) + dt_bias[c]));
+  const int c = (int)(at % per) * 4, h = c / dim_s;
+  const float ea = -exp_f(A_log[h]);
+  const quad_t zv = *reinterpret_cast<const quad_t*>(z + t * ldz + c);
+  const float4_t bias = *reinterpret_cast<const float4_t*>(dt_bias + c);
+  float4_t out;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) out[e] = exp_f(ea * softplus_f(to_f(zv[e]) + bias[e]));
+  *reinterpret_cast<float4_t*>(g + t * heads * dim_s + c) = out;
   if (c % dim_s == 0) beta[t * heads + h] = sigmoid_f(to_f(b[t * ldb + h]));
 }
 
@@ -226,7 +263,7 @@ __global__ __launch_bounds__(256) void delta_decode_kernel(DeltaStepArgs a) {
   // decays: two lanes per key channel
   const T* Wa = reinterpret_cast<const T*>(a.Wa);
   const T* Wg = reinterpret_cast<const T*>(a.Wg);
-  const float ea = expf(a.A_log[head]);
+  const float ea = exp_f(a.A_log[head]);
   const int half = tid & 1, cut = (a.rank_a / 2 + 7) / 8 * 8;
   for (int d = tid >> 1; d < D; d += 128) {
     float z = 0.f;
@@ -235,7 +272,7 @@ __global__ __launch_bounds__(256) void delta_decode_kernel(DeltaStepArgs a) {
       z = half ? dot_row<T>(w + cut, lat + cut, a.rank_a - cut) : dot_row<T>(w, lat, cut);
     }
     z = dpp_add<0xB1>(z);
-    if (half == 0) sg[d] = d < a.dim_s ? expf(-ea * softplus_f(z + a.dt_bias[head * a.dim_s + d])) : 0.f;
+    if (half == 0) sg[d] = d < a.dim_s ? exp_f(-ea * softplus_f(z + a.dt_bias[head * a.dim_s + d])) : 0.f;
   }
   // output gates: a row of 16 lanes per column
   float gz = 0.f;
@@ -258,7 +295,9 @@ __global__ __launch_bounds__(256) void delta_decode_kernel(DeltaStepArgs a) {
   __syncthreads();
   const float v = col_ok ? a.p[a.off_v + (int64_t)head * a.vdim_s + col] : 0.f;
   const float beta = sigmoid_f(a.p[a.off_b + head]);
-  const float o = delta_step<E>(S, sq, sk, sg, sub, v, beta, skq);
+  DeltaToken<E> tok;
+  tok.load(sq, sk, sg, sub, v, beta, skq);
+  const float o = delta_step<E>(S, tok);
   store_state<E>(S, sp, sub, a.dim_s, col_ok);
   if (col_ok && sub == 0) {
     a.o[(int64_t)head * a.vdim_s + col] = o;

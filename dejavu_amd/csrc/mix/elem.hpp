@@ -67,14 +67,35 @@ __device__ __forceinline__ float wave_sum(float v) {
   return v + __shfl_xor(v, 32, kWave);
 }
 
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
-__device__ __forceinline__ float silu_f(float z) { return z / (1.f + expf(-z)); }
-__device__ __forceinline__ float softplus_f(float z) { return z > 0.f ? z + log1pf(expf(-z)) : log1pf(expf(z)); }
+// fp32 exponential from the hardware's base-2 one: x log2(e) is kept in two parts, the second as a correction of the
+// result.  Arguments are held where the result is finite.
+__device__ __forceinline__ float exp_f(float x) {
+  x = fminf(fmaxf(x, -104.f), 88.5f);
+  const float hi = x * 1.44269504f;
+  const float lo = __builtin_fmaf(x, 1.92596299e-8f, __builtin_fmaf(x, 1.44269504f, -hi));
+  const float r = __builtin_amdgcn_exp2f(hi);
+  return __builtin_fmaf(r, lo * 0.693147181f, r);
+}
+__device__ __forceinline__ float rcp_f(float x) { return __builtin_amdgcn_rcpf(x); }
+__device__ __forceinline__ float sigmoid_f(float z) { return rcp_f(1.f + exp_f(-z)); }
+__device__ __forceinline__ float silu_f(float z) { return z * sigmoid_f(z); }
+// log(1 + e), 0 <= e <= 1: the Taylor series where 1 + e would lose the digits of e
+__device__ __forceinline__ float log1p_f(float e) {
+  const float series = e * (1.f - e * (0.5f - e * (0.333333333f - e * 0.25f)));
+  return e < 0.015625f ? series : __logf(1.f + e);
+}
+__device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.f) + log1p_f(exp_f(-fabsf(z))); }
+__device__ __forceinline__ float tanh_f(float x) {
+  const float t = exp_f(-2.f * fabsf(x)), x2 = x * x;
+  const float big = copysignf((1.f - t) * rcp_f(1.f + t), x);
+  const float series = x * (1.f - x2 * (0.333333333f - x2 * (0.133333333f - x2 * 0.0539682540f)));
+  return x2 < 0.01f ? series : big;
+}
 
 // Dynamic tanh: tanh(alpha x) w + b, per channel.
 using DynTanh = dvDynTanh;
 __device__ __forceinline__ float dyn_tanh(float x, const DynTanh& n, int c) {
-  return __builtin_fmaf(tanhf(n.alpha * x), n.w[c], n.b[c]);
+  return __builtin_fmaf(tanh_f(n.alpha * x), n.w[c], n.b[c]);
 }
 
 // The sequence position of a call: on the device (captured decode steps) or passed by the host.

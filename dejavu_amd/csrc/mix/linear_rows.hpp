@@ -44,16 +44,32 @@ __device__ __forceinline__ void stage_row(const RowsArgs& a, T* xs, float* red) 
     const float s = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / a.norm_dim + a.eps);
     for (int i = tid; i < K; i += 256) xs[i] = from_f<T>(x[i] * s * a.xw[i]);
   } else {
-    // one head per wave at a time
+    // a row of 16 lanes per head; eight channels per lane at a time, the first 128 kept in registers
     const float* x = reinterpret_cast<const float*>(a.x);
-    const int heads = K / a.head_stride, lane = tid & 63;
-    for (int h = tid >> 6; h < heads; h += 4) {
+    const int heads = K / a.head_stride, sub = tid & 15;
+    for (int h = tid >> 4; h < heads; h += 16) {
       const float* xh = x + (int64_t)h * a.head_stride;
+      const float* gh = a.gate + (int64_t)h * a.head_stride;
+      Pack8<float> v;
+      v.zero();
+      if (sub * 8 < a.head_stride) v.load(xh + sub * 8);
       float ss = 0.f;
-      for (int c = lane; c < a.norm_dim; c += 64) ss = __builtin_fmaf(xh[c], xh[c], ss);
-      const float s = 1.f / sqrtf(wave_sum(ss) / a.norm_dim + a.eps);
-      for (int c = lane; c < a.head_stride; c += 64)
-        xs[h * a.head_stride + c] = from_f<T>(xh[c] * s * a.xw[c] * a.gate[(int64_t)h * a.head_stride + c]);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss = __builtin_fmaf(v.get(e), v.get(e), ss);
+      for (int c = 128 + sub * 8; c < a.head_stride; c += 128) {
+        Pack8<float> u;
+        u.load(xh + c);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss = __builtin_fmaf(u.get(e), u.get(e), ss);
+      }
+      const float s = 1.f / sqrtf(row16_sum(ss) / a.norm_dim + a.eps);
+      for (int c = sub * 8; c < a.head_stride; c += 128) {
+        Pack8<float> u = v, g;
+        if (c >= 128) u.load(xh + c);
+        g.load(gh + c);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) xs[h * a.head_stride + c + e] = from_f<T>(u.get(e) * s * a.xw[c + e] * g.get(e));
+      }
     }
   }
   __syncthreads();

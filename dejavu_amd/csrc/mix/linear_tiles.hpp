@@ -45,7 +45,7 @@ __global__ __launch_bounds__(256) void linear_tiles_kernel(TileArgs a) {
       const bool in = k + kq < a.K;
 #pragma unroll
       for (int i = 0; i < RT; ++i) {
-        if (in) w[u][i].load_stream(wp[i] + k);
+        if (in) w[u][i].load(wp[i] + k);
         else w[u][i].zero();
       }
 #pragma unroll

@@ -7,9 +7,96 @@ namespace dv {
 using ConvGroup = dvConvGroup;
 using ConvArgs = dvConvArgs;
 
-// One wave per (token, head); a lane holds up to NE channels.  TO: type of the outputs.
-template <typename T, typename TO, int NE>
+// A lane owns eight channels of one head and walks TB consecutive tokens with the last TAPS inputs in registers; the
+// LPH lanes of a head (a power of two, 8 LPH >= stride) add up its norm.  Grid: (units of heads, token blocks).
+constexpr int kConvTokens = 8;
+
+template <int LPH>
+__device__ __forceinline__ float lanes_sum(float v) {
+  if constexpr (LPH >= 2) v = dpp_add<0xB1>(v);
+  if constexpr (LPH >= 4) v = dpp_add<0x4E>(v);
+  if constexpr (LPH >= 8) v = dpp_add<0x141>(v);
+  if constexpr (LPH >= 16) v = dpp_add<0x140>(v);
+  if constexpr (LPH >= 32) v += __shfl_xor(v, 16, kWave);
+  if constexpr (LPH >= 64) v += __shfl_xor(v, 32, kWave);
+  return v;
+}
+
+template <typename T, typename TO, int LPH, int TAPS>
 __global__ __launch_bounds__(256) void short_conv_kernel(ConvArgs a) {
+  constexpr int HPB = 256 / LPH;  // heads per workgroup
+  const int heads = a.g[0].heads + a.g[1].heads + a.g[2].heads;
+  const int unit = blockIdx.x * HPB + threadIdx.x / LPH, c = threadIdx.x % LPH * 8;
+  int h = unit < heads ? unit : 0, base = 0, gi = 0;
+  if (h >= a.g[0].heads) {
+    h -= a.g[0].heads;
+    base = a.g[0].heads * a.g[0].stride;
+    gi = 1;
+    if (h >= a.g[1].heads) {
+      h -= a.g[1].heads;
+      base += a.g[1].heads * a.g[1].stride;
+      gi = 2;
+    }
+  }
+  const ConvGroup g = a.g[gi];
+  const bool on = unit < heads && c < g.stride;
+  const int ch = base + h * g.stride + c;
+  const T* in = reinterpret_cast<const T*>(a.in) + ch;
+  float w[TAPS][8], u[TAPS][8];
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+    for (int e = 0; e < 8; ++e) w[j][e] = on ? a.w[(int64_t)(ch + e) * TAPS + j] : 0.f;
+  const int t0 = blockIdx.y * kConvTokens, t1 = min(a.n, t0 + kConvTokens);
+  Pack8<T> next[kConvTokens];
+#pragma unroll
+  for (int i = 0; i < kConvTokens; ++i) {
+    if (on && t0 + i < t1) next[i].load(in + (int64_t)(t0 + i) * a.ldi);
+    else next[i].zero();
+  }
+#pragma unroll
+  for (int j = 0; j < TAPS - 1; ++j) {  // the inputs before the block
+    const int s = t0 - (TAPS - 1) + j;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      float x = 0.f;
+      if (on) x = s >= 0 ? to_f(in[(int64_t)s * a.ldi + e]) : a.state[(int64_t)(ch + e) * (TAPS - 1) + TAPS - 1 + s];
+      u[j][e] = x;
+    }
+  }
+  TO* out = reinterpret_cast<TO*>(g.out) + (int64_t)h * g.stride + c;
+#pragma unroll
+  for (int i = 0; i < kConvTokens; ++i) {
+    float y[8], ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      u[TAPS - 1][e] = next[i].get(e);
+      float v = 0.f;
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) v = __builtin_fmaf(w[j][e], u[j][e], v);
+      y[e] = a.silu ? silu_f(v) : v;
+      if (c + e < g.dim) ss = __builtin_fmaf(y[e], y[e], ss);
+    }
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) u[j][e] = u[j + 1][e];
+    ss = lanes_sum<LPH>(on ? ss : 0.f);  // by every lane: the lanes of a head may share a wave with a group without norm
+    const float s = g.norm == 1 ? 1.f / sqrtf(ss / g.dim + g.eps) : (g.norm == 2 ? g.scale / sqrtf(ss + 1e-6f) : 1.f);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) y[e] *= s;
+    if (on && t0 + i < t1) {
+      __attribute__((aligned(16))) TO o[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) o[e] = from_f<TO>(y[e]);
+      *reinterpret_cast<Pack8<TO>*>(out + (int64_t)(t0 + i) * g.ld) = *reinterpret_cast<const Pack8<TO>*>(o);
+    }
+  }
+}
+
+// Any number of taps and any head size: one wave per (token, head), values computed twice where a norm needs them.
+template <typename T, typename TO>
+__global__ __launch_bounds__(256) void short_conv_any_kernel(ConvArgs a) {
   const int lane = threadIdx.x & 63;
   const int heads = a.g[0].heads + a.g[1].heads + a.g[2].heads;
   const int64_t task = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
@@ -29,34 +116,28 @@ __global__ __launch_bounds__(256) void short_conv_kernel(ConvArgs a) {
   const ConvGroup g = a.g[gi];
   const T* in = reinterpret_cast<const T*>(a.in);
   base += h * g.stride;
-  float v[NE], ss = 0.f;
-#pragma unroll
-  for (int i = 0; i < NE; ++i) {
-    const int c = lane + i * 64;
-    v[i] = 0.f;
-    if (c < g.stride) {
-      const int ch = base + c;
-      float y = 0.f;
-      for (int j = 0; j < a.taps; ++j) {
-        const int s = t - (a.taps - 1) + j;
-        const float u = s >= 0 ? to_f(in[s * a.ldi + ch]) : a.state[(int64_t)ch * (a.taps - 1) + a.taps - 1 + s];
-        y = __builtin_fmaf(a.w[(int64_t)ch * a.taps + j], u, y);
-      }
-      v[i] = a.silu ? silu_f(y) : y;
-      if (c < g.dim) ss = __builtin_fmaf(v[i], v[i], ss);
+  auto value = [&](int c) {
+    const int ch = base + c;
+    float y = 0.f;
+    for (int j = 0; j < a.taps; ++j) {
+      const int s = t - (a.taps - 1) + j;
+      const float u = s >= 0 ? to_f(in[s * a.ldi + ch]) : a.state[(int64_t)ch * (a.taps - 1) + a.taps - 1 + s];
+      y = __builtin_fmaf(a.w[(int64_t)ch * a.taps + j], u, y);
     }
-  }
+    return a.silu ? silu_f(y) : y;
+  };
   float s = 1.f;
   if (g.norm) {
+    float ss = 0.f;
+    for (int c = lane; c < g.dim; c += 64) {
+      const float v = value(c);
+      ss = __builtin_fmaf(v, v, ss);
+    }
     ss = wave_sum(ss);
     s = g.norm == 1 ? 1.f / sqrtf(ss / g.dim + g.eps) : g.scale / sqrtf(ss + 1e-6f);
   }
   TO* out = reinterpret_cast<TO*>(g.out) + (int64_t)t * g.ld + (int64_t)h * g.stride;
-#pragma unroll
-  for (int i = 0; i < NE; ++i) {
-    const int c = lane + i * 64;
-    if (c < g.stride) out[c] = from_f<TO>(v[i] * s);
-  }
+  for (int c = lane; c < g.stride; c += 64) out[c] = from_f<TO>(value(c) * s);
 }
 
 // state <- the last taps - 1 inputs of (state, in[0..n)).  One thread per channel; in place: a slot is written

@@ -31,19 +31,29 @@ __device__ __forceinline__ void residual_apply(const ResidualArgs& a, int64_t at
   if (a.h) reinterpret_cast<T*>(a.h)[at] = from_f<T>(dyn_tanh(v, a.pre, c));
 }
 
-// y == nullptr: only x += x0 and h = pre(x).
+// y == nullptr: only x += x0 and h = pre(x).  Four channels per thread (width % 4 == 0).
 template <typename T>
-__global__ __launch_bounds__(256) void residual_norm_kernel(const T* __restrict__ y, int64_t count, int width,
+__global__ __launch_bounds__(256) void residual_norm_kernel(const T* __restrict__ y, int64_t quads, int width,
                                                             ResidualArgs a) {
-  for (int64_t at = (int64_t)blockIdx.x * 256 + threadIdx.x; at < count; at += (int64_t)gridDim.x * 256) {
+  typedef T quad_t __attribute__((ext_vector_type(4)));
+  for (int64_t q = (int64_t)blockIdx.x * 256 + threadIdx.x; q < quads; q += (int64_t)gridDim.x * 256) {
+    const int64_t at = q * 4;
     const int c = (int)(at % width);
+    float4_t v = *reinterpret_cast<const float4_t*>(a.x + at);
     if (y) {
-      residual_apply<T>(a, at, c, to_f(y[at]));
-    } else {
-      float v = a.x[at];
-      if (a.x0) v += a.x0[at];
-      a.x[at] = v;
-      if (a.h) reinterpret_cast<T*>(a.h)[at] = from_f<T>(dyn_tanh(v, a.pre, c));
+      const quad_t u = *reinterpret_cast<const quad_t*>(y + at);
+      const float4_t w = *reinterpret_cast<const float4_t*>(a.post.w + c), b = *reinterpret_cast<const float4_t*>(a.post.b + c);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] += __builtin_fmaf(tanh_f(a.post.alpha * to_f(u[e])), w[e], b[e]);
+    }
+    if (a.x0) v += *reinterpret_cast<const float4_t*>(a.x0 + at);
+    *reinterpret_cast<float4_t*>(a.x + at) = v;
+    if (a.h) {
+      const float4_t w = *reinterpret_cast<const float4_t*>(a.pre.w + c), b = *reinterpret_cast<const float4_t*>(a.pre.b + c);
+      quad_t h;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) h[e] = from_f<T>(__builtin_fmaf(tanh_f(a.pre.alpha * v[e]), w[e], b[e]));
+      *reinterpret_cast<quad_t*>(reinterpret_cast<T*>(a.h) + at) = h;
     }
   }
 }
@@ -67,39 +77,88 @@ __global__ __launch_bounds__(256) void clamped_glu_kernel(const T* __restrict__ 
   for (int e = 0; e < 4; ++e) y[i + e] = from_f<T>(clamped_glu_f(v.get(2 * e), v.get(2 * e + 1), limit));
 }
 
-// y = x * rsqrt(mean(x^2) + eps) * w over the first `dim` entries of every row (entries up to ldy: weight 0).
-// One wave per row.
+// y = x / sqrt(mean(x^2) + eps) * w, the mean over the first `dim` entries (those up to `padded`, a multiple of 8, are
+// zero).  One wave per row, eight entries per lane at a time.
 template <typename T>
 __global__ __launch_bounds__(256) void rms_rows_kernel(const T* __restrict__ x, int64_t ldx, int64_t rows, int dim,
                                                        int padded, const float* __restrict__ w, float eps,
                                                        T* __restrict__ y, int64_t ldy) {
+  constexpr int NP = 4;  // packets a lane keeps; longer rows read the rest twice
   const int64_t r = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (r >= rows) return;
   const int lane = threadIdx.x & 63;
+  const T* xr = x + r * ldx;
+  Pack8<T> v[NP];
   float ss = 0.f;
-  for (int c = lane; c < dim; c += 64) {
-    const float v = to_f(x[r * ldx + c]);
-    ss = __builtin_fmaf(v, v, ss);
+#pragma unroll
+  for (int i = 0; i < NP; ++i) {
+    const int c = (i * 64 + lane) * 8;
+    if (c < padded) v[i].load(xr + c);
+    else v[i].zero();
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss = __builtin_fmaf(v[i].get(e), v[i].get(e), ss);
+  }
+  for (int c = (NP * 64 + lane) * 8; c < padded; c += 512) {
+    Pack8<T> t;
+    t.load(xr + c);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss = __builtin_fmaf(t.get(e), t.get(e), ss);
   }
   const float s = 1.f / sqrtf(wave_sum(ss) / dim + eps);
-  for (int c = lane; c < padded; c += 64) y[r * ldy + c] = from_f<T>(to_f(x[r * ldx + c]) * s * w[c]);
+  auto put = [&](const Pack8<T>& t, int c) {
+    __attribute__((aligned(16))) T o[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) o[e] = from_f<T>(t.get(e) * s * w[c + e]);
+    *reinterpret_cast<Pack8<T>*>(y + r * ldy + c) = *reinterpret_cast<const Pack8<T>*>(o);
+  };
+#pragma unroll
+  for (int i = 0; i < NP; ++i) {
+    const int c = (i * 64 + lane) * 8;
+    if (c < padded) put(v[i], c);
+  }
+  for (int c = (NP * 64 + lane) * 8; c < padded; c += 512) {
+    Pack8<T> t;
+    t.load(xr + c);
+    put(t, c);
+  }
 }
 
-// y[i, h, :] = o[i, h, :] / rms(o[i, h, :]) * w * sigmoid(gate[i, h, :]); one wave per (token, head).
+// y[i, h, :] = o[i, h, :] / rms(o[i, h, :]) * w * sigmoid(gate[i, h, :]).  A row of 16 lanes per (token, head); eight
+// channels per lane at a time, the first 128 kept in registers.
 template <typename T>
 __global__ __launch_bounds__(256) void gated_head_norm_kernel(const float* __restrict__ o, const T* __restrict__ gate,
                                                               int64_t ldg, int64_t rows, int heads, int vdim,
                                                               int padded, const float* __restrict__ w, float eps,
                                                               T* __restrict__ y) {
-  const int64_t r = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (r >= rows * heads) return;
-  const int lane = threadIdx.x & 63;
-  const int64_t row = r / heads, head = r % heads;
+  const int64_t r = (int64_t)blockIdx.x * 16 + (threadIdx.x >> 4);
+  const int sub = threadIdx.x & 15;
+  const bool ok = r < rows * heads;  // whole rows of lanes: the sum below stays inside one
+  const int64_t row = ok ? r / heads : 0, head = ok ? r % heads : 0;
+  const float* src = o + (ok ? r : 0) * padded;
+  Pack8<float> v;
+  v.zero();
+  if (sub * 8 < padded) v.load(src + sub * 8);
   float ss = 0.f;
-  for (int c = lane; c < vdim; c += 64) ss = __builtin_fmaf(o[r * padded + c], o[r * padded + c], ss);
-  const float s = 1.f / sqrtf(wave_sum(ss) / vdim + eps);
-  for (int c = lane; c < padded; c += 64)
-    y[r * padded + c] = from_f<T>(o[r * padded + c] * s * w[c] * sigmoid_f(to_f(gate[row * ldg + head * padded + c])));
+#pragma unroll
+  for (int e = 0; e < 8; ++e) ss = __builtin_fmaf(v.get(e), v.get(e), ss);
+  for (int c = 128 + sub * 8; c < padded; c += 128) {
+    Pack8<float> t;
+    t.load(src + c);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss = __builtin_fmaf(t.get(e), t.get(e), ss);
+  }
+  const float s = 1.f / sqrtf(row16_sum(ss) / vdim + eps);
+  if (!ok) return;
+  for (int c = sub * 8; c < padded; c += 128) {
+    Pack8<float> t = v;
+    if (c >= 128) t.load(src + c);
+    Pack8<T> g;
+    g.load(gate + row * ldg + head * padded + c);
+    __attribute__((aligned(16))) T out[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) out[e] = from_f<T>(t.get(e) * s * w[c + e] * sigmoid_f(g.get(e)));
+    *reinterpret_cast<Pack8<T>*>(y + r * padded + c) = *reinterpret_cast<const Pack8<T>*>(out);
+  }
 }
 
 // First index of the largest of `vocab` fp32 logits, and the bookkeeping of a generation loop (one workgroup):

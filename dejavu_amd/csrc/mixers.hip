@@ -5,6 +5,7 @@
 
 #include <atomic>
 
+#include "mix/attn_latent.hpp"
 #include "mix/attn_rows.hpp"
 #include "mix/attn_tiles.hpp"
 #include "mix/delta_rule.hpp"
@@ -75,12 +76,36 @@ int linear_row_any(int before, int after, const RowsArgs& a, hipStream_t s) {
   return DV_ERR_UNSUPPORTED;
 }
 
+// ---- short convolution -------------------------------------------------------
+template <typename T, typename TO, int LPH>
+int short_conv_lanes(const ConvArgs& a, int heads, hipStream_t s) {
+  const dim3 grid(blocks_of(heads, 256 / LPH), blocks_of(a.n, kConvTokens));
+  switch (a.taps) {
+    case 1: hipLaunchKernelGGL((short_conv_kernel<T, TO, LPH, 1>), grid, dim3(256), 0, s, a); break;
+    case 2: hipLaunchKernelGGL((short_conv_kernel<T, TO, LPH, 2>), grid, dim3(256), 0, s, a); break;
+    case 3: hipLaunchKernelGGL((short_conv_kernel<T, TO, LPH, 3>), grid, dim3(256), 0, s, a); break;
+    default: hipLaunchKernelGGL((short_conv_kernel<T, TO, LPH, 4>), grid, dim3(256), 0, s, a); break;
+  }
+  return launched();
+}
+template <typename T, typename TO>
+int short_conv_types(const ConvArgs& a, int heads, int widest, hipStream_t s) {
+  if (a.taps > 4 || widest > 512 || (a.n + kConvTokens - 1) / kConvTokens > 65535) {
+    hipLaunchKernelGGL((short_conv_any_kernel<T, TO>), dim3(blocks_of((int64_t)a.n * heads, 4)), dim3(256), 0, s, a);
+    return launched();
+  }
+  if (widest <= 64) return short_conv_lanes<T, TO, 8>(a, heads, s);
+  if (widest <= 128) return short_conv_lanes<T, TO, 16>(a, heads, s);
+  if (widest <= 256) return short_conv_lanes<T, TO, 32>(a, heads, s);
+  return short_conv_lanes<T, TO, 64>(a, heads, s);
+}
+
 // ---- attention rows --------------------------------------------------------
 template <typename T, typename TQ, int RH>
 int attn_rows_rh(const AttnArgs& a, hipStream_t s) {
   const int rep = a.H / a.G;
   const dim3 grid(a.splits, a.G * ((rep + RH - 1) / RH), a.n);
-  const size_t lds = (size_t)RH * a.dim_s * 4 + 256 * 8 * 4;
+  const size_t lds = (size_t)RH * a.dim_s * 4 + 256 * 8 * 4 + (size_t)(a.dim_s + a.vdim_s) * sizeof(T);
   return launch_lds<attn_rows_kernel<T, TQ, RH>>(grid, dim3(256), lds, s, a);
 }
 template <typename T, typename TQ>
@@ -92,9 +117,15 @@ int attn_rows_any(const AttnArgs& a, hipStream_t s) {
   return attn_rows_rh<T, TQ, 1>(a, s);
 }
 
+template <int RT>
+int latent_tiles(const AttnArgs& a, hipStream_t s) {
+  if (a.H <= 16) return launch_lds<latent_attn_kernel<RT, 1>>(dim3(a.splits, 1), dim3(256), latent_lds_bytes<RT, 1>(), s, a);
+  return launch_lds<latent_attn_kernel<RT, 2>>(dim3(a.splits, (a.H + 31) / 32), dim3(256), latent_lds_bytes<RT, 2>(), s, a);
+}
+
 int attn_args_ok(const AttnArgs* a) {
   if (!a || !a->q || !a->k || !a->v || a->n < 1 || a->H < 1 || a->G < 1 || a->H % a->G || a->dim_s < 8 ||
-      a->vdim_s < 8 || a->splits < 1 || (a->splits > 1 && !a->part) || (a->splits == 1 && !a->out) ||
+      a->vdim_s < 8 || a->splits < 1 || a->splits > kMaxSplits || (a->splits > 1 && !a->part) || (a->splits == 1 && !a->out) ||
       (!a->fresh_k != !a->fresh_v))
     return DV_ERR_INVALID_ARG;
   if (a->dim_s % 8 || a->vdim_s % 8 || a->ldk % 8 || a->ldv % 8 || a->k_head % 8 || a->v_head % 8 || !al16(a->k) ||
@@ -132,9 +163,10 @@ int dv_mix_residual(int dtype, const void* y, int64_t n, int width, const dvResi
   if (!dtype_ok(dtype) || n < 1 || width < 1 || !r || !r->x || (y && (!r->post.w || !r->post.b)) ||
       (r->h && (!r->pre.w || !r->pre.b)))
     return DV_ERR_INVALID_ARG;
-  const int64_t count = n * width;
+  if (width % 8 || !al16(r->x) || !al16(y) || !al16(r->h)) return DV_ERR_ALIGNMENT;
+  const int64_t count = n * width / 4;
   unsigned grid = blocks_of(count, 256);
-  if (grid > 16384) grid = 16384;
+  if (grid > 8192) grid = 8192;
   if (dtype == DV_BF16)
     hipLaunchKernelGGL((residual_norm_kernel<bf16_t>), dim3(grid), dim3(256), 0, st(stream), (const bf16_t*)y, count, width, *r);
   else
@@ -156,6 +188,7 @@ int dv_mix_clamped_glu(int dtype, const void* gu, int64_t count, float limit, vo
 int dv_mix_rms_rows(int dtype, const void* x, int64_t ldx, int64_t rows, int dim, int padded, const float* w, float eps,
                     void* y, int64_t ldy, void* stream) {
   if (!dtype_ok(dtype) || !x || !w || !y || rows < 1 || dim < 1 || padded < dim) return DV_ERR_INVALID_ARG;
+  if (padded % 8 || ldx % 8 || ldy % 8 || !al16(x) || !al16(y)) return DV_ERR_ALIGNMENT;
   const dim3 grid(blocks_of(rows, 4));
   if (dtype == DV_BF16)
     hipLaunchKernelGGL((rms_rows_kernel<bf16_t>), grid, dim3(256), 0, st(stream), (const bf16_t*)x, ldx, rows, dim, padded, w, eps, (bf16_t*)y, ldy);
@@ -168,7 +201,8 @@ int dv_mix_gated_head_norm(int dtype, const float* o, const void* gate, int64_t 
                            int padded, const float* w, float eps, void* y, void* stream) {
   if (!dtype_ok(dtype) || !o || !gate || !w || !y || rows < 1 || heads < 1 || vdim < 1 || padded < vdim)
     return DV_ERR_INVALID_ARG;
-  const dim3 grid(blocks_of(rows * heads, 4));
+  if (padded % 8 || ldg % 8 || !al16(o) || !al16(gate) || !al16(y)) return DV_ERR_ALIGNMENT;
+  const dim3 grid(blocks_of(rows * heads, 16));
   if (dtype == DV_BF16)
     hipLaunchKernelGGL((gated_head_norm_kernel<bf16_t>), grid, dim3(256), 0, st(stream), o, (const bf16_t*)gate, ldg, rows, heads, vdim, padded, w, eps, (bf16_t*)y);
   else
@@ -185,7 +219,8 @@ int dv_mix_linear_row(int dtype, int before, int after, const dvRowArgs* a, void
   if (after == DV_OUT_CONV && (!a->conv_w || a->taps < 1 || (a->taps > 1 && !a->conv_state) || a->conv_rows > a->M))
     return DV_ERR_INVALID_ARG;
   if (before == DV_ROW_RMS && (!a->xw || a->norm_dim < 1 || a->norm_dim > a->K)) return DV_ERR_INVALID_ARG;
-  if (before == DV_ROW_HEADS && (!a->xw || !a->gate || a->head_stride < 1 || a->K % a->head_stride ||
+  if (before == DV_ROW_HEADS && (!a->xw || !a->gate || a->head_stride < 8 || a->head_stride % 8 ||
+                                 a->K % a->head_stride ||
                                  a->norm_dim < 1 || a->norm_dim > a->head_stride))
     return DV_ERR_INVALID_ARG;
   if (a->side_x && (!a->side_w || !a->side_out || a->side_dim < 1)) return DV_ERR_INVALID_ARG;
@@ -229,19 +264,12 @@ int dv_mix_short_conv(int dtype, int out_f32, const dvConvArgs* a, void* stream)
     if (g.heads > 0 && g.stride > widest) widest = g.stride;
   }
   if (heads == 0) return DV_ERR_INVALID_ARG;
-  if (widest > 1024) return DV_ERR_UNSUPPORTED;
-  const dim3 grid(blocks_of((int64_t)a->n * heads, 4));
-#define DV_CONV(T, TO)                                                                                       \
-  do {                                                                                                       \
-    if (widest <= 128) hipLaunchKernelGGL((short_conv_kernel<T, TO, 2>), grid, dim3(256), 0, st(stream), *a); \
-    else if (widest <= 256) hipLaunchKernelGGL((short_conv_kernel<T, TO, 4>), grid, dim3(256), 0, st(stream), *a); \
-    else hipLaunchKernelGGL((short_conv_kernel<T, TO, 16>), grid, dim3(256), 0, st(stream), *a);             \
-  } while (0)
-  if (dtype == DV_F32) DV_CONV(float, float);
-  else if (out_f32) DV_CONV(bf16_t, float);
-  else DV_CONV(bf16_t, bf16_t);
-#undef DV_CONV
-  return launched();
+  for (const dvConvGroup& g : a->g)
+    if (g.heads > 0 && (g.stride % 8 || g.ld % 8 || !al16(g.out))) return DV_ERR_ALIGNMENT;
+  if (a->ldi % 8 || !al16(a->in)) return DV_ERR_ALIGNMENT;
+  if (dtype == DV_F32) return short_conv_types<float, float>(*a, heads, widest, st(stream));
+  if (out_f32) return short_conv_types<bf16_t, float>(*a, heads, widest, st(stream));
+  return short_conv_types<bf16_t, bf16_t>(*a, heads, widest, st(stream));
 }
 
 int dv_mix_conv_state(int dtype, const void* in, int64_t ldi, int n, int channels, int taps, float* state, void* stream) {
@@ -279,10 +307,10 @@ int dv_mix_attn_rows(int dtype, int q_f32, const dvAttnArgs* a, void* stream) {
   else if (q_f32) rc = attn_rows_any<bf16_t, float>(*a, st(stream));
   else rc = attn_rows_any<bf16_t, bf16_t>(*a, st(stream));
   if (rc != DV_OK || a->splits == 1) return rc;
-  const dim3 grid(a->H, a->n);
-  if (dtype == DV_F32) hipLaunchKernelGGL((attn_merge_kernel<float, float>), grid, dim3(256), 0, st(stream), *a);
-  else if (q_f32) hipLaunchKernelGGL((attn_merge_kernel<bf16_t, float>), grid, dim3(256), 0, st(stream), *a);
-  else hipLaunchKernelGGL((attn_merge_kernel<bf16_t, bf16_t>), grid, dim3(256), 0, st(stream), *a);
+  const dim3 grid(a->H, (a->vdim_s + 63) / 64, a->n);
+  if (dtype == DV_F32) hipLaunchKernelGGL((attn_merge_kernel<float, float>), grid, dim3(256), 0, st(stream), *a, (float*)a->out);
+  else if (q_f32) hipLaunchKernelGGL((attn_merge_kernel<bf16_t, float>), grid, dim3(256), 0, st(stream), *a, (bf16_t*)a->out);
+  else hipLaunchKernelGGL((attn_merge_kernel<bf16_t, bf16_t>), grid, dim3(256), 0, st(stream), *a, (bf16_t*)a->out);
   return launched();
 }
 
@@ -320,23 +348,28 @@ int dv_mix_latent_absorb(int dtype, const float* q, const void* W, int H, int di
   return launched();
 }
 
-int dv_mix_latent_attn(int dtype, const dvAttnArgs* a, const void* W, int vrows, void* out, void* stream) {
-  if (!dtype_ok(dtype) || !W || !out || vrows < 1 || !a || a->n != 1 || a->G != 1 || !a->part) return DV_ERR_INVALID_ARG;
-  dvAttnArgs b = *a;
-  // one split also goes through the partial sums: the value product reads them
-  const int splits = b.splits;
-  if (splits < 2) return DV_ERR_INVALID_ARG;
-  int rc = attn_args_ok(&b);
+int dv_mix_latent_attn(int dtype, const dvAttnArgs* a, float* lat, const void* W, int vrows, void* out, void* stream) {
+  if (!dtype_ok(dtype) || !W || !out || !lat || vrows < 1 || !a || a->n != 1 || a->G != 1 || !a->part || a->splits < 2 ||
+      a->k != a->v || a->dim_s != a->vdim_s || a->window > 0 || a->ring > 0 || a->base != 0 || a->fresh_k || a->norm_dim > 0)
+    return DV_ERR_INVALID_ARG;
+  int rc = attn_args_ok(a);
   if (rc != DV_OK) return rc;
-  if (!al16(W)) return DV_ERR_ALIGNMENT;
-  rc = dtype == DV_BF16 ? attn_rows_any<bf16_t, float>(b, st(stream)) : attn_rows_any<float, float>(b, st(stream));
+  if (!al16(W) || !al16(a->part)) return DV_ERR_ALIGNMENT;
+  const int rank = a->vdim_s;
+  if (dtype == DV_F32) rc = attn_rows_any<float, float>(*a, st(stream));
+  else if (rank <= 64) rc = latent_tiles<4>(*a, st(stream));
+  else if (rank <= 128) rc = latent_tiles<8>(*a, st(stream));
+  else if (rank <= 256) rc = latent_tiles<16>(*a, st(stream));
+  else if (rank <= 512) rc = latent_tiles<32>(*a, st(stream));
+  else rc = attn_rows_any<bf16_t, float>(*a, st(stream));
   if (rc != DV_OK) return rc;
-  const dim3 grid(b.H, vrows <= 16 ? 1 : (vrows <= 64 ? 2 : 8));
-  const size_t lds = (size_t)b.vdim_s * 4;
+  hipLaunchKernelGGL((attn_merge_kernel<float, float>), dim3(a->H, (rank + 63) / 64, 1), dim3(256), 0, st(stream), *a, lat);
+  const dim3 grid(a->H, vrows <= 16 ? 1 : (vrows <= 64 ? 4 : 8));
+  const size_t lds = (size_t)rank * 4;
   if (dtype == DV_BF16)
-    hipLaunchKernelGGL((latent_out_kernel<bf16_t>), grid, dim3(256), lds, st(stream), b, (const bf16_t*)W, vrows, (bf16_t*)out);
+    hipLaunchKernelGGL((latent_out_kernel<bf16_t>), grid, dim3(256), lds, st(stream), lat, (const bf16_t*)W, rank, vrows, (bf16_t*)out);
   else
-    hipLaunchKernelGGL((latent_out_kernel<float>), grid, dim3(256), lds, st(stream), b, (const float*)W, vrows, (float*)out);
+    hipLaunchKernelGGL((latent_out_kernel<float>), grid, dim3(256), lds, st(stream), lat, (const float*)W, rank, vrows, (float*)out);
   return launched();
 }
 
@@ -344,7 +377,8 @@ int dv_mix_delta_gates(int dtype, const void* z, int64_t ldz, const void* b, int
                        const float* dt_bias, int n, int heads, int dim_s, float* g, float* beta, void* stream) {
   if (!dtype_ok(dtype) || !z || !b || !A_log || !dt_bias || n < 1 || heads < 1 || dim_s < 1 || !g || !beta)
     return DV_ERR_INVALID_ARG;
-  const dim3 grid(blocks_of((int64_t)n * heads * dim_s, 256));
+  if (dim_s % 8 || ldz % 8 || !al16(z) || !al16(g) || !al16(dt_bias)) return DV_ERR_ALIGNMENT;
+  const dim3 grid(blocks_of((int64_t)n * heads * dim_s / 4, 256));
   if (dtype == DV_BF16)
     hipLaunchKernelGGL((delta_gates_kernel<bf16_t>), grid, dim3(256), 0, st(stream), (const bf16_t*)z, ldz, (const bf16_t*)b, ldb, A_log, dt_bias, n, heads, dim_s, g, beta);
   else

@@ -266,7 +266,7 @@ def ring_copy(buf: torch.Tensor, ring: torch.Tensor, first: int, to_ring: bool) 
 def decode_splits(keys: int) -> int:
     """Workgroups that share the keys of a decode row.  ``keys`` is the most there can be: the value may not depend
     on the position, which captured steps only know on the device."""
-    return max(1, min(64, (keys + 127) // 128))
+    return max(1, min(64, (keys + 63) // 64), min(128, keys // 128))
 
 
 def _attn_args(q, k, v, n, H, G, dim_s, vdim_s, scale, sink, gate, window, ring, base, pos_dev, pos):
@@ -336,7 +336,9 @@ def latent_attention_row(q, k_up, v_up, cache, heads, scale, gate, pos_dev, pos)
     part = torch.empty(heads * a.splits * (rank + 2), dtype=torch.float32, device=q.device)
     a.part = part.data_ptr()
     out = torch.empty(1, heads * vdim_s, dtype=cache.dtype, device=q.device)
-    check(lib.dv_mix_latent_attn(code, _ref(a), _ptr(v_up), vdim_s, _ptr(out), _stream()), "dv_mix_latent_attn")
+    # the queries are not needed any more when the merged latents are written: they share their memory
+    check(lib.dv_mix_latent_attn(code, _ref(a), _ptr(ql), _ptr(v_up), vdim_s, _ptr(out), _stream()),
+          "dv_mix_latent_attn")
     return out
 
 

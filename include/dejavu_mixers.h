@@ -122,7 +122,7 @@ typedef struct {
   const int* pos_dev;      /* position of query row 0 */
   int pos_host;
   void* out;               /* [n][H][vdim_s] */
-  float* part;             /* splits > 1: [n][H][splits][vdim_s + 2] fp32 scratch */
+  float* part;             /* splits > 1 (at most 128): [n][H][splits][vdim_s + 2] scratch */
   int splits;
   const float* fresh_k;    /* decode: this token's key / value rows (fp32), stored in their slots first */
   const float* fresh_v;
@@ -184,9 +184,10 @@ DV_API int dv_mix_attn_tiles(const dvAttnArgs* args, int keys, void* stream);
 /* Latent decode row: out [H][rank] = q[h] W_uk[h]; W [H][dim_s][rank]. */
 DV_API int dv_mix_latent_absorb(int dtype, const float* q, const void* W, int H, int dim_s, int rank, float* out,
                                 void* stream);
-/* Latent decode row: attention over the cache (args: G = 1, k == v, vdim_s = rank, splits partials, no output),
- * then W_uv [H][vrows][rank] and the gate. */
-DV_API int dv_mix_latent_attn(int dtype, const dvAttnArgs* args, const void* W, int vrows, void* out, void* stream);
+/* Latent decode row: attention over the cache (args: G = 1, k == v, dim_s = vdim_s = rank, at least two splits with
+ * `part`, q and gate fp32), gated; lat [H][rank] fp32 receives it, out [H][vrows] = W_uv [H][vrows][rank] lat. */
+DV_API int dv_mix_latent_attn(int dtype, const dvAttnArgs* args, float* lat, const void* W, int vrows, void* out,
+                              void* stream);
 DV_API int dv_mix_delta_gates(int dtype, const void* z, int64_t ldz, const void* b, int64_t ldb, const float* A_log,
                               const float* dt_bias, int n, int heads, int dim_s, float* g, float* beta, void* stream);
 DV_API int dv_mix_delta_scan(const dvDeltaArgs* args, void* stream);
