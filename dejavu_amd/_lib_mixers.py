@@ -42,7 +42,7 @@ AttnArgs = _struct("AttnArgs", ("q", _p), ("ldq", _l), ("k", _p), ("ldk", _l), (
                    ("pos_dev", _p), ("pos_host", _i), ("out", _p), ("part", _p), ("splits", _i), ("fresh_k", _p),
                    ("fresh_v", _p), ("norm_dim", _i), ("eps", _f))
 DeltaArgs = _struct("DeltaArgs", ("q", _p), ("k", _p), ("v", _p), ("g", _p), ("beta", _p), ("S", _p), ("o", _p),
-                    ("n", _i), ("heads", _i), ("kv_heads", _i), ("dim_s", _i), ("vdim_s", _i))
+                    ("tm", _p), ("n", _i), ("heads", _i), ("kv_heads", _i), ("dim_s", _i), ("vdim_s", _i))
 DeltaStepArgs = _struct("DeltaStepArgs", ("p", _p), ("off_k", _i), ("off_v", _i), ("off_b", _i), ("off_a", _i),
                         ("off_g", _i), ("heads", _i), ("kv_heads", _i), ("dim", _i), ("dim_s", _i), ("vdim_s", _i),
                         ("Wa", _p), ("Wg", _p), ("rank_a", _i), ("rank_g", _i), ("A_log", _p), ("dt_bias", _p),
@@ -64,7 +64,7 @@ SIGNATURES = {
     "dv_mix_attn_rows": (_i, [_i, _i, _P(AttnArgs), _p]),
     "dv_mix_attn_tiles": (_i, [_P(AttnArgs), _i, _p]),
     "dv_mix_latent_absorb": (_i, [_i, _p, _p, _i, _i, _i, _p, _p]),
-    "dv_mix_latent_attn": (_i, [_i, _P(AttnArgs), _p, _p, _i, _p, _p]),
+    "dv_mix_latent_attn": (_i, [_i, _P(AttnArgs), _p, _i, _p, _p]),
     "dv_mix_delta_gates": (_i, [_i, _p, _l, _p, _l, _p, _p, _i, _i, _i, _p, _p, _p]),
     "dv_mix_delta_scan": (_i, [_P(DeltaArgs), _p]),
     "dv_mix_delta_step": (_i, [_i, _P(DeltaStepArgs), _p]),

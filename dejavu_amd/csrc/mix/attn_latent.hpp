@@ -35,26 +35,28 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(AttnArgs a) {
   const bf16_t* C = reinterpret_cast<const bf16_t*>(a.k);
   uint4_t cf[ST];
   auto fetch = [&](int jt) {
-    const int j = jt + wave * 16 + l16;
-    const uint4_t z = {0, 0, 0, 0};
+    // past the last token the weights are zero, past the last channel the queries are
+    const bf16_t* row = C + (int64_t)min(jt + wave * 16 + l16, j1 - 1) * a.ldk;
 #pragma unroll
-    for (int s = 0; s < ST; ++s) {
-      const int d = s * 32 + q4 * 8;
-      cf[s] = (j < j1 && d < rank) ? *reinterpret_cast<const uint4_t*>(C + (int64_t)j * a.ldk + d) : z;
-    }
+    for (int s = 0; s < ST; ++s) cf[s] = *reinterpret_cast<const uint4_t*>(row + min(s * 32 + q4 * 8, rank - 8));
   };
   if (j0 < j1) fetch(j0);
-  // queries as bf16, eight at a time
+  // queries as bf16, eight at a time, all of a thread's requested together
   const float* Q = reinterpret_cast<const float*>(a.q);
-  for (int i = tid; i < HT * 16 * RT * 2; i += 256) {
-    const int h = i / (RT * 2), d = i % (RT * 2) * 8;
-    bf16x8_t v;
-    Pack8<float> f;
-    f.zero();
-    if (h0 + h < a.H && d < rank) f.load(Q + (int64_t)(h0 + h) * rank + d);
+  constexpr int QN = HT * 16 * RT * 2 / 256 > 0 ? HT * 16 * RT * 2 / 256 : 1;
+  Pack8<float> qr[QN];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) v[e] = (bf16_t)f.get(e);
-    *reinterpret_cast<bf16x8_t*>(qs + h * QL + d) = v;
+  for (int u = 0; u < QN; ++u) {
+    const int i = u * 256 + tid, h = i / (RT * 2), d = i % (RT * 2) * 8;
+    qr[u].load(Q + (int64_t)min(h0 + h, a.H - 1) * rank + min(d, rank - 8));
+  }
+#pragma unroll
+  for (int u = 0; u < QN; ++u) {
+    const int i = u * 256 + tid, h = i / (RT * 2), d = i % (RT * 2) * 8;
+    bf16x8_t v;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] = (bf16_t)(d < rank ? qr[u].get(e) : 0.f);
+    if (h < HT * 16) *reinterpret_cast<bf16x8_t*>(qs + h * QL + d) = v;
   }
   float4_t o[TW][HT];
   float m[HT], l[HT];

@@ -29,6 +29,11 @@ __device__ __forceinline__ float attn_factor(const AttnArgs& a, int row, int hea
 
 constexpr int kAttnKeys = 64;
 
+// Floats for the sums of the key groups at the end of attn_rows_kernel.
+__host__ __device__ inline int attn_red_floats(int rh, int vdim_s) {
+  return vdim_s <= 256 && 4 * rh * vdim_s > 256 * 8 ? 4 * rh * vdim_s : 256 * 8;
+}
+
 // Grid: (splits, G * chunks of RH query heads, n).
 // Keys and values of a tile of 64 are requested together, before the queries are staged, so a split of one tile waits
 // for memory once.  With fresh_k / fresh_v this token's key and value come from LDS (and are stored in their slots).
@@ -36,8 +41,8 @@ template <typename T, typename TQ, int RH>
 __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
   float* qs = reinterpret_cast<float*>(smem_raw);  // [RH][dim_s]
-  float* red = qs + RH * a.dim_s;                  // [256][8]
-  T* kf = reinterpret_cast<T*>(red + 256 * 8);     // this token's key [dim_s] and value [vdim_s]
+  float* red = qs + RH * a.dim_s;
+  T* kf = reinterpret_cast<T*>(red + attn_red_floats(RH, a.vdim_s));     // this token's key [dim_s] and value [vdim_s]
   T* vf = kf + a.dim_s;
   __shared__ float ps[RH][kAttnKeys], corr[RH], ms[RH], ls[RH];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, sub = tid & 15;
@@ -53,7 +58,12 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
   const int fresh = a.fresh_k ? pos : -1;
   const T* K = reinterpret_cast<const T*>(a.k) + (int64_t)g * a.k_head;
   const T* V = reinterpret_cast<const T*>(a.v) + (int64_t)g * a.v_head;
-  auto slot = [&](int j) -> int64_t { return a.ring > 0 ? j % a.ring : j - a.base; };
+  // keys of a split lie in consecutive slots but for one wrap (a ring holds at least the window)
+  const int s0 = a.ring > 0 ? j0 % a.ring : j0 - a.base;
+  auto slot = [&](int j) -> int64_t {
+    const int s = s0 + (j - j0);
+    return a.ring > 0 && s >= a.ring ? s - a.ring : s;
+  };
   const int nc = a.vdim_s / 8, groups = 256 / nc;
   const int chunk = tid % nc, grp = tid / nc;
 
@@ -62,15 +72,13 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
   auto load_tile = [&](int jt) {
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
-      const int j = jt + u * 16 + (tid >> 4);
-      if (sub * 8 < a.dim_s && j < j1 && j != fresh) kv[u].load(K + slot(j) * a.ldk + sub * 8);
-      else kv[u].zero();
+      const int j = min(jt + u * 16 + (tid >> 4), j1 - 1);
+      kv[u].load(K + slot(j) * a.ldk + min(sub * 8, a.dim_s - 8));
     }
 #pragma unroll
     for (int u = 0; u < VU; ++u) {
-      const int j = jt + grp + u * groups;
-      if (grp < groups && grp + u * groups < kAttnKeys && j < j1 && j != fresh) vv[u].load(V + slot(j) * a.ldv + chunk * 8);
-      else vv[u].zero();
+      const int j = min(jt + grp + u * groups, j1 - 1);
+      vv[u].load(V + slot(j) * a.ldv + chunk * 8);
     }
   };
   if (j0 < j1) load_tile(j0);
@@ -135,8 +143,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
         const int j = jt + u * 16 + (tid >> 4);
         if (j == fresh && j < j1) kt[u] = *reinterpret_cast<const Pack8<T>*>(kf + c);
         else if (c < 128) kt[u] = kv[u];
-        else if (j < j1) kt[u].load(K + slot(j) * a.ldk + c);
-        else kt[u].zero();
+        else kt[u].load(K + slot(min(j, j1 - 1)) * a.ldk + c);
       }
 #pragma unroll
       for (int r = 0; r < RH; ++r) {
@@ -207,29 +214,58 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
     if (jt + kAttnKeys < j1) load_tile(jt + kAttnKeys);
     __syncthreads();
   }
-  // the key groups of a head are added up in LDS, one head at a time
+  // The key groups are added up: inside a wave by exchanges where whole groups lie side by side in it, the rest in
+  // LDS, a head at a time.
+  const bool pow2 = nc <= 32 && (nc & (nc - 1)) == 0;
+  if (pow2) {
+#pragma unroll
+    for (int r = 0; r < RH; ++r)
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        for (int off = 32; off >= nc; off >>= 1) acc[r][e] += __shfl_xor(acc[r][e], off, kWave);
+  }
+  auto finish = [&](int r, int d, float t) {
+    const int head = h0 + r;
+    if (a.splits == 1) {
+      float c;
+      const float f = attn_factor<TQ>(a, row, head, ms[r], ls[r], &c);
+      reinterpret_cast<T*>(a.out)[((int64_t)row * a.H + head) * a.vdim_s + d] = from_f<T>(t * c * f);
+    } else {
+      float* p = a.part + (((int64_t)row * a.H + head) * a.splits + split) * (a.vdim_s + 2);
+      p[d] = t;
+      if (d == 0) {
+        p[a.vdim_s] = ms[r];
+        p[a.vdim_s + 1] = ls[r];
+      }
+    }
+  };
+  if (pow2) {
+    // red holds [4 waves][RH][vdim_s] (at most 4 * RH * 256 floats)
+    if (lane < nc) {
+#pragma unroll
+      for (int r = 0; r < RH; ++r)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) red[(wave * RH + r) * a.vdim_s + lane * 8 + e] = acc[r][e];
+    }
+    __syncthreads();
+    for (int i = tid; i < nh * a.vdim_s; i += 256) {
+      const int r = i / a.vdim_s, d = i % a.vdim_s;
+      float t = 0.f;
+      for (int w = 0; w < 4; ++w) t += red[(w * RH + r) * a.vdim_s + d];
+      finish(r, d, t);
+    }
+    return;
+  }
 #pragma unroll
   for (int r = 0; r < RH; ++r) {
     if (r < nh) {
 #pragma unroll
       for (int e = 0; e < 8; ++e) red[tid * 8 + e] = acc[r][e];
       __syncthreads();
-      const int head = h0 + r;
-      float c = 1.f, f = 1.f;
-      if (a.splits == 1) f = attn_factor<TQ>(a, row, head, ms[r], ls[r], &c);
       for (int d = tid; d < a.vdim_s; d += 256) {
         float t = 0.f;
         for (int i = 0; i < groups; ++i) t += red[(i * nc + d / 8) * 8 + (d & 7)];
-        if (a.splits == 1) {
-          reinterpret_cast<T*>(a.out)[((int64_t)row * a.H + head) * a.vdim_s + d] = from_f<T>(t * c * f);
-        } else {
-          a.part[(((int64_t)row * a.H + head) * a.splits + split) * (a.vdim_s + 2) + d] = t;
-        }
-      }
-      if (a.splits > 1 && tid == 0) {
-        float* p = a.part + (((int64_t)row * a.H + head) * a.splits + split) * (a.vdim_s + 2) + a.vdim_s;
-        p[0] = ms[r];
-        p[1] = ls[r];
+        finish(r, d, t);
       }
       __syncthreads();
     }
@@ -239,41 +275,41 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
 // Adds up the splits of a (row, head): out[row][head][d].  Grid (H, ceil(vdim_s / 64), n); four groups of threads
 // share the splits of 64 entries.
 constexpr int kMaxSplits = 128;
+// By one wave: the weight of every split, and the maximum and denominator of all.
+__device__ __forceinline__ void split_weights(const float* __restrict__ p, int splits, int stride, int vdim_s, int lane,
+                                              float* ws, float* ml) {
+  const bool in0 = lane < splits, in1 = lane + 64 < splits;
+  const float* p0 = p + (int64_t)(in0 ? lane : 0) * stride + vdim_s;
+  const float* p1 = p + (int64_t)(in1 ? lane + 64 : 0) * stride + vdim_s;
+  const float m0 = in0 ? p0[0] : -1e30f, l0 = in0 ? p0[1] : 0.f, m1 = in1 ? p1[0] : -1e30f, l1 = in1 ? p1[1] : 0.f;
+  const float m = butterfly_max<64>(fmaxf(m0, m1));
+  const float w0 = exp_f(m0 - m), w1 = exp_f(m1 - m);
+  if (in0) ws[lane] = w0;
+  if (in1) ws[lane + 64] = w1;
+  const float l = wave_sum(w0 * l0 + w1 * l1);
+  if (lane == 0) {
+    ml[0] = m;
+    ml[1] = l;
+  }
+}
 template <typename TO, typename TQ>
 __global__ __launch_bounds__(256) void attn_merge_kernel(AttnArgs a, TO* __restrict__ out) {
   __shared__ float ws[kMaxSplits], acc[4][64], ml[2];
   const int head = blockIdx.x, row = blockIdx.z, stride = a.vdim_s + 2, lane = threadIdx.x & 63, grp = threadIdx.x >> 6;
   const float* p = a.part + ((int64_t)row * a.H + head) * a.splits * stride;
-  if (grp == 0) {
-    float m0 = -1e30f, m1 = -1e30f, l = 0.f;
-    if (lane < a.splits) m0 = p[(int64_t)lane * stride + a.vdim_s];
-    if (lane + 64 < a.splits) m1 = p[(int64_t)(lane + 64) * stride + a.vdim_s];
-    const float m = butterfly_max<64>(fmaxf(m0, m1));
-    const float w0 = exp_f(m0 - m), w1 = exp_f(m1 - m);
-    if (lane < a.splits) {
-      ws[lane] = w0;
-      l = w0 * p[(int64_t)lane * stride + a.vdim_s + 1];
-    }
-    if (lane + 64 < a.splits) {
-      ws[lane + 64] = w1;
-      l = __builtin_fmaf(w1, p[(int64_t)(lane + 64) * stride + a.vdim_s + 1], l);
-    }
-    l = wave_sum(l);
-    if (lane == 0) {
-      ml[0] = m;
-      ml[1] = l;
-    }
-  }
-  __syncthreads();
   const int d = blockIdx.y * 64 + lane;
+  constexpr int PV = 16;  // sums requested before the weights are known
+  float v[PV];
+#pragma unroll
+  for (int i = 0; i < PV; ++i) v[i] = d < a.vdim_s && grp + 4 * i < a.splits ? p[(int64_t)(grp + 4 * i) * stride + d] : 0.f;
+  if (grp == 0) split_weights(p, a.splits, stride, a.vdim_s, lane, ws, ml);
+  __syncthreads();
   float t = 0.f;
-  if (d < a.vdim_s) {
-#pragma unroll 4
-    for (int s = grp; s < a.splits; s += 4) {
-      const float w = ws[s];
-      if (w > 0.f) t = __builtin_fmaf(p[(int64_t)s * stride + d], w, t);  // splits without tokens hold no sums
-    }
-  }
+#pragma unroll
+  for (int i = 0; i < PV; ++i)
+    if (grp + 4 * i < a.splits) t = __builtin_fmaf(v[i], ws[grp + 4 * i], t);
+  if (d < a.vdim_s)
+    for (int s = grp + 4 * PV; s < a.splits; s += 4) t = __builtin_fmaf(p[(int64_t)s * stride + d], ws[s], t);
   acc[grp][lane] = t;
   __syncthreads();
   if (grp == 0 && d < a.vdim_s) {
@@ -315,23 +351,51 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(const float* __restr
   }
 }
 
-// Latent attention, one decode row: out[h] = W_uv[h] lat[h], lat fp32 [H][rank].  Grid (H, row parts).
+// Latent attention, one decode row: merges the splits of head h, gates, and applies W_uv[h].  Grid (H, row parts):
+// every part merges the whole latent for itself.  The first weights are requested before anything else.
 template <typename T>
-__global__ __launch_bounds__(256) void latent_out_kernel(const float* __restrict__ lat_all, const T* __restrict__ W,
-                                                         int rank, int vrows, T* __restrict__ out) {
+__global__ __launch_bounds__(256) void latent_out_kernel(AttnArgs a, const T* __restrict__ W, int vrows, T* __restrict__ out) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
   float* lat = reinterpret_cast<float*>(smem_raw);
-  const int head = blockIdx.x, lane = threadIdx.x & 63;
-  for (int d = threadIdx.x; d < rank; d += 256) lat[d] = lat_all[(int64_t)head * rank + d];
-  __syncthreads();
-  for (int r = blockIdx.y * 4 + (threadIdx.x >> 6); r < vrows; r += gridDim.y * 4) {
-    const T* w = W + ((int64_t)head * vrows + r) * rank;
-    float acc = 0.f;
-    for (int i = lane * 8; i < rank; i += 512) {
-      Pack8<T> v;
-      v.load(w + i);
+  __shared__ float ws[kMaxSplits], ml[2];
+  const int head = blockIdx.x, rank = a.vdim_s, stride = rank + 2, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const float* p = a.part + (int64_t)head * a.splits * stride;
+  constexpr int PR = 4;  // weight rows a wave requests ahead
+  Pack8<T> w[PR];
+  const int r0 = blockIdx.y * 4 + wave, rstep = gridDim.y * 4;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) acc = __builtin_fmaf(v.get(e), lat[i + e], acc);
+  for (int i = 0; i < PR; ++i) {
+    const int r = r0 + i * rstep;
+    if (r < vrows && lane * 8 < rank) w[i].load(W + ((int64_t)head * vrows + r) * rank + lane * 8);
+    else w[i].zero();
+  }
+  if (wave == 0) split_weights(p, a.splits, stride, rank, lane, ws, ml);
+  __syncthreads();
+  float c;
+  const float f = attn_factor<float>(a, 0, head, ml[0], ml[1], &c) * c;
+  typedef float float2_v __attribute__((ext_vector_type(2)));
+  for (int d = threadIdx.x * 2; d < rank; d += 512) {
+    float2_v t = {0.f, 0.f};
+#pragma unroll 16
+    for (int s = 0; s < a.splits; ++s) t += *reinterpret_cast<const float2_v*>(p + (int64_t)s * stride + d) * ws[s];
+    lat[d] = t[0] * f;
+    lat[d + 1] = t[1] * f;
+  }
+  __syncthreads();
+  for (int i = 0, r = r0; r < vrows; ++i, r += rstep) {
+    const T* wr = W + ((int64_t)head * vrows + r) * rank;
+    float acc = 0.f;
+    for (int k = lane * 8; k < rank; k += 512) {
+      Pack8<T> v;
+      if (k < 512 && i < PR) {
+#pragma unroll
+        for (int u = 0; u < PR; ++u)
+          if (u == i) v = w[u];
+      } else {
+        v.load(wr + k);
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) acc = __builtin_fmaf(v.get(e), lat[k + e], acc);
     }
     acc = wave_sum(acc);
     if (lane == 0) out[(int64_t)head * vrows + r] = from_f<T>(acc);

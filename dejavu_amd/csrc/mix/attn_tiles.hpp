@@ -48,18 +48,17 @@ __global__ __launch_bounds__(256) void attn_tiles_kernel(AttnArgs a, int keys /*
   constexpr int VV = (kTileK / 2 * VT * 4 + 255) / 256;   // pairs of 16-byte loads of V per thread
   uint4_t kr[KV], vr[VV][2];
   auto fetch = [&](int k0) {
-    const uint4_t z = {0, 0, 0, 0};
+    // past the last key the weights are zero; past the last channel the queries are, or nothing is stored
 #pragma unroll
     for (int i = 0; i < KV; ++i) {
       const int at = i * 256 + tid, r = at / (DT * 2), d = at % (DT * 2) * 8;
-      kr[i] = (r < kTileK && k0 + r < keys && d < a.dim_s) ? *reinterpret_cast<const uint4_t*>(K + (int64_t)(k0 + r) * a.ldk + d) : z;
+      kr[i] = *reinterpret_cast<const uint4_t*>(K + (int64_t)min(k0 + r, keys - 1) * a.ldk + min(d, a.dim_s - 8));
     }
 #pragma unroll
     for (int i = 0; i < VV; ++i) {
-      const int at = i * 256 + tid, r = at % (kTileK / 2) * 2, d = at / (kTileK / 2) * 8;
-      const bool ok = d < a.vdim_s;
-      vr[i][0] = ok && k0 + r < keys ? *reinterpret_cast<const uint4_t*>(V + (int64_t)(k0 + r) * a.ldv + d) : z;
-      vr[i][1] = ok && k0 + r + 1 < keys ? *reinterpret_cast<const uint4_t*>(V + (int64_t)(k0 + r + 1) * a.ldv + d) : z;
+      const int at = i * 256 + tid, r = at % (kTileK / 2) * 2, d = min(at / (kTileK / 2) * 8, a.vdim_s - 8);
+      vr[i][0] = *reinterpret_cast<const uint4_t*>(V + (int64_t)min(k0 + r, keys - 1) * a.ldv + d);
+      vr[i][1] = *reinterpret_cast<const uint4_t*>(V + (int64_t)min(k0 + r + 1, keys - 1) * a.ldv + d);
     }
   };
   auto put = [&]() {

@@ -1,11 +1,17 @@
-// Gated delta rule with one decay per head and key channel; the state is fp32 and stays in registers while a
-// portion is walked.
+// Gated delta rule with one decay per head and key channel, in fp32.
 //
 //   S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
 //
-// The columns of S (value channels) are independent: a workgroup owns 16 columns of one head, a row of 16 lanes
-// one column, a lane the key channels 64 c + 4 s .. + 3 (s: lane of the row).  Both reductions over the key
-// channels are taken of the decayed state, o = (diag(g) S)^T q + (k . q) u, so a token has one dependent reduction.
+// A portion is walked in chunks of 16 tokens.  With P(i, j) = g_{j+1} .. g_i per channel (products, never exponentials
+// of summed logarithms: they are as exact as the token-by-token recurrence and cannot overflow) and S_0 the state at
+// the start of the chunk,
+//
+//   L[i, j] = sum_d k_i k_j P(i, j)  (j < i)     M[i, j] = sum_d q_i k_j P(i, j)  (j <= i)
+//   U = T (V - Kt S_0),  T = (1 + diag(beta) L)^-1 diag(beta),  Kt_i = P(i, 0) k_i  (g_1 included)
+//   O = Qt S_0 + M U,    S = P(16, 0) S_0 + Kh^T U,             Kh_j = P(16, j) k_j
+//
+// T and M depend on no state: one kernel makes them for all chunks at once.  The second kernel carries the state from
+// chunk to chunk; its products run on the fp32 matrix instructions.  A decode step uses the recurrence itself.
 // State layout [heads][vdim][dim] (key channels contiguous).
 #pragma once
 #include "elem.hpp"
@@ -75,116 +81,253 @@ __device__ __forceinline__ void store_state(const float (&S)[E], float* __restri
   }
 }
 
-constexpr int kDeltaTokens = 16;  // tokens staged at a time (one 16-lane row each for k . q)
-constexpr int kDeltaCols = 16;    // columns of S per workgroup
+constexpr int kDeltaCols = 16;   // columns of S per workgroup
+constexpr int kDeltaChunk = 16;  // tokens per chunk
 
-// A portion of n tokens.  Grid: heads * ceil(vdim_s / 16) workgroups, head fastest.
+// T and M of a chunk and head: tm[(chunk * heads + head) * 512] = T [16][16], then M [16][16].  A row of 16 lanes owns
+// key j and walks the later tokens.  Grid: (heads, chunks); D = 16 E >= dim_s.
 template <int E>
-__global__ __launch_bounds__(256) void delta_scan_kernel(DeltaArgs a) {
-  constexpr int D = 16 * E, TC = kDeltaTokens;
-  constexpr int V4 = TC * D / 4 / 256;  // float4 per thread and tensor (E / 4)
-  constexpr int NB = E <= 8 ? 2 : 1;    // staging buffers
-  __shared__ __attribute__((aligned(16))) float sq[NB][TC][D], sk[NB][TC][D], sg[NB][TC][D];
-  __shared__ float sv[NB][TC][kDeltaCols], sb[NB][TC], skq[NB][TC];
-  const int head = blockIdx.x % a.heads, tile = blockIdx.x / a.heads;
-  const int kvh = head / (a.heads / a.kv_heads);
-  const int tid = threadIdx.x, sub = tid & 15;
-  const int colw = tid >> 4, col = tile * kDeltaCols + colw;  // the 16 rows of 16 lanes: one column each
-  const bool col_ok = col < a.vdim_s;
-  float S[E];
-  float* sp = a.S + ((int64_t)head * a.vdim_s + (col_ok ? col : 0)) * a.dim_s;
-  load_state<E>(S, sp, sub, a.dim_s, col_ok);
-
-  float4_t rq[V4], rk[V4], rg[V4];
-  float rv, rb = 0.f;
-  auto fetch = [&](int t0) {
+__global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaArgs a) {
+  constexpr int D = 16 * E, C = kDeltaChunk;
+  extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
+  float* sq = reinterpret_cast<float*>(smem_raw);  // [16][D] each
+  float* sk = sq + C * D;
+  float* sg = sk + C * D;
+  __shared__ __attribute__((aligned(16))) float L[C][C], M[C][C];
+  __shared__ float sb[C];
+  const int head = blockIdx.x, t0 = blockIdx.y * C, kvh = head / (a.heads / a.kv_heads);
+  const int tid = threadIdx.x, sub = tid & 15, j = tid >> 4;
 #pragma unroll
-    for (int i = 0; i < V4; ++i) {
-      const int at = (i * 256 + tid) * 4, t = at / D, d = at % D;
-      const bool ok = t0 + t < a.n && d < a.dim_s;
-      const float4_t z = {0.f, 0.f, 0.f, 0.f};
-      const int64_t kvat = ((int64_t)(t0 + t) * a.kv_heads + kvh) * a.dim_s + d;
-      rq[i] = ok ? *reinterpret_cast<const float4_t*>(a.q + kvat) : z;
-      rk[i] = ok ? *reinterpret_cast<const float4_t*>(a.k + kvat) : z;
-      rg[i] = ok ? *reinterpret_cast<const float4_t*>(a.g + ((int64_t)(t0 + t) * a.heads + head) * a.dim_s + d) : z;
-    }
-    const int t = t0 + (tid >> 4), c = tile * kDeltaCols + sub;
-    rv = (t < a.n && c < a.vdim_s) ? a.v[((int64_t)t * a.heads + head) * a.vdim_s + c] : 0.f;
-    if (sub == 0) rb = t < a.n ? a.beta[(int64_t)t * a.heads + head] : 0.f;
-  };
-  auto put = [&](int buf) {
+  for (int i = 0; i < E / 4; ++i) {
+    const int at = (i * 256 + tid) * 4, t = at / D, d = at % D;
+    const bool ok = t0 + t < a.n && d < a.dim_s;
+    const int64_t row = min(t0 + t, a.n - 1);
+    const int dc = min(d, a.dim_s - 4);
+    const float4_t z = {0.f, 0.f, 0.f, 0.f};
+    const float4_t q = *reinterpret_cast<const float4_t*>(a.q + (row * a.kv_heads + kvh) * a.dim_s + dc);
+    const float4_t k = *reinterpret_cast<const float4_t*>(a.k + (row * a.kv_heads + kvh) * a.dim_s + dc);
+    const float4_t g = *reinterpret_cast<const float4_t*>(a.g + (row * a.heads + head) * a.dim_s + dc);
+    *reinterpret_cast<float4_t*>(sq + at) = ok ? q : z;
+    *reinterpret_cast<float4_t*>(sk + at) = ok ? k : z;
+    *reinterpret_cast<float4_t*>(sg + at) = ok ? g : z;
+  }
+  if (tid < C) sb[tid] = t0 + tid < a.n ? a.beta[(int64_t)(t0 + tid) * a.heads + head] : 0.f;
+  L[j][sub] = 0.f;
+  M[j][sub] = 0.f;
+  __syncthreads();
+  float4_t p[E / 4];  // k_j P(i, j)
 #pragma unroll
-    for (int i = 0; i < V4; ++i) {
-      const int at = (i * 256 + tid) * 4;
-      *reinterpret_cast<float4_t*>(&sq[buf][0][0] + at) = rq[i];
-      *reinterpret_cast<float4_t*>(&sk[buf][0][0] + at) = rk[i];
-      *reinterpret_cast<float4_t*>(&sg[buf][0][0] + at) = rg[i];
-    }
-    sv[buf][tid >> 4][sub] = rv;
-    if (sub == 0) sb[buf][tid >> 4] = rb;
-  };
-  auto dot_kq = [&](int buf) {
-    float d = 0.f;
-    const int t = tid >> 4;
+  for (int c = 0; c < E / 4; ++c) p[c] = *reinterpret_cast<const float4_t*>(sk + j * D + c * 64 + sub * 4);
+  for (int i = j; i < C; ++i) {
+    float kk = 0.f, qk = 0.f;
 #pragma unroll
     for (int c = 0; c < E / 4; ++c) {
-      const float4_t x = *reinterpret_cast<const float4_t*>(&sk[buf][t][c * 64 + sub * 4]);
-      const float4_t y = *reinterpret_cast<const float4_t*>(&sq[buf][t][c * 64 + sub * 4]);
+      const int at = i * D + c * 64 + sub * 4;
+      const float4_t qv = *reinterpret_cast<const float4_t*>(sq + at), kv = *reinterpret_cast<const float4_t*>(sk + at);
+      if (i > j) p[c] *= *reinterpret_cast<const float4_t*>(sg + at);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) d = __builtin_fmaf(x[e], y[e], d);
+      for (int e = 0; e < 4; ++e) {
+        kk = __builtin_fmaf(p[c][e], kv[e], kk);
+        qk = __builtin_fmaf(p[c][e], qv[e], qk);
+      }
     }
-    d = row16_sum(d);
-    if (sub == 0) skq[buf][t] = d;
+    kk = row16_sum(kk);
+    qk = row16_sum(qk);
+    if (sub == 0) {
+      M[i][j] = qk;
+      if (i > j) L[i][j] = sb[i] * kk;
+    }
+  }
+  __syncthreads();
+  float* out = a.tm + ((int64_t)blockIdx.y * a.heads + head) * 512;
+  if (tid < C) {  // column tid of T by forward substitution
+    float x[C];
+#pragma unroll
+    for (int i = 0; i < C; ++i) {
+      float v = i == tid ? sb[i] : 0.f;
+#pragma unroll
+      for (int k = 0; k < i; ++k) v = __builtin_fmaf(-L[i][k], x[k], v);
+      x[i] = v;
+      out[i * C + tid] = v;
+    }
+  }
+  out[256 + tid] = M[j][sub];
+}
+
+// Chunk after chunk for 16 columns of a head.  Wave w owns key channels [16 NT w, 16 NT (w + 1)) of the state, as
+// accumulators of the 16x16x4 products: element i of a lane is channel 4 (lane / 16) + i of a tile, column lane % 16,
+// which is also the operand layout of the products with Kt and Qt when their channels are taken in that order.  The
+// four waves' partial products meet in LDS once per chunk; U is then made by every wave for itself.
+template <int NT>
+struct DeltaChunkLds {
+  static constexpr int D = 64 * NT, KL = D + 4, TL = 20;
+  float kt[16 * KL], qt[16 * KL];  // [token][channel]
+  float kh[D * TL];                // [channel][token]
+  float tmat[16 * TL], mmat[16 * TL];
+  float v[16 * 16];                // [token][column]
+  float gc[D];                     // decay over the whole chunk
+};
+template <int NT>
+constexpr size_t delta_scan_lds_bytes() {
+  return 2 * sizeof(DeltaChunkLds<NT>) + 2 * 4 * 2 * 64 * 16;  // two stages; partial products, two stages
+}
+
+// Grid: heads * ceil(vdim_s / 16), head fastest (the workgroups of a head share an XCD's L2 when heads % 8 == 0).
+template <int NT>
+__global__ __launch_bounds__(256) void delta_scan_kernel(DeltaArgs a) {
+  using Lds = DeltaChunkLds<NT>;
+  constexpr int D = Lds::D, KL = Lds::KL, TL = Lds::TL, C = kDeltaChunk;
+  constexpr int IT = (2 * D + 255) / 256;  // (role, channel) items per thread
+  extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
+  Lds* st = reinterpret_cast<Lds*>(smem_raw);
+  float4_t* part = reinterpret_cast<float4_t*>(smem_raw + 2 * sizeof(Lds));  // [stage][wave][2][64]
+  const int head = blockIdx.x % a.heads, tile = blockIdx.x / a.heads;
+  const int kvh = head / (a.heads / a.kv_heads);
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int l16 = lane & 15, q4 = lane >> 4;
+  const int col = tile * kDeltaCols + l16;
+  const bool col_ok = col < a.vdim_s;
+  float* sp = a.S + ((int64_t)head * a.vdim_s + (col_ok ? col : 0)) * a.dim_s;
+  float4_t S[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    const int d = (wave * NT + t) * 16 + q4 * 4;
+    S[t] = (col_ok && d < a.dim_s) ? *reinterpret_cast<const float4_t*>(sp + d) : float4_t{0.f, 0.f, 0.f, 0.f};
+  }
+
+  // staging: role 0 makes Kt and Qt of a channel, role 1 Kh and the chunk's decay
+  float rg[IT][C], rk[IT][C], rq[IT][C], rtm[2], rv;
+  const int gs = a.heads * a.dim_s, ks_ = a.kv_heads * a.dim_s;  // elements between tokens
+  const int vc = min(tile * kDeltaCols + (tid & 15), a.vdim_s - 1);
+  auto fetch = [&](int t0) {
+    const float* gp = a.g + (int64_t)t0 * gs + head * a.dim_s;
+    const float* kp = a.k + (int64_t)t0 * ks_ + kvh * a.dim_s;
+    const float* qp = a.q + (int64_t)t0 * ks_ + kvh * a.dim_s;
+    const int last = a.n - 1 - t0;
+#pragma unroll
+    for (int it = 0; it < IT; ++it) {
+      const int d = min((it * 256 + tid) % D, a.dim_s - 1);
+#pragma unroll
+      for (int t = 0; t < C; ++t) {
+        const int row = min(t, last);
+        rg[it][t] = gp[row * gs + d];
+        rk[it][t] = kp[row * ks_ + d];
+        rq[it][t] = qp[row * ks_ + d];
+      }
+    }
+    const float* tm = a.tm + ((int64_t)(t0 / C) * a.heads + head) * 512;
+    rtm[0] = tm[tid];
+    rtm[1] = tm[256 + tid];
+    rv = a.v[((int64_t)t0 + min(tid >> 4, last)) * a.heads * a.vdim_s + head * a.vdim_s + vc];
+  };
+  auto put = [&](Lds& b, int t0) {
+    // what was read past the end of the portion or of the channels
+    const int cnt = a.n - t0;
+#pragma unroll
+    for (int it = 0; it < IT; ++it) {
+      const bool in = (it * 256 + tid) % D < a.dim_s;
+#pragma unroll
+      for (int t = 0; t < C; ++t) {
+        if (!in || t >= cnt) {
+          rg[it][t] = 1.f;
+          rk[it][t] = 0.f;
+          rq[it][t] = 0.f;
+        }
+      }
+    }
+    if ((tid >> 4) >= cnt) rv = 0.f;
+#pragma unroll
+    for (int it = 0; it < IT; ++it) {
+      const int item = it * 256 + tid, role = item / D, d = item % D;
+      if (item < 2 * D) {
+        if (role == 0) {
+          float p = 1.f;
+#pragma unroll
+          for (int t = 0; t < C; ++t) {
+            p *= rg[it][t];
+            b.kt[t * KL + d] = p * rk[it][t];
+            b.qt[t * KL + d] = p * rq[it][t];
+          }
+        } else {
+          float p = 1.f;
+          float kh[C];
+#pragma unroll
+          for (int t = C - 1; t >= 0; --t) {
+            kh[t] = p * rk[it][t];
+            p *= rg[it][t];
+          }
+          b.gc[d] = p;
+#pragma unroll
+          for (int t = 0; t < C; t += 4)
+            *reinterpret_cast<float4_t*>(&b.kh[d * TL + t]) = float4_t{kh[t], kh[t + 1], kh[t + 2], kh[t + 3]};
+        }
+      }
+    }
+    b.tmat[(tid >> 4) * TL + (tid & 15)] = rtm[0];
+    b.mmat[(tid >> 4) * TL + (tid & 15)] = rtm[1];
+    b.v[tid] = rv;
   };
 
   fetch(0);
-  put(0);
+  put(st[0], 0);
   __syncthreads();
-  dot_kq(0);
-  __syncthreads();
-  for (int t0 = 0, buf = 0; t0 < a.n; t0 += TC, buf = (buf + 1) % NB) {
-    const bool more = t0 + TC < a.n;
-    if (more) fetch(t0 + TC);
-    const int cnt = a.n - t0 < TC ? a.n - t0 : TC;
-    float mine = 0.f;  // lane s keeps the read-out of token s
-    DeltaToken<E> cur, nxt;
-    auto get = [&](DeltaToken<E>& d, int t) {
-      d.load(sq[buf][t], sk[buf][t], sg[buf][t], sub, sv[buf][t][colw], sb[buf][t], skq[buf][t]);
-    };
-    auto run = [&](const DeltaToken<E>& d, int t) {
-      const float o = delta_step<E>(S, d);
-      if (sub == t) mine = o;
-    };
-    get(cur, 0);
-    if (cnt == TC) {  // the operands of a token are requested one token ahead
+  for (int t0 = 0, buf = 0; t0 < a.n; t0 += C, buf ^= 1) {
+    const Lds& b = st[buf];
+    const bool more = t0 + C < a.n;
+    if (more) fetch(t0 + C);
+    // partial Kt S and Qt S over this wave's channels
+    float4_t ks = {0.f, 0.f, 0.f, 0.f}, qs = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int t = 0; t < TC; t += 2) {
-        get(nxt, t + 1);
-        __builtin_amdgcn_sched_barrier(0);
-        run(cur, t);
-        __builtin_amdgcn_sched_barrier(0);
-        if (t + 2 < TC) get(cur, t + 2);
-        __builtin_amdgcn_sched_barrier(0);
-        run(nxt, t + 1);
-        __builtin_amdgcn_sched_barrier(0);
-      }
-    } else {
-      for (int t = 0; t < cnt; ++t) {
-        get(cur, t);
-        run(cur, t);
+    for (int t = 0; t < NT; ++t) {
+      const int d = (wave * NT + t) * 16 + q4 * 4;
+      const float4_t kt = *reinterpret_cast<const float4_t*>(&b.kt[l16 * KL + d]);
+      const float4_t qt = *reinterpret_cast<const float4_t*>(&b.qt[l16 * KL + d]);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        ks = __builtin_amdgcn_mfma_f32_16x16x4f32(kt[i], S[t][i], ks, 0, 0, 0);
+        qs = __builtin_amdgcn_mfma_f32_16x16x4f32(qt[i], S[t][i], qs, 0, 0, 0);
       }
     }
-    if (col_ok && sub < cnt) a.o[((int64_t)(t0 + sub) * a.heads + head) * a.vdim_s + col] = mine;
-    if (more) {
-      const int nb = (buf + 1) % NB;
-      if (NB == 1) __syncthreads();  // everybody is done with the only buffer
-      put(nb);
-      __syncthreads();
-      dot_kq(nb);
-      __syncthreads();
+    float4_t* pp = part + buf * 512;
+    pp[wave * 128 + lane] = ks;
+    pp[wave * 128 + 64 + lane] = qs;
+    __syncthreads();
+    float4_t w;  // V - Kt S: tokens 4 q4 .. + 3 of this lane's column
+    const float4_t sum = (pp[lane] + pp[128 + lane]) + (pp[256 + lane] + pp[384 + lane]);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) w[i] = b.v[(q4 * 4 + i) * 16 + l16] - sum[i];
+    const float4_t tm = *reinterpret_cast<const float4_t*>(&b.tmat[l16 * TL + q4 * 4]);
+    float4_t u = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < 4; ++i) u = __builtin_amdgcn_mfma_f32_16x16x4f32(tm[i], w[i], u, 0, 0, 0);
+    if (wave == 3) {
+      float4_t o = (pp[64 + lane] + pp[192 + lane]) + (pp[320 + lane] + pp[448 + lane]);
+      const float4_t mm = *reinterpret_cast<const float4_t*>(&b.mmat[l16 * TL + q4 * 4]);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) o = __builtin_amdgcn_mfma_f32_16x16x4f32(mm[i], u[i], o, 0, 0, 0);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = t0 + q4 * 4 + i;
+        if (col_ok && t < a.n) a.o[((int64_t)t * a.heads + head) * a.vdim_s + col] = o[i];
+      }
     }
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+      const int d0 = (wave * NT + t) * 16;
+      const float4_t gc = *reinterpret_cast<const float4_t*>(&b.gc[d0 + q4 * 4]);
+      const float4_t kh = *reinterpret_cast<const float4_t*>(&b.kh[(d0 + l16) * TL + q4 * 4]);
+      S[t] *= gc;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(kh[i], u[i], S[t], 0, 0, 0);
+    }
+    if (more) put(st[buf ^ 1], t0 + C);  // that stage was read before the barrier above
+    __syncthreads();
   }
-  store_state<E>(S, sp, sub, a.dim_s, col_ok);
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    const int d = (wave * NT + t) * 16 + q4 * 4;
+    if (col_ok && d < a.dim_s) *reinterpret_cast<float4_t*>(sp + d) = S[t];
+  }
 }
 
 // g = exp(-exp(A_log) softplus(z + dt_bias)), beta = sigmoid(b).  Four channels of a head per thread (dim_s % 4 == 0).

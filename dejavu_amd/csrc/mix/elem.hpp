@@ -98,6 +98,9 @@ __device__ __forceinline__ float dyn_tanh(float x, const DynTanh& n, int c) {
   return __builtin_fmaf(tanh_f(n.alpha * x), n.w[c], n.b[c]);
 }
 
+// Loads below are unconditional from clamped addresses wherever a bound can be met (what lies past it is masked where
+// it is used): a guarded load becomes a branch, and a row of branches keeps few loads in flight.
+
 // The sequence position of a call: on the device (captured decode steps) or passed by the host.
 __device__ __forceinline__ int seq_position(const int* dev, int host) { return dev ? *dev : host; }
 

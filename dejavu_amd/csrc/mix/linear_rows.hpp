@@ -107,7 +107,7 @@ __global__ __launch_bounds__(256) void linear_rows_kernel(RowsArgs a) {
 #pragma unroll
     for (int r = 0; r < R; ++r) {
       const int row = task * R + r;
-      wr[r] = W + (int64_t)(row < a.M ? row : 0) * a.ldw + lane * 8;
+      wr[r] = W + (int64_t)(row < a.M ? row : 0) * a.ldw;
     }
   };
   auto load_w = [&](int base) {
@@ -115,8 +115,7 @@ __global__ __launch_bounds__(256) void linear_rows_kernel(RowsArgs a) {
     for (int u = 0; u < U; ++u)
 #pragma unroll
       for (int r = 0; r < R; ++r) {
-        if (base + u * CH + lane * 8 < K) w[u][r].load_stream(wr[r] + base + u * CH);
-        else w[u][r].zero();
+        w[u][r].load_stream(wr[r] + min(base + u * CH + lane * 8, K - 8));
       }
   };
   if (t < ntasks) {  // the first weights are requested before x is there

@@ -25,12 +25,12 @@ __global__ __launch_bounds__(256) void linear_tiles_kernel(TileArgs a) {
 #pragma unroll
   for (int i = 0; i < RT; ++i) {
     const int m = m0 + i * 16 + r16;
-    wp[i] = W + (int64_t)(m < a.M ? m : 0) * a.ldw + kq;
+    wp[i] = W + (int64_t)(m < a.M ? m : 0) * a.ldw;
   }
 #pragma unroll
   for (int i = 0; i < NT; ++i) {
     const int n = n0 + i * 16 + r16;
-    xp[i] = X + (int64_t)(n < a.n ? n : 0) * a.ldx + kq;
+    xp[i] = X + (int64_t)(n < a.n ? n : 0) * a.ldx;
   }
   float4_t acc[RT][NT];
 #pragma unroll
@@ -41,18 +41,21 @@ __global__ __launch_bounds__(256) void linear_tiles_kernel(TileArgs a) {
     Pack8<bf16_t> w[U][RT], x[U][NT];
 #pragma unroll
     for (int u = 0; u < U; ++u) {
-      const int k = k0 + u * 32;
-      const bool in = k + kq < a.K;
+      const int k = min(k0 + u * 32 + kq, a.K - 8);
 #pragma unroll
-      for (int i = 0; i < RT; ++i) {
-        if (in) w[u][i].load(wp[i] + k);
-        else w[u][i].zero();
-      }
+      for (int i = 0; i < RT; ++i) w[u][i].load(wp[i] + k);
 #pragma unroll
-      for (int j = 0; j < NT; ++j) {
-        if (in) x[u][j].load(xp[j] + k);
-        else x[u][j].zero();
-      }
+      for (int j = 0; j < NT; ++j) x[u][j].load(xp[j] + k);
+    }
+    if (k0 + 32 * U > a.K) {  // past the end of the rows
+#pragma unroll
+      for (int u = 0; u < U; ++u)
+#pragma unroll
+        for (int j = 0; j < NT; ++j)
+          if (k0 + u * 32 + kq >= a.K) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) x[u][j].v[e] = 0u;
+          }
     }
 #pragma unroll
     for (int u = 0; u < U; ++u)

@@ -9,7 +9,7 @@ using ConvArgs = dvConvArgs;
 
 // A lane owns eight channels of one head and walks TB consecutive tokens with the last TAPS inputs in registers; the
 // LPH lanes of a head (a power of two, 8 LPH >= stride) add up its norm.  Grid: (units of heads, token blocks).
-constexpr int kConvTokens = 8;
+constexpr int kConvTokens = 16;
 
 template <int LPH>
 __device__ __forceinline__ float lanes_sum(float v) {
@@ -26,7 +26,7 @@ template <typename T, typename TO, int LPH, int TAPS>
 __global__ __launch_bounds__(256) void short_conv_kernel(ConvArgs a) {
   constexpr int HPB = 256 / LPH;  // heads per workgroup
   const int heads = a.g[0].heads + a.g[1].heads + a.g[2].heads;
-  const int unit = blockIdx.x * HPB + threadIdx.x / LPH, c = threadIdx.x % LPH * 8;
+  const int unit = blockIdx.x * HPB + threadIdx.x / LPH, c0 = threadIdx.x % LPH * 8;
   int h = unit < heads ? unit : 0, base = 0, gi = 0;
   if (h >= a.g[0].heads) {
     h -= a.g[0].heads;
@@ -39,29 +39,37 @@ __global__ __launch_bounds__(256) void short_conv_kernel(ConvArgs a) {
     }
   }
   const ConvGroup g = a.g[gi];
-  const bool on = unit < heads && c < g.stride;
+  const bool on = unit < heads && c0 < g.stride;
+  const int c = min(c0, g.stride - 8);
   const int ch = base + h * g.stride + c;
   const T* in = reinterpret_cast<const T*>(a.in) + ch;
   float w[TAPS][8], u[TAPS][8];
+  {
+    float4_t wv[TAPS * 2];  // eight channels x TAPS, contiguous
 #pragma unroll
-  for (int j = 0; j < TAPS; ++j)
+    for (int i = 0; i < TAPS * 2; ++i)
+      wv[i] = *reinterpret_cast<const float4_t*>(a.w + (int64_t)ch * TAPS + i * 4);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) w[j][e] = on ? a.w[(int64_t)(ch + e) * TAPS + j] : 0.f;
+    for (int e = 0; e < 8; ++e)
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) w[j][e] = wv[(e * TAPS + j) >> 2][(e * TAPS + j) & 3];
+  }
   const int t0 = blockIdx.y * kConvTokens, t1 = min(a.n, t0 + kConvTokens);
   Pack8<T> next[kConvTokens];
 #pragma unroll
   for (int i = 0; i < kConvTokens; ++i) {
-    if (on && t0 + i < t1) next[i].load(in + (int64_t)(t0 + i) * a.ldi);
-    else next[i].zero();
+    next[i].load(in + (int64_t)min(t0 + i, t1 - 1) * a.ldi);
   }
 #pragma unroll
   for (int j = 0; j < TAPS - 1; ++j) {  // the inputs before the block
     const int s = t0 - (TAPS - 1) + j;
+    Pack8<T> v;
+    v.load(in + (int64_t)max(s, 0) * a.ldi);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      float x = 0.f;
-      if (on) x = s >= 0 ? to_f(in[(int64_t)s * a.ldi + e]) : a.state[(int64_t)(ch + e) * (TAPS - 1) + TAPS - 1 + s];
-      u[j][e] = x;
+    for (int e = 0; e < 8; ++e) u[j][e] = v.get(e);
+    if (s < 0) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) u[j][e] = a.state[(int64_t)(ch + e) * (TAPS - 1) + TAPS - 1 + s];
     }
   }
   TO* out = reinterpret_cast<TO*>(g.out) + (int64_t)h * g.stride + c;

@@ -105,7 +105,7 @@ template <typename T, typename TQ, int RH>
 int attn_rows_rh(const AttnArgs& a, hipStream_t s) {
   const int rep = a.H / a.G;
   const dim3 grid(a.splits, a.G * ((rep + RH - 1) / RH), a.n);
-  const size_t lds = (size_t)RH * a.dim_s * 4 + 256 * 8 * 4 + (size_t)(a.dim_s + a.vdim_s) * sizeof(T);
+  const size_t lds = (size_t)RH * a.dim_s * 4 + (size_t)attn_red_floats(RH, a.vdim_s) * 4 + (size_t)(a.dim_s + a.vdim_s) * sizeof(T);
   return launch_lds<attn_rows_kernel<T, TQ, RH>>(grid, dim3(256), lds, s, a);
 }
 template <typename T, typename TQ>
@@ -115,6 +115,28 @@ int attn_rows_any(const AttnArgs& a, hipStream_t s) {
   if (rep >= 3) return attn_rows_rh<T, TQ, 4>(a, s);
   if (rep == 2) return attn_rows_rh<T, TQ, 2>(a, s);
   return attn_rows_rh<T, TQ, 1>(a, s);
+}
+
+// ---- delta rule --------------------------------------------------------------
+template <int NT>
+int delta_scan(const DeltaArgs& a, hipStream_t s) {
+  const int chunks = (a.n + kDeltaChunk - 1) / kDeltaChunk;
+  const int step = 32768;  // chunks per launch of the first kernel
+  for (int c = 0; c < chunks; c += step) {
+    DeltaArgs b = a;
+    const int64_t t0 = (int64_t)c * kDeltaChunk;
+    b.q += t0 * a.kv_heads * a.dim_s;
+    b.k += t0 * a.kv_heads * a.dim_s;
+    b.g += t0 * a.heads * a.dim_s;
+    b.beta += t0 * a.heads;
+    b.tm += (int64_t)c * a.heads * 512;
+    b.n = (int)(a.n - t0);
+    const int rc = launch_lds<delta_chunk_kernel<4 * NT>>(dim3(a.heads, chunks - c < step ? chunks - c : step), dim3(256),
+                                                          (size_t)3 * kDeltaChunk * 64 * NT * 4, s, b);
+    if (rc != DV_OK) return rc;
+  }
+  return launch_lds<delta_scan_kernel<NT>>(dim3((unsigned)(a.heads * ((a.vdim_s + kDeltaCols - 1) / kDeltaCols))),
+                                           dim3(256), delta_scan_lds_bytes<NT>(), s, a);
 }
 
 template <int RT>
@@ -348,8 +370,8 @@ int dv_mix_latent_absorb(int dtype, const float* q, const void* W, int H, int di
   return launched();
 }
 
-int dv_mix_latent_attn(int dtype, const dvAttnArgs* a, float* lat, const void* W, int vrows, void* out, void* stream) {
-  if (!dtype_ok(dtype) || !W || !out || !lat || vrows < 1 || !a || a->n != 1 || a->G != 1 || !a->part || a->splits < 2 ||
+int dv_mix_latent_attn(int dtype, const dvAttnArgs* a, const void* W, int vrows, void* out, void* stream) {
+  if (!dtype_ok(dtype) || !W || !out || vrows < 1 || !a || a->n != 1 || a->G != 1 || !a->part || a->splits < 2 ||
       a->k != a->v || a->dim_s != a->vdim_s || a->window > 0 || a->ring > 0 || a->base != 0 || a->fresh_k || a->norm_dim > 0)
     return DV_ERR_INVALID_ARG;
   int rc = attn_args_ok(a);
@@ -363,13 +385,12 @@ int dv_mix_latent_attn(int dtype, const dvAttnArgs* a, float* lat, const void* W
   else if (rank <= 512) rc = latent_tiles<32>(*a, st(stream));
   else rc = attn_rows_any<bf16_t, float>(*a, st(stream));
   if (rc != DV_OK) return rc;
-  hipLaunchKernelGGL((attn_merge_kernel<float, float>), dim3(a->H, (rank + 63) / 64, 1), dim3(256), 0, st(stream), *a, lat);
-  const dim3 grid(a->H, vrows <= 16 ? 1 : (vrows <= 64 ? 4 : 8));
+  const dim3 grid(a->H, vrows <= 32 ? 1 : (vrows <= 64 ? 2 : 4));
   const size_t lds = (size_t)rank * 4;
   if (dtype == DV_BF16)
-    hipLaunchKernelGGL((latent_out_kernel<bf16_t>), grid, dim3(256), lds, st(stream), lat, (const bf16_t*)W, rank, vrows, (bf16_t*)out);
+    hipLaunchKernelGGL((latent_out_kernel<bf16_t>), grid, dim3(256), lds, st(stream), *a, (const bf16_t*)W, vrows, (bf16_t*)out);
   else
-    hipLaunchKernelGGL((latent_out_kernel<float>), grid, dim3(256), lds, st(stream), lat, (const float*)W, rank, vrows, (float*)out);
+    hipLaunchKernelGGL((latent_out_kernel<float>), grid, dim3(256), lds, st(stream), *a, (const float*)W, vrows, (float*)out);
   return launched();
 }
 
@@ -387,17 +408,15 @@ int dv_mix_delta_gates(int dtype, const void* z, int64_t ldz, const void* b, int
 }
 
 int dv_mix_delta_scan(const dvDeltaArgs* a, void* stream) {
-  if (!a || !a->q || !a->k || !a->v || !a->g || !a->beta || !a->S || !a->o || a->n < 1 || a->heads < 1 ||
+  if (!a || !a->q || !a->k || !a->v || !a->g || !a->beta || !a->S || !a->o || !a->tm || a->n < 1 || a->heads < 1 ||
       a->kv_heads < 1 || a->heads % a->kv_heads || a->dim_s < 8 || a->vdim_s < 1)
     return DV_ERR_INVALID_ARG;
   if (a->dim_s % 8 || !al16(a->q) || !al16(a->k) || !al16(a->g) || !al16(a->S)) return DV_ERR_ALIGNMENT;
-  const dim3 grid((unsigned)(a->heads * ((a->vdim_s + kDeltaCols - 1) / kDeltaCols)));
-  if (a->dim_s <= 64) hipLaunchKernelGGL((delta_scan_kernel<4>), grid, dim3(256), 0, st(stream), *a);
-  else if (a->dim_s <= 128) hipLaunchKernelGGL((delta_scan_kernel<8>), grid, dim3(256), 0, st(stream), *a);
-  else if (a->dim_s <= 192) hipLaunchKernelGGL((delta_scan_kernel<12>), grid, dim3(256), 0, st(stream), *a);
-  else if (a->dim_s <= 256) hipLaunchKernelGGL((delta_scan_kernel<16>), grid, dim3(256), 0, st(stream), *a);
-  else return DV_ERR_UNSUPPORTED;
-  return launched();
+  if (a->dim_s <= 64) return delta_scan<1>(*a, st(stream));
+  if (a->dim_s <= 128) return delta_scan<2>(*a, st(stream));
+  if (a->dim_s <= 192) return delta_scan<3>(*a, st(stream));
+  if (a->dim_s <= 256) return delta_scan<4>(*a, st(stream));
+  return DV_ERR_UNSUPPORTED;
 }
 
 int dv_mix_delta_step(int dtype, const dvDeltaStepArgs* a, void* stream) {

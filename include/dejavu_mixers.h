@@ -138,6 +138,7 @@ typedef struct {
   const float* beta;       /* [n][heads] */
   float* S;                /* [heads][vdim_s][dim_s] */
   float* o;                /* [n][heads][vdim_s] */
+  float* tm;               /* scratch: ceil(n / 16) * heads * 512 */
   int n, heads, kv_heads, dim_s, vdim_s;
 } dvDeltaArgs;
 
@@ -185,9 +186,8 @@ DV_API int dv_mix_attn_tiles(const dvAttnArgs* args, int keys, void* stream);
 DV_API int dv_mix_latent_absorb(int dtype, const float* q, const void* W, int H, int dim_s, int rank, float* out,
                                 void* stream);
 /* Latent decode row: attention over the cache (args: G = 1, k == v, dim_s = vdim_s = rank, at least two splits with
- * `part`, q and gate fp32), gated; lat [H][rank] fp32 receives it, out [H][vrows] = W_uv [H][vrows][rank] lat. */
-DV_API int dv_mix_latent_attn(int dtype, const dvAttnArgs* args, float* lat, const void* W, int vrows, void* out,
-                              void* stream);
+ * `part`, q and gate fp32), gated, times W_uv [H][vrows][rank]; out [H][vrows]. */
+DV_API int dv_mix_latent_attn(int dtype, const dvAttnArgs* args, const void* W, int vrows, void* out, void* stream);
 DV_API int dv_mix_delta_gates(int dtype, const void* z, int64_t ldz, const void* b, int64_t ldb, const float* A_log,
                               const float* dt_bias, int n, int heads, int dim_s, float* g, float* beta, void* stream);
 DV_API int dv_mix_delta_scan(const dvDeltaArgs* args, void* stream);
