@@ -42,7 +42,7 @@ AttnArgs = _struct("AttnArgs", ("q", _p), ("ldq", _l), ("k", _p), ("ldk", _l), (
                    ("pos_dev", _p), ("pos_host", _i), ("out", _p), ("part", _p), ("splits", _i), ("fresh_k", _p),
                    ("fresh_v", _p), ("norm_dim", _i), ("eps", _f))
 DeltaArgs = _struct("DeltaArgs", ("q", _p), ("k", _p), ("v", _p), ("g", _p), ("beta", _p), ("S", _p), ("o", _p),
-                    ("tm", _p), ("n", _i), ("heads", _i), ("kv_heads", _i), ("dim_s", _i), ("vdim_s", _i))
+                    ("tm", _p), ("tm_floats", _l), ("n", _i), ("heads", _i), ("kv_heads", _i), ("dim_s", _i), ("vdim_s", _i))
 DeltaStepArgs = _struct("DeltaStepArgs", ("p", _p), ("off_k", _i), ("off_v", _i), ("off_b", _i), ("off_a", _i),
                         ("off_g", _i), ("heads", _i), ("kv_heads", _i), ("dim", _i), ("dim_s", _i), ("vdim_s", _i),
                         ("Wa", _p), ("Wg", _p), ("rank_a", _i), ("rank_g", _i), ("A_log", _p), ("dt_bias", _p),

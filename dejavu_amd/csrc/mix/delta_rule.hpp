@@ -10,8 +10,9 @@
 //   U = T (V - Kt S_0),  T = (1 + diag(beta) L)^-1 diag(beta),  Kt_i = P(i, 0) k_i  (g_1 included)
 //   O = Qt S_0 + M U,    S = P(16, 0) S_0 + Kh^T U,             Kh_j = P(16, j) k_j
 //
-// T and M depend on no state: one kernel makes them for all chunks at once.  The second kernel carries the state from
-// chunk to chunk; its products run on the fp32 matrix instructions.  A decode step uses the recurrence itself.
+// Everything but U, O and S depends on no state: one kernel makes it for many chunks at once.  The second kernel
+// carries the state from chunk to chunk; its products run on the fp32 matrix instructions.  A decode step uses the
+// recurrence itself.
 // State layout [heads][vdim][dim] (key channels contiguous).
 #pragma once
 #include "elem.hpp"
@@ -84,11 +85,22 @@ __device__ __forceinline__ void store_state(const float (&S)[E], float* __restri
 constexpr int kDeltaCols = 16;   // columns of S per workgroup
 constexpr int kDeltaChunk = 16;  // tokens per chunk
 
-// T and M of a chunk and head: tm[(chunk * heads + head) * 512] = T [16][16], then M [16][16].  A row of 16 lanes owns
-// key j and walks the later tokens.  Grid: (heads, chunks); D = 16 E >= dim_s.
-template <int E>
+// What the first kernel leaves for a chunk and head, in floats and in the order the second kernel's lanes load it
+// (lane = 16 q + r, four floats per lane, 256 floats per operand): for every tile of 16 channels Kt and Qt (token r,
+// channels 4 q ..), Kh (channel r, tokens 4 q ..); then T and M (row r, columns 4 q ..); then the decay over the chunk
+// per channel.  D = 64 NT >= dim_s.
+template <int NT>
+struct DeltaChunk {
+  static constexpr int D = 64 * NT;
+  static constexpr int kt = 0, qt = 16 * D, kh = 32 * D, t = 48 * D, m = t + 256, gc = m + 256, floats = gc + D;
+};
+
+// A row of 16 lanes owns key j and walks the later tokens for T and M; then a thread owns a channel for the rest.
+// Grid: (heads, chunks).
+template <int NT>
 __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaArgs a) {
-  constexpr int D = 16 * E, C = kDeltaChunk;
+  using Out = DeltaChunk<NT>;
+  constexpr int E = 4 * NT, D = 64 * NT, C = kDeltaChunk;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
   float* sq = reinterpret_cast<float*>(smem_raw);  // [16][D] each
   float* sk = sq + C * D;
@@ -109,7 +121,7 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaArgs a) {
     const float4_t g = *reinterpret_cast<const float4_t*>(a.g + (row * a.heads + head) * a.dim_s + dc);
     *reinterpret_cast<float4_t*>(sq + at) = ok ? q : z;
     *reinterpret_cast<float4_t*>(sk + at) = ok ? k : z;
-    *reinterpret_cast<float4_t*>(sg + at) = ok ? g : z;
+    *reinterpret_cast<float4_t*>(sg + at) = ok ? g : float4_t{1.f, 1.f, 1.f, 1.f};  // past the end: nothing decays
   }
   if (tid < C) sb[tid] = t0 + tid < a.n ? a.beta[(int64_t)(t0 + tid) * a.heads + head] : 0.f;
   L[j][sub] = 0.f;
@@ -139,7 +151,7 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaArgs a) {
     }
   }
   __syncthreads();
-  float* out = a.tm + ((int64_t)blockIdx.y * a.heads + head) * 512;
+  float* out = a.tm + ((int64_t)blockIdx.y * a.heads + head) * Out::floats;
   if (tid < C) {  // column tid of T by forward substitution
     float x[C];
 #pragma unroll
@@ -148,45 +160,81 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaArgs a) {
 #pragma unroll
       for (int k = 0; k < i; ++k) v = __builtin_fmaf(-L[i][k], x[k], v);
       x[i] = v;
-      out[i * C + tid] = v;
+      out[Out::t + ((tid >> 2) * 16 + i) * 4 + (tid & 3)] = v;
     }
   }
-  out[256 + tid] = M[j][sub];
+  out[Out::m + ((sub >> 2) * 16 + j) * 4 + (sub & 3)] = M[j][sub];
+  // a thread per channel makes Kt and Qt, another one Kh; they change places with k, q and g in LDS
+  constexpr int IT = (2 * D + 255) / 256;
+  float r0[IT][C], r1[IT][C];
+#pragma unroll
+  for (int it = 0; it < IT; ++it) {
+    const int item = it * 256 + 255 - tid, d = item % D;  // the first wave, busy with T, comes last
+    float p = 1.f;
+    if (item < D) {
+#pragma unroll
+      for (int t = 0; t < C; ++t) {
+        p *= sg[t * D + d];
+        r0[it][t] = p * sk[t * D + d];
+        r1[it][t] = p * sq[t * D + d];
+      }
+    } else if (item < 2 * D) {
+#pragma unroll
+      for (int t = C - 1; t >= 0; --t) {
+        r0[it][t] = p * sk[t * D + d];
+        p *= sg[t * D + d];
+      }
+      out[Out::gc + d] = p;
+    }
+  }
+  __syncthreads();
+#pragma unroll
+  for (int it = 0; it < IT; ++it) {
+    const int item = it * 256 + 255 - tid, d = item % D;
+#pragma unroll
+    for (int t = 0; t < C; ++t) {
+      if (item < D) {
+        sk[t * D + d] = r0[it][t];
+        sq[t * D + d] = r1[it][t];
+      } else if (item < 2 * D) {
+        sg[t * D + d] = r0[it][t];
+      }
+    }
+  }
+  __syncthreads();
+  for (int i = tid; i < 4 * D; i += 256) {
+    const int tile = i >> 6, q = (i >> 4) & 3, r = i & 15;
+    *reinterpret_cast<float4_t*>(out + Out::kt + i * 4) = *reinterpret_cast<const float4_t*>(sk + r * D + tile * 16 + q * 4);
+    *reinterpret_cast<float4_t*>(out + Out::qt + i * 4) = *reinterpret_cast<const float4_t*>(sq + r * D + tile * 16 + q * 4);
+    const float* g = sg + q * 4 * D + tile * 16 + r;
+    *reinterpret_cast<float4_t*>(out + Out::kh + i * 4) = float4_t{g[0], g[D], g[2 * D], g[3 * D]};
+  }
 }
 
 // Chunk after chunk for 16 columns of a head.  Wave w owns key channels [16 NT w, 16 NT (w + 1)) of the state, as
 // accumulators of the 16x16x4 products: element i of a lane is channel 4 (lane / 16) + i of a tile, column lane % 16,
-// which is also the operand layout of the products with Kt and Qt when their channels are taken in that order.  The
-// four waves' partial products meet in LDS once per chunk; U is then made by every wave for itself.
+// which is also the operand layout of the products with Kt and Qt when their channels are taken in that order.  All
+// operands are loaded by the lanes that use them, a chunk ahead.  The waves' parts of Kt S meet in LDS once per chunk
+// and every wave makes U for itself.  A wave's part of O is Qt S over its channels plus every fourth token's share of
+// M U; the parts meet at the next chunk's barrier.
 template <int NT>
-struct DeltaChunkLds {
-  static constexpr int D = 64 * NT, KL = D + 4, TL = 20;
-  float kt[16 * KL], qt[16 * KL];  // [token][channel]
-  float kh[D * TL];                // [channel][token]
-  float tmat[16 * TL], mmat[16 * TL];
-  float v[16 * 16];                // [token][column]
-  float gc[D];                     // decay over the whole chunk
+struct DeltaOperands {
+  float4_t kt[NT], qt[NT], kh[NT], gc[NT], t;
+  float m, v[4];
 };
-template <int NT>
-constexpr size_t delta_scan_lds_bytes() {
-  return 2 * sizeof(DeltaChunkLds<NT>) + 2 * 4 * 2 * 64 * 16;  // two stages; partial products, two stages
-}
 
 // Grid: heads * ceil(vdim_s / 16), head fastest (the workgroups of a head share an XCD's L2 when heads % 8 == 0).
 template <int NT>
 __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaArgs a) {
-  using Lds = DeltaChunkLds<NT>;
-  constexpr int D = Lds::D, KL = Lds::KL, TL = Lds::TL, C = kDeltaChunk;
-  constexpr int IT = (2 * D + 255) / 256;  // (role, channel) items per thread
-  extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
-  Lds* st = reinterpret_cast<Lds*>(smem_raw);
-  float4_t* part = reinterpret_cast<float4_t*>(smem_raw + 2 * sizeof(Lds));  // [stage][wave][2][64]
+  using In = DeltaChunk<NT>;
+  constexpr int C = kDeltaChunk;
+  __shared__ __attribute__((aligned(16))) float4_t kpart[2][4][64], opart[2][4][64];
   const int head = blockIdx.x % a.heads, tile = blockIdx.x / a.heads;
-  const int kvh = head / (a.heads / a.kv_heads);
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int l16 = lane & 15, q4 = lane >> 4;
   const int col = tile * kDeltaCols + l16;
   const bool col_ok = col < a.vdim_s;
+  const int vstep = a.heads * a.vdim_s;
   float* sp = a.S + ((int64_t)head * a.vdim_s + (col_ok ? col : 0)) * a.dim_s;
   float4_t S[NT];
 #pragma unroll
@@ -194,135 +242,77 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaArgs a) {
     const int d = (wave * NT + t) * 16 + q4 * 4;
     S[t] = (col_ok && d < a.dim_s) ? *reinterpret_cast<const float4_t*>(sp + d) : float4_t{0.f, 0.f, 0.f, 0.f};
   }
-
-  // staging: role 0 makes Kt and Qt of a channel, role 1 Kh and the chunk's decay
-  float rg[IT][C], rk[IT][C], rq[IT][C], rtm[2], rv;
-  const int gs = a.heads * a.dim_s, ks_ = a.kv_heads * a.dim_s;  // elements between tokens
-  const int vc = min(tile * kDeltaCols + (tid & 15), a.vdim_s - 1);
-  auto fetch = [&](int t0) {
-    const float* gp = a.g + (int64_t)t0 * gs + head * a.dim_s;
-    const float* kp = a.k + (int64_t)t0 * ks_ + kvh * a.dim_s;
-    const float* qp = a.q + (int64_t)t0 * ks_ + kvh * a.dim_s;
-    const int last = a.n - 1 - t0;
-#pragma unroll
-    for (int it = 0; it < IT; ++it) {
-      const int d = min((it * 256 + tid) % D, a.dim_s - 1);
-#pragma unroll
-      for (int t = 0; t < C; ++t) {
-        const int row = min(t, last);
-        rg[it][t] = gp[row * gs + d];
-        rk[it][t] = kp[row * ks_ + d];
-        rq[it][t] = qp[row * ks_ + d];
-      }
-    }
-    const float* tm = a.tm + ((int64_t)(t0 / C) * a.heads + head) * 512;
-    rtm[0] = tm[tid];
-    rtm[1] = tm[256 + tid];
-    rv = a.v[((int64_t)t0 + min(tid >> 4, last)) * a.heads * a.vdim_s + head * a.vdim_s + vc];
-  };
-  auto put = [&](Lds& b, int t0) {
-    // what was read past the end of the portion or of the channels
-    const int cnt = a.n - t0;
-#pragma unroll
-    for (int it = 0; it < IT; ++it) {
-      const bool in = (it * 256 + tid) % D < a.dim_s;
-#pragma unroll
-      for (int t = 0; t < C; ++t) {
-        if (!in || t >= cnt) {
-          rg[it][t] = 1.f;
-          rk[it][t] = 0.f;
-          rq[it][t] = 0.f;
-        }
-      }
-    }
-    if ((tid >> 4) >= cnt) rv = 0.f;
-#pragma unroll
-    for (int it = 0; it < IT; ++it) {
-      const int item = it * 256 + tid, role = item / D, d = item % D;
-      if (item < 2 * D) {
-        if (role == 0) {
-          float p = 1.f;
-#pragma unroll
-          for (int t = 0; t < C; ++t) {
-            p *= rg[it][t];
-            b.kt[t * KL + d] = p * rk[it][t];
-            b.qt[t * KL + d] = p * rq[it][t];
-          }
-        } else {
-          float p = 1.f;
-          float kh[C];
-#pragma unroll
-          for (int t = C - 1; t >= 0; --t) {
-            kh[t] = p * rk[it][t];
-            p *= rg[it][t];
-          }
-          b.gc[d] = p;
-#pragma unroll
-          for (int t = 0; t < C; t += 4)
-            *reinterpret_cast<float4_t*>(&b.kh[d * TL + t]) = float4_t{kh[t], kh[t + 1], kh[t + 2], kh[t + 3]};
-        }
-      }
-    }
-    b.tmat[(tid >> 4) * TL + (tid & 15)] = rtm[0];
-    b.mmat[(tid >> 4) * TL + (tid & 15)] = rtm[1];
-    b.v[tid] = rv;
-  };
-
-  fetch(0);
-  put(st[0], 0);
-  __syncthreads();
-  for (int t0 = 0, buf = 0; t0 < a.n; t0 += C, buf ^= 1) {
-    const Lds& b = st[buf];
-    const bool more = t0 + C < a.n;
-    if (more) fetch(t0 + C);
-    // partial Kt S and Qt S over this wave's channels
-    float4_t ks = {0.f, 0.f, 0.f, 0.f}, qs = {0.f, 0.f, 0.f, 0.f};
+  const float* vcol = a.v + head * a.vdim_s + min(col, a.vdim_s - 1);
+  const int chunks = (a.n + C - 1) / C;
+  // rows of V past the end meet zeros of T
+  auto load = [&](DeltaOperands<NT>& x, int c) {
+    const float* src = a.tm + ((int64_t)c * a.heads + head) * In::floats;
 #pragma unroll
     for (int t = 0; t < NT; ++t) {
-      const int d = (wave * NT + t) * 16 + q4 * 4;
-      const float4_t kt = *reinterpret_cast<const float4_t*>(&b.kt[l16 * KL + d]);
-      const float4_t qt = *reinterpret_cast<const float4_t*>(&b.qt[l16 * KL + d]);
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        ks = __builtin_amdgcn_mfma_f32_16x16x4f32(kt[i], S[t][i], ks, 0, 0, 0);
-        qs = __builtin_amdgcn_mfma_f32_16x16x4f32(qt[i], S[t][i], qs, 0, 0, 0);
-      }
+      const int tt = wave * NT + t;
+      x.kt[t] = *reinterpret_cast<const float4_t*>(src + In::kt + tt * 256 + lane * 4);
+      x.qt[t] = *reinterpret_cast<const float4_t*>(src + In::qt + tt * 256 + lane * 4);
+      x.kh[t] = *reinterpret_cast<const float4_t*>(src + In::kh + tt * 256 + lane * 4);
+      x.gc[t] = *reinterpret_cast<const float4_t*>(src + In::gc + tt * 16 + q4 * 4);
     }
-    float4_t* pp = part + buf * 512;
-    pp[wave * 128 + lane] = ks;
-    pp[wave * 128 + 64 + lane] = qs;
-    __syncthreads();
-    float4_t w;  // V - Kt S: tokens 4 q4 .. + 3 of this lane's column
-    const float4_t sum = (pp[lane] + pp[128 + lane]) + (pp[256 + lane] + pp[384 + lane]);
+    x.t = *reinterpret_cast<const float4_t*>(src + In::t + lane * 4);
+    x.m = src[In::m + lane * 4 + wave];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) w[i] = b.v[(q4 * 4 + i) * 16 + l16] - sum[i];
-    const float4_t tm = *reinterpret_cast<const float4_t*>(&b.tmat[l16 * TL + q4 * 4]);
+    for (int i = 0; i < 4; ++i) x.v[i] = vcol[(int64_t)min(c * C + q4 * 4 + i, a.n - 1) * vstep];
+  };
+  // read-outs of a chunk: a lane stores token 4 wave + q4 of its column
+  const float* op = reinterpret_cast<const float*>(opart) + (wave * 16 + l16) * 4 + q4;
+  float* ocol = a.o + (int64_t)head * a.vdim_s + col;
+  auto store_o = [&](int c, int par) {
+    const float* p = op + par * 1024;
+    const int t = c * C + wave * 4 + q4;
+    const float o = (p[0] + p[256]) + (p[512] + p[768]);
+    if (col_ok && t < a.n) ocol[(int64_t)t * vstep] = o;
+  };
+  auto step = [&](const DeltaOperands<NT>& x, int c, int par) {
+    float4_t ks[NT];
+#pragma unroll
+    for (int t = 0; t < NT; ++t) ks[t] = float4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int t = 0; t < NT; ++t) ks[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kt[t][i], S[t][i], ks[t], 0, 0, 0);
+#pragma unroll
+    for (int t = 1; t < NT; ++t) ks[0] += ks[t];
+    kpart[par][wave][lane] = ks[0];
+    float4_t qs = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int t = 0; t < NT; ++t) qs = __builtin_amdgcn_mfma_f32_16x16x4f32(x.qt[t][i], S[t][i], qs, 0, 0, 0);
+    __syncthreads();
+    const float4_t sum = (kpart[par][0][lane] + kpart[par][1][lane]) + (kpart[par][2][lane] + kpart[par][3][lane]);
     float4_t u = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int i = 0; i < 4; ++i) u = __builtin_amdgcn_mfma_f32_16x16x4f32(tm[i], w[i], u, 0, 0, 0);
-    if (wave == 3) {
-      float4_t o = (pp[64 + lane] + pp[192 + lane]) + (pp[320 + lane] + pp[448 + lane]);
-      const float4_t mm = *reinterpret_cast<const float4_t*>(&b.mmat[l16 * TL + q4 * 4]);
+    for (int i = 0; i < 4; ++i) u = __builtin_amdgcn_mfma_f32_16x16x4f32(x.t[i], x.v[i] - sum[i], u, 0, 0, 0);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) o = __builtin_amdgcn_mfma_f32_16x16x4f32(mm[i], u[i], o, 0, 0, 0);
+    for (int t = 0; t < NT; ++t) S[t] *= x.gc[t];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int t = t0 + q4 * 4 + i;
-        if (col_ok && t < a.n) a.o[((int64_t)t * a.heads + head) * a.vdim_s + col] = o[i];
-      }
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int t = 0; t < NT; ++t) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kh[t][i], u[i], S[t], 0, 0, 0);
+    const float uw = wave == 0 ? u[0] : (wave == 1 ? u[1] : (wave == 2 ? u[2] : u[3]));
+    qs = __builtin_amdgcn_mfma_f32_16x16x4f32(x.m, uw, qs, 0, 0, 0);
+    if (c > 0) store_o(c - 1, par ^ 1);
+    opart[par][wave][lane] = qs;
+  };
+  DeltaOperands<NT> even, odd;
+  load(even, 0);
+  for (int c = 0; c < chunks; c += 2) {
+    load(odd, min(c + 1, chunks - 1));
+    step(even, c, 0);
+    if (c + 1 < chunks) {
+      load(even, min(c + 2, chunks - 1));
+      step(odd, c + 1, 1);
     }
-#pragma unroll
-    for (int t = 0; t < NT; ++t) {
-      const int d0 = (wave * NT + t) * 16;
-      const float4_t gc = *reinterpret_cast<const float4_t*>(&b.gc[d0 + q4 * 4]);
-      const float4_t kh = *reinterpret_cast<const float4_t*>(&b.kh[(d0 + l16) * TL + q4 * 4]);
-      S[t] *= gc;
-#pragma unroll
-      for (int i = 0; i < 4; ++i) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(kh[i], u[i], S[t], 0, 0, 0);
-    }
-    if (more) put(st[buf ^ 1], t0 + C);  // that stage was read before the barrier above
-    __syncthreads();
   }
+  __syncthreads();
+  store_o(chunks - 1, (chunks - 1) & 1);
 #pragma unroll
   for (int t = 0; t < NT; ++t) {
     const int d = (wave * NT + t) * 16 + q4 * 4;

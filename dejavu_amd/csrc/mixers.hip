@@ -118,25 +118,29 @@ int attn_rows_any(const AttnArgs& a, hipStream_t s) {
 }
 
 // ---- delta rule --------------------------------------------------------------
+constexpr int kDeltaSegment = 4096;  // tokens whose chunk blocks are in memory at a time
 template <int NT>
 int delta_scan(const DeltaArgs& a, hipStream_t s) {
-  const int chunks = (a.n + kDeltaChunk - 1) / kDeltaChunk;
-  const int step = 32768;  // chunks per launch of the first kernel
-  for (int c = 0; c < chunks; c += step) {
+  const size_t need = (size_t)((a.n < kDeltaSegment ? a.n : kDeltaSegment) + kDeltaChunk - 1) / kDeltaChunk * a.heads *
+                      DeltaChunk<NT>::floats;
+  if ((size_t)a.tm_floats < need) return DV_ERR_WORKSPACE;
+  for (int t0 = 0; t0 < a.n; t0 += kDeltaSegment) {
     DeltaArgs b = a;
-    const int64_t t0 = (int64_t)c * kDeltaChunk;
-    b.q += t0 * a.kv_heads * a.dim_s;
-    b.k += t0 * a.kv_heads * a.dim_s;
-    b.g += t0 * a.heads * a.dim_s;
-    b.beta += t0 * a.heads;
-    b.tm += (int64_t)c * a.heads * 512;
-    b.n = (int)(a.n - t0);
-    const int rc = launch_lds<delta_chunk_kernel<4 * NT>>(dim3(a.heads, chunks - c < step ? chunks - c : step), dim3(256),
-                                                          (size_t)3 * kDeltaChunk * 64 * NT * 4, s, b);
+    b.q += (int64_t)t0 * a.kv_heads * a.dim_s;
+    b.k += (int64_t)t0 * a.kv_heads * a.dim_s;
+    b.v += (int64_t)t0 * a.heads * a.vdim_s;
+    b.g += (int64_t)t0 * a.heads * a.dim_s;
+    b.o += (int64_t)t0 * a.heads * a.vdim_s;
+    b.beta += (int64_t)t0 * a.heads;
+    b.n = a.n - t0 < kDeltaSegment ? a.n - t0 : kDeltaSegment;
+    int rc = launch_lds<delta_chunk_kernel<NT>>(dim3(a.heads, (b.n + kDeltaChunk - 1) / kDeltaChunk), dim3(256),
+                                                (size_t)3 * kDeltaChunk * 64 * NT * 4, s, b);
+    if (rc != DV_OK) return rc;
+    rc = launch_lds<delta_scan_kernel<NT>>(dim3((unsigned)(a.heads * ((a.vdim_s + kDeltaCols - 1) / kDeltaCols))),
+                                           dim3(256), 0, s, b);
     if (rc != DV_OK) return rc;
   }
-  return launch_lds<delta_scan_kernel<NT>>(dim3((unsigned)(a.heads * ((a.vdim_s + kDeltaCols - 1) / kDeltaCols))),
-                                           dim3(256), delta_scan_lds_bytes<NT>(), s, a);
+  return DV_OK;
 }
 
 template <int RT>
@@ -411,7 +415,7 @@ int dv_mix_delta_scan(const dvDeltaArgs* a, void* stream) {
   if (!a || !a->q || !a->k || !a->v || !a->g || !a->beta || !a->S || !a->o || !a->tm || a->n < 1 || a->heads < 1 ||
       a->kv_heads < 1 || a->heads % a->kv_heads || a->dim_s < 8 || a->vdim_s < 1)
     return DV_ERR_INVALID_ARG;
-  if (a->dim_s % 8 || !al16(a->q) || !al16(a->k) || !al16(a->g) || !al16(a->S)) return DV_ERR_ALIGNMENT;
+  if (a->dim_s % 8 || !al16(a->q) || !al16(a->k) || !al16(a->g) || !al16(a->S) || !al16(a->tm)) return DV_ERR_ALIGNMENT;
   if (a->dim_s <= 64) return delta_scan<1>(*a, st(stream));
   if (a->dim_s <= 128) return delta_scan<2>(*a, st(stream));
   if (a->dim_s <= 192) return delta_scan<3>(*a, st(stream));

@@ -356,9 +356,10 @@ def delta_scan(q, k, v, g, beta, S, heads: int, kv_heads: int) -> torch.Tensor:
     n, vs, ds = q.shape[0], S.shape[1], S.shape[2]
     o = torch.empty(n, heads, vs, dtype=torch.float32, device=q.device)
     assert q.shape == k.shape == (n, kv_heads * ds) and v.shape == (n, heads * vs) and g.shape == (n, heads * ds)
-    tm = torch.empty((n + 15) // 16 * heads * 512, dtype=torch.float32, device=q.device)
+    tm = torch.empty((min(n, 4096) + 15) // 16 * heads * (49 * ((ds + 63) // 64 * 64) + 512), dtype=torch.float32,
+                     device=q.device)
     a = L.DeltaArgs(q=q.data_ptr(), k=k.data_ptr(), v=v.data_ptr(), g=g.data_ptr(), beta=beta.data_ptr(),
-                    S=S.data_ptr(), o=o.data_ptr(), tm=tm.data_ptr(), n=n, heads=heads, kv_heads=kv_heads, dim_s=ds, vdim_s=vs)
+                    S=S.data_ptr(), o=o.data_ptr(), tm=tm.data_ptr(), tm_floats=tm.numel(), n=n, heads=heads, kv_heads=kv_heads, dim_s=ds, vdim_s=vs)
     check(lib.dv_mix_delta_scan(_ref(a), _stream()), "dv_mix_delta_scan")
     return o
 

@@ -138,7 +138,8 @@ typedef struct {
   const float* beta;       /* [n][heads] */
   float* S;                /* [heads][vdim_s][dim_s] */
   float* o;                /* [n][heads][vdim_s] */
-  float* tm;               /* scratch: ceil(n / 16) * heads * 512 */
+  float* tm;               /* scratch of tm_floats: ceil(min(n, 4096) / 16) * heads * (49 D + 512), */
+  int64_t tm_floats;       /* D: dim_s rounded up to a multiple of 64 */
   int n, heads, kv_heads, dim_s, vdim_s;
 } dvDeltaArgs;
 

@@ -216,6 +216,8 @@ def test_host_side_argument_checks():
     assert L.lib.dv_mix_ring_copy(0, A, 64, A, 4, 64, 0, 5, 64, 1, None) == -1  # more rows than the ring has
     d = L.DeltaArgs(q=A, k=A, v=A, g=A, beta=A, S=A, o=A, tm=A, n=2, heads=2, kv_heads=1, dim_s=264, vdim_s=8)
     assert L.lib.dv_mix_delta_scan(ref(d), None) == -2
+    d.dim_s, d.tm_floats = 64, 100
+    assert L.lib.dv_mix_delta_scan(ref(d), None) == -4                       # scratch too small
     with pytest.raises(RuntimeError, match="no CPU fallback"):
         from dejavu_amd import mixer_ops
         mixer_ops.linear(torch.zeros(1, 8), torch.zeros(8, 8))
