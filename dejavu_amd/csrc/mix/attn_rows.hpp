@@ -7,10 +7,34 @@ namespace dv {
 
 using AttnArgs = dvAttnArgs;
 
-__device__ __forceinline__ float rms_factor(const float* x, int dim, float eps, int lane) {
-  float ss = 0.f;
-  for (int c = lane; c < dim; c += 64) ss = __builtin_fmaf(x[c], x[c], ss);
-  return 1.f / sqrtf(wave_sum(ss) / dim + eps);
+// By one wave: put(c, x[c] / rms(x)) for every entry, the mean over norm_dim entries (0: put(c, x[c])).
+template <typename T, typename F>
+__device__ __forceinline__ void normed_row(const T* __restrict__ x, int n, int norm_dim, float eps, int lane, F put) {
+  constexpr int NX = 4;  // values a lane keeps; longer rows read the rest again
+  float v[NX];
+#pragma unroll
+  for (int u = 0; u < NX; ++u) v[u] = to_f(x[min(lane + u * 64, n - 1)]);
+  float s = 1.f;
+  if (norm_dim > 0) {
+    float ss = 0.f;
+#pragma unroll
+    for (int u = 0; u < NX; ++u)
+      if (lane + u * 64 < norm_dim) ss = __builtin_fmaf(v[u], v[u], ss);
+    for (int c = lane + NX * 64; c < norm_dim; c += 64) ss = __builtin_fmaf(to_f(x[c]), to_f(x[c]), ss);
+    s = 1.f / sqrtf(wave_sum(ss) / norm_dim + eps);
+  }
+#pragma unroll
+  for (int u = 0; u < NX; ++u)
+    if (lane + u * 64 < n) put(lane + u * 64, v[u] * s);
+  for (int c = lane + NX * 64; c < n; c += 64) put(c, to_f(x[c]) * s);
+}
+
+// Partial sums of a split: `part` holds [n][H][splits][vdim_s] sums, then [n][H][splits][2] (maximum, denominator).
+__device__ __forceinline__ float* part_sums(const AttnArgs& a, int row, int head, int split) {
+  return a.part + (((int64_t)row * a.H + head) * a.splits + split) * a.vdim_s;
+}
+__device__ __forceinline__ float* part_ml(const AttnArgs& a, int row, int head, int split) {
+  return a.part + (int64_t)a.n * a.H * a.splits * a.vdim_s + (((int64_t)row * a.H + head) * a.splits + split) * 2;
 }
 
 // Final value of a head: sums / (denominator + exp(sink)), times the gate.
@@ -64,8 +88,11 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
     const int s = s0 + (j - j0);
     return a.ring > 0 && s >= a.ring ? s - a.ring : s;
   };
-  const int nc = a.vdim_s / 8, groups = 256 / nc;
-  const int chunk = tid % nc, grp = tid / nc;
+  const int nc = a.vdim_s / 8;
+  const bool pow2 = nc <= 32 && (nc & (nc - 1)) == 0;
+  const int sh = 31 - __builtin_clz(nc);
+  const int groups = pow2 ? 256 >> sh : 256 / nc;
+  const int grp = pow2 ? tid >> sh : tid / nc, chunk = pow2 ? tid & (nc - 1) : tid - grp * nc;
 
   constexpr int VU = 4;  // values a thread keeps of a tile (all of them with at least 16 key groups)
   Pack8<T> kv[4], vv[VU];
@@ -85,16 +112,9 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
 
   for (int r = wave; r < RH; r += 4) {
     const TQ* q = reinterpret_cast<const TQ*>(a.q) + (int64_t)row * a.ldq + (int64_t)(h0 + (r < nh ? r : 0)) * a.dim_s;
-    float ss = 0.f;
-    for (int c = lane; c < a.dim_s; c += 64) {
-      const float x = r < nh ? to_f(q[c]) : 0.f;
-      qs[r * a.dim_s + c] = x;
-      if (c < a.norm_dim) ss = __builtin_fmaf(x, x, ss);
-    }
-    if (a.norm_dim > 0) {  // a lane reads back what it wrote
-      const float s = 1.f / sqrtf(wave_sum(ss) / a.norm_dim + a.eps);
-      for (int c = lane; c < a.dim_s; c += 64) qs[r * a.dim_s + c] *= s;
-    }
+    const bool normed = a.norm_dim > 0;
+    normed_row(q, a.dim_s, normed ? a.norm_dim : 0, a.eps, lane,
+               [&](int c, float x) { qs[r * a.dim_s + c] = r < nh ? x : 0.f; });
   }
   if (tid < RH) {
     ms[tid] = -1e30f;
@@ -103,22 +123,19 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
   if (a.fresh_k && j0 <= pos && pos < j1) {
     const bool first = h0 == g * rep;  // one of the workgroups of a key/value head stores the rows
     if (wave == 2) {
-      const float* x = a.fresh_k + (int64_t)g * a.dim_s;
-      const float s = a.norm_dim > 0 ? rms_factor(x, a.norm_dim, a.eps, lane) : 1.f;
       T* o = const_cast<T*>(K) + slot(pos) * a.ldk;
-      for (int c = lane; c < a.dim_s; c += 64) {
-        const T t = from_f<T>(x[c] * s);
+      normed_row(a.fresh_k + (int64_t)g * a.dim_s, a.dim_s, a.norm_dim, a.eps, lane, [&](int c, float x) {
+        const T t = from_f<T>(x);
         kf[c] = t;
         if (first) o[c] = t;
-      }
+      });
     } else if (wave == 3) {
-      const float* x = a.fresh_v + (int64_t)g * a.vdim_s;
       T* o = const_cast<T*>(V) + slot(pos) * a.ldv;
-      for (int c = lane; c < a.vdim_s; c += 64) {
-        const T t = from_f<T>(x[c]);
+      normed_row(a.fresh_v + (int64_t)g * a.vdim_s, a.vdim_s, 0, 0.f, lane, [&](int c, float x) {
+        const T t = from_f<T>(x);
         vf[c] = t;
         if (first) o[c] = t;
-      }
+      });
     }
   }
   __syncthreads();
@@ -216,13 +233,13 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
   }
   // The key groups are added up: inside a wave by exchanges where whole groups lie side by side in it, the rest in
   // LDS, a head at a time.
-  const bool pow2 = nc <= 32 && (nc & (nc - 1)) == 0;
   if (pow2) {
+    for (int off = 32; off >= nc; off >>= 1) {
 #pragma unroll
-    for (int r = 0; r < RH; ++r)
+      for (int r = 0; r < RH; ++r)
 #pragma unroll
-      for (int e = 0; e < 8; ++e)
-        for (int off = 32; off >= nc; off >>= 1) acc[r][e] += __shfl_xor(acc[r][e], off, kWave);
+        for (int e = 0; e < 8; ++e) acc[r][e] += __shfl_xor(acc[r][e], off, kWave);
+    }
   }
   auto finish = [&](int r, int d, float t) {
     const int head = h0 + r;
@@ -231,11 +248,11 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
       const float f = attn_factor<TQ>(a, row, head, ms[r], ls[r], &c);
       reinterpret_cast<T*>(a.out)[((int64_t)row * a.H + head) * a.vdim_s + d] = from_f<T>(t * c * f);
     } else {
-      float* p = a.part + (((int64_t)row * a.H + head) * a.splits + split) * (a.vdim_s + 2);
-      p[d] = t;
+      part_sums(a, row, head, split)[d] = t;
       if (d == 0) {
-        p[a.vdim_s] = ms[r];
-        p[a.vdim_s + 1] = ls[r];
+        float* p = part_ml(a, row, head, split);
+        p[0] = ms[r];
+        p[1] = ls[r];
       }
     }
   };
@@ -249,7 +266,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
     }
     __syncthreads();
     for (int i = tid; i < nh * a.vdim_s; i += 256) {
-      const int r = i / a.vdim_s, d = i % a.vdim_s;
+      const int r = i >> (sh + 3), d = i & (a.vdim_s - 1);
       float t = 0.f;
       for (int w = 0; w < 4; ++w) t += red[(w * RH + r) * a.vdim_s + d];
       finish(r, d, t);
@@ -276,12 +293,12 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
 // share the splits of 64 entries.
 constexpr int kMaxSplits = 128;
 // By one wave: the weight of every split, and the maximum and denominator of all.
-__device__ __forceinline__ void split_weights(const float* __restrict__ p, int splits, int stride, int vdim_s, int lane,
-                                              float* ws, float* ml) {
+__device__ __forceinline__ void split_weights(const float* __restrict__ p, int splits, int lane, float* ws, float* ml) {
   const bool in0 = lane < splits, in1 = lane + 64 < splits;
-  const float* p0 = p + (int64_t)(in0 ? lane : 0) * stride + vdim_s;
-  const float* p1 = p + (int64_t)(in1 ? lane + 64 : 0) * stride + vdim_s;
-  const float m0 = in0 ? p0[0] : -1e30f, l0 = in0 ? p0[1] : 0.f, m1 = in1 ? p1[0] : -1e30f, l1 = in1 ? p1[1] : 0.f;
+  const float* p0 = p + (in0 ? lane : 0) * 2;
+  const float* p1 = p + (in1 ? lane + 64 : 0) * 2;
+  const float a0 = p0[0], b0 = p0[1], a1 = p1[0], b1 = p1[1];
+  const float m0 = in0 ? a0 : -1e30f, l0 = in0 ? b0 : 0.f, m1 = in1 ? a1 : -1e30f, l1 = in1 ? b1 : 0.f;
   const float m = butterfly_max<64>(fmaxf(m0, m1));
   const float w0 = exp_f(m0 - m), w1 = exp_f(m1 - m);
   if (in0) ws[lane] = w0;
@@ -295,14 +312,14 @@ __device__ __forceinline__ void split_weights(const float* __restrict__ p, int s
 template <typename TO, typename TQ>
 __global__ __launch_bounds__(256) void attn_merge_kernel(AttnArgs a, TO* __restrict__ out) {
   __shared__ float ws[kMaxSplits], acc[4][64], ml[2];
-  const int head = blockIdx.x, row = blockIdx.z, stride = a.vdim_s + 2, lane = threadIdx.x & 63, grp = threadIdx.x >> 6;
-  const float* p = a.part + ((int64_t)row * a.H + head) * a.splits * stride;
+  const int head = blockIdx.x, row = blockIdx.z, stride = a.vdim_s, lane = threadIdx.x & 63, grp = threadIdx.x >> 6;
+  const float* p = part_sums(a, row, head, 0);
   const int d = blockIdx.y * 64 + lane;
   constexpr int PV = 16;  // sums requested before the weights are known
   float v[PV];
 #pragma unroll
-  for (int i = 0; i < PV; ++i) v[i] = d < a.vdim_s && grp + 4 * i < a.splits ? p[(int64_t)(grp + 4 * i) * stride + d] : 0.f;
-  if (grp == 0) split_weights(p, a.splits, stride, a.vdim_s, lane, ws, ml);
+  for (int i = 0; i < PV; ++i) v[i] = p[(int64_t)min(grp + 4 * i, a.splits - 1) * stride + min(d, a.vdim_s - 1)];
+  if (grp == 0) split_weights(part_ml(a, row, head, 0), a.splits, lane, ws, ml);
   __syncthreads();
   float t = 0.f;
 #pragma unroll
@@ -356,49 +373,93 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(const float* __restr
 template <typename T>
 __global__ __launch_bounds__(256) void latent_out_kernel(AttnArgs a, const T* __restrict__ W, int vrows, T* __restrict__ out) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
-  float* lat = reinterpret_cast<float*>(smem_raw);
+  float* sums = reinterpret_cast<float*>(smem_raw);  // [thread groups][rank]
   __shared__ float ws[kMaxSplits], ml[2];
-  const int head = blockIdx.x, rank = a.vdim_s, stride = rank + 2, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const float* p = a.part + (int64_t)head * a.splits * stride;
-  constexpr int PR = 4;  // weight rows a wave requests ahead
+  const int head = blockIdx.x, rank = a.vdim_s, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const float* p = part_sums(a, 0, head, 0);
+  constexpr int PR = 8;  // weight rows a wave takes at a time
   Pack8<T> w[PR];
   const int r0 = blockIdx.y * 4 + wave, rstep = gridDim.y * 4;
+  const T* wh = W + (int64_t)head * vrows * rank;
+  auto load_rows = [&](int r) {
 #pragma unroll
-  for (int i = 0; i < PR; ++i) {
-    const int r = r0 + i * rstep;
-    if (r < vrows && lane * 8 < rank) w[i].load(W + ((int64_t)head * vrows + r) * rank + lane * 8);
-    else w[i].zero();
+    for (int i = 0; i < PR; ++i) w[i].load(wh + min(r + i * rstep, vrows - 1) * rank + min(lane * 8, rank - 8));
+  };
+  load_rows(r0);
+  // four channels per thread; the thread groups share the splits, eight of them requested together
+  const int nv = rank / 4, ng = nv < 256 ? 256 / nv : 1, grp = threadIdx.x / nv, v0 = threadIdx.x % nv;
+  const bool batch = a.splits >= 8 * ng && grp < ng;  // the first eight before the weights are known
+  float4_t first[8];
+  if (batch) {
+#pragma unroll
+    for (int u = 0; u < 8; ++u) first[u] = *reinterpret_cast<const float4_t*>(p + (grp + u * ng) * rank + v0 * 4);
   }
-  if (wave == 0) split_weights(p, a.splits, stride, rank, lane, ws, ml);
+  if (wave == 0) split_weights(part_ml(a, 0, head, 0), a.splits, lane, ws, ml);
   __syncthreads();
   float c;
   const float f = attn_factor<float>(a, 0, head, ml[0], ml[1], &c) * c;
-  typedef float float2_v __attribute__((ext_vector_type(2)));
-  for (int d = threadIdx.x * 2; d < rank; d += 512) {
-    float2_v t = {0.f, 0.f};
-#pragma unroll 16
-    for (int s = 0; s < a.splits; ++s) t += *reinterpret_cast<const float2_v*>(p + (int64_t)s * stride + d) * ws[s];
-    lat[d] = t[0] * f;
-    lat[d + 1] = t[1] * f;
+  const int step = ng * rank;
+  for (int v = v0; v < nv; v += 256) {  // one turn unless the latent has more than 1024 channels
+    if (grp < ng) {
+      float4_t t = {0.f, 0.f, 0.f, 0.f};
+      const float* q = p + grp * rank + v * 4;
+      int s = grp;
+      if (batch && v == v0) {
+#pragma unroll
+        for (int u = 0; u < 8; ++u) t += first[u] * ws[s + u * ng];
+        s += 8 * ng;
+        q += 8 * step;
+      }
+      for (; s + 7 * ng < a.splits; s += 8 * ng, q += 8 * step) {
+        float4_t x[8];
+#pragma unroll
+        for (int u = 0; u < 8; ++u) x[u] = *reinterpret_cast<const float4_t*>(q + u * step);
+#pragma unroll
+        for (int u = 0; u < 8; ++u) t += x[u] * ws[s + u * ng];
+      }
+      for (; s < a.splits; s += ng, q += step) t += *reinterpret_cast<const float4_t*>(q) * ws[s];
+      *reinterpret_cast<float4_t*>(sums + (grp * nv + v) * 4) = t * f;
+    }
   }
   __syncthreads();
-  for (int i = 0, r = r0; r < vrows; ++i, r += rstep) {
-    const T* wr = W + ((int64_t)head * vrows + r) * rank;
-    float acc = 0.f;
-    for (int k = lane * 8; k < rank; k += 512) {
-      Pack8<T> v;
-      if (k < 512 && i < PR) {
-#pragma unroll
-        for (int u = 0; u < PR; ++u)
-          if (u == i) v = w[u];
-      } else {
-        v.load(wr + k);
-      }
-#pragma unroll
-      for (int e = 0; e < 8; ++e) acc = __builtin_fmaf(v.get(e), lat[k + e], acc);
+  if (ng > 1) {
+    for (int d = threadIdx.x; d < rank; d += 256) {
+      float t = sums[d];
+      for (int g = 1; g < ng; ++g) t += sums[g * rank + d];
+      sums[d] = t;  // only this thread reads entry d of the other groups
     }
-    acc = wave_sum(acc);
-    if (lane == 0) out[(int64_t)head * vrows + r] = from_f<T>(acc);
+    __syncthreads();
+  }
+  const float* lat = sums;
+  for (int r = r0; r < vrows; r += PR * rstep) {
+    float sum[PR];
+#pragma unroll
+    for (int i = 0; i < PR; ++i) sum[i] = 0.f;
+    if (lane * 8 < rank) {
+      Pack8<float> x;
+      x.load(lat + lane * 8);
+#pragma unroll
+      for (int i = 0; i < PR; ++i)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) sum[i] = __builtin_fmaf(w[i].get(e), x.get(e), sum[i]);
+    }
+    for (int k = 512 + lane * 8; k < rank; k += 512) {
+#pragma unroll
+      for (int i = 0; i < PR; ++i) {
+        Pack8<T> v;
+        v.load(wh + min(r + i * rstep, vrows - 1) * rank + k);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) sum[i] = __builtin_fmaf(v.get(e), lat[k + e], sum[i]);
+      }
+    }
+    if (r + PR * rstep < vrows) load_rows(r + PR * rstep);
+    float mine = 0.f;
+#pragma unroll
+    for (int i = 0; i < PR; ++i) {
+      const float t = wave_sum(sum[i]);
+      if (lane == i) mine = t;
+    }
+    if (lane < PR && r + lane * rstep < vrows) out[(int64_t)head * vrows + r + lane * rstep] = from_f<T>(mine);
   }
 }
 

@@ -350,11 +350,16 @@ using DeltaStepArgs = dvDeltaStepArgs;
 template <typename T>
 __device__ __forceinline__ float dot_row(const T* __restrict__ w, const float* x, int n) {
   float acc = 0.f;
-  for (int i = 0; i < n; i += 8) {
-    Pack8<T> v;
-    v.load(w + i);
+  for (int i = 0; i < n; i += 64) {  // eight packets requested together
+    Pack8<T> v[8];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) acc = __builtin_fmaf(v.get(e), x[i + e], acc);
+    for (int u = 0; u < 8; ++u) v[u].load(w + min(i + u * 8, n - 8));
+#pragma unroll
+    for (int u = 0; u < 8; ++u)
+      if (i + u * 8 < n) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc = __builtin_fmaf(v[u].get(e), x[i + u * 8 + e], acc);
+      }
   }
   return acc;
 }

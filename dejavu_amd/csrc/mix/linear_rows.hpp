@@ -29,20 +29,35 @@ __device__ __forceinline__ void stage_row(const RowsArgs& a, T* xs, float* red) 
   const int tid = threadIdx.x, K = a.K;
   if constexpr (BEFORE == DV_ROW_PLAIN) {
     const T* x = reinterpret_cast<const T*>(a.x);
-    for (int i = tid * 8; i < K; i += 256 * 8) {
-      Pack8<T> v;
-      v.load(x + i);
-      *reinterpret_cast<Pack8<T>*>(xs + i) = v;
+    for (int i = tid * 8; i < K; i += 4 * 2048) {  // four packets requested together
+      Pack8<T> v[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) v[u].load(x + min(i + u * 2048, K - 8));
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+        if (i + u * 2048 < K) *reinterpret_cast<Pack8<T>*>(xs + i + u * 2048) = v[u];
     }
   } else if constexpr (BEFORE == DV_ROW_RMS) {
     const float* x = reinterpret_cast<const float*>(a.x);
-    float ss = 0.f;
-    for (int i = tid; i < a.norm_dim; i += 256) ss = __builtin_fmaf(x[i], x[i], ss);
+    constexpr int NX = 8;  // values and weights a thread keeps; longer rows read the rest again
+    float v[NX], w[NX], ss = 0.f;
+#pragma unroll
+    for (int u = 0; u < NX; ++u) {
+      v[u] = x[min(tid + u * 256, K - 1)];
+      w[u] = a.xw[min(tid + u * 256, K - 1)];
+    }
+#pragma unroll
+    for (int u = 0; u < NX; ++u)
+      if (tid + u * 256 < a.norm_dim) ss = __builtin_fmaf(v[u], v[u], ss);
+    for (int i = tid + NX * 256; i < a.norm_dim; i += 256) ss = __builtin_fmaf(x[i], x[i], ss);
     ss = wave_sum(ss);
     if ((tid & 63) == 0) red[tid >> 6] = ss;
     __syncthreads();
     const float s = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / a.norm_dim + a.eps);
-    for (int i = tid; i < K; i += 256) xs[i] = from_f<T>(x[i] * s * a.xw[i]);
+#pragma unroll
+    for (int u = 0; u < NX; ++u)
+      if (tid + u * 256 < K) xs[tid + u * 256] = from_f<T>(v[u] * s * w[u]);
+    for (int i = tid + NX * 256; i < K; i += 256) xs[i] = from_f<T>(x[i] * s * a.xw[i]);
   } else {
     // a row of 16 lanes per head; eight channels per lane at a time, the first 128 kept in registers
     const float* x = reinterpret_cast<const float*>(a.x);

@@ -9,7 +9,7 @@ using ConvArgs = dvConvArgs;
 
 // A lane owns eight channels of one head and walks TB consecutive tokens with the last TAPS inputs in registers; the
 // LPH lanes of a head (a power of two, 8 LPH >= stride) add up its norm.  Grid: (units of heads, token blocks).
-constexpr int kConvTokens = 16;
+constexpr int kConvTokens = 8;
 
 template <int LPH>
 __device__ __forceinline__ float lanes_sum(float v) {

@@ -4,20 +4,30 @@
 
 namespace dv {
 
-// x = x0 = embed[token]; h = norm(x).  One workgroup per token.
+// x = x0 = embed[token]; h = norm(x).  Eight channels per thread; grid (tokens, ceil(width / 2048)).
 template <typename T>
 __global__ __launch_bounds__(256) void embed_norm_kernel(const int64_t* __restrict__ tokens, int64_t vocab,
                                                          const T* __restrict__ embed, int width, float* __restrict__ x,
                                                          float* __restrict__ x0, DynTanh norm, T* __restrict__ h) {
   const int64_t i = blockIdx.x;
+  const int c = (blockIdx.y * 256 + threadIdx.x) * 8;
+  if (c >= width) return;
   const int64_t tok = tokens[i];
-  const bool ok = tok >= 0 && tok < vocab;
-  for (int c = threadIdx.x; c < width; c += blockDim.x) {
-    const float v = ok ? to_f(embed[tok * width + c]) : 0.f;
-    x[i * width + c] = v;
-    if (x0) x0[i * width + c] = v;
-    h[i * width + c] = from_f<T>(dyn_tanh(v, norm, c));
+  Pack8<T> v;
+  if (tok >= 0 && tok < vocab) v.load(embed + tok * width + c);
+  else v.zero();
+  Pack8<float> f;
+  __attribute__((aligned(16))) T o[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const float t = v.get(e);
+    if (e < 4) f.a[e] = t;
+    else f.b[e - 4] = t;
+    o[e] = from_f<T>(dyn_tanh(t, norm, c + e));
   }
+  *reinterpret_cast<Pack8<float>*>(x + i * width + c) = f;
+  if (x0) *reinterpret_cast<Pack8<float>*>(x0 + i * width + c) = f;
+  *reinterpret_cast<Pack8<T>*>(h + i * width + c) = *reinterpret_cast<const Pack8<T>*>(o);
 }
 
 using ResidualArgs = dvResidual;

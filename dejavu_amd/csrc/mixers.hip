@@ -143,10 +143,20 @@ int delta_scan(const DeltaArgs& a, hipStream_t s) {
   return DV_OK;
 }
 
+template <int RT, int HT>
+int latent_heads(const AttnArgs& a, hipStream_t s) {
+  constexpr int NW = RT >= 8 ? 8 : 4;
+  return launch_lds<latent_attn_kernel<RT, HT, NW>>(dim3(a.splits, (a.H + 16 * HT - 1) / (16 * HT)), dim3(64 * NW),
+                                                    latent_lds_bytes<RT, HT, NW>(), s, a);
+}
+// Sixteen heads per workgroup; with many heads (workgroups enough without it) and room in LDS 32, so that the cache is
+// read half as often.
 template <int RT>
 int latent_tiles(const AttnArgs& a, hipStream_t s) {
-  if (a.H <= 16) return launch_lds<latent_attn_kernel<RT, 1>>(dim3(a.splits, 1), dim3(256), latent_lds_bytes<RT, 1>(), s, a);
-  return launch_lds<latent_attn_kernel<RT, 2>>(dim3(a.splits, (a.H + 31) / 32), dim3(256), latent_lds_bytes<RT, 2>(), s, a);
+  if constexpr (RT <= 16) {
+    if (a.splits * ((a.H + 15) / 16) > 512) return latent_heads<RT, 2>(a, s);
+  }
+  return latent_heads<RT, 1>(a, s);
 }
 
 int attn_args_ok(const AttnArgs* a) {
@@ -175,12 +185,14 @@ int dv_mix_embed(int dtype, const void* tokens, int64_t vocab, const void* embed
                  const dvDynTanh* norm, void* h, void* stream) {
   if (!dtype_ok(dtype) || !tokens || !embed || n < 1 || width < 1 || !x || !norm || !norm->w || !norm->b || !h)
     return DV_ERR_INVALID_ARG;
+  if (width % 8 || !al16(embed) || !al16(x) || !al16(x0) || !al16(h)) return DV_ERR_ALIGNMENT;
   const int64_t* t = reinterpret_cast<const int64_t*>(tokens);
+  const dim3 grid(n, (width + 2047) / 2048);
   if (dtype == DV_BF16)
-    hipLaunchKernelGGL((embed_norm_kernel<bf16_t>), dim3(n), dim3(256), 0, st(stream), t, vocab, (const bf16_t*)embed,
+    hipLaunchKernelGGL((embed_norm_kernel<bf16_t>), grid, dim3(256), 0, st(stream), t, vocab, (const bf16_t*)embed,
                        width, x, x0, *norm, (bf16_t*)h);
   else
-    hipLaunchKernelGGL((embed_norm_kernel<float>), dim3(n), dim3(256), 0, st(stream), t, vocab, (const float*)embed,
+    hipLaunchKernelGGL((embed_norm_kernel<float>), grid, dim3(256), 0, st(stream), t, vocab, (const float*)embed,
                        width, x, x0, *norm, (float*)h);
   return launched();
 }
@@ -390,7 +402,7 @@ int dv_mix_latent_attn(int dtype, const dvAttnArgs* a, const void* W, int vrows,
   else rc = attn_rows_any<bf16_t, float>(*a, st(stream));
   if (rc != DV_OK) return rc;
   const dim3 grid(a->H, vrows <= 32 ? 1 : (vrows <= 64 ? 2 : 4));
-  const size_t lds = (size_t)rank * 4;
+  const size_t lds = (size_t)(rank / 4 < 256 ? 256 / (rank / 4) : 1) * rank * 4;
   if (dtype == DV_BF16)
     hipLaunchKernelGGL((latent_out_kernel<bf16_t>), grid, dim3(256), lds, st(stream), *a, (const bf16_t*)W, vrows, (bf16_t*)out);
   else

@@ -266,7 +266,7 @@ def ring_copy(buf: torch.Tensor, ring: torch.Tensor, first: int, to_ring: bool) 
 def decode_splits(keys: int) -> int:
     """Workgroups that share the keys of a decode row.  ``keys`` is the most there can be: the value may not depend
     on the position, which captured steps only know on the device."""
-    return max(1, min(64, (keys + 63) // 64), min(128, keys // 128))
+    return max(1, min(16, (keys + 63) // 64), min(128, keys // 128))
 
 
 def _attn_args(q, k, v, n, H, G, dim_s, vdim_s, scale, sink, gate, window, ring, base, pos_dev, pos):
@@ -332,7 +332,7 @@ def latent_attention_row(q, k_up, v_up, cache, heads, scale, gate, pos_dev, pos)
           "dv_mix_latent_absorb")
     a = _attn_args(ql.view(1, -1), cache, cache, 1, heads, 1, rank, rank, scale, None, None, None, 0, 0, pos_dev, pos)
     a.gate, a.ldg = gate.data_ptr(), heads
-    a.splits = max(2, decode_splits(cache.shape[0]))
+    a.splits = max(2, min(128, (cache.shape[0] + 127) // 128))
     part = torch.empty(heads * a.splits * (rank + 2), dtype=torch.float32, device=q.device)
     a.part = part.data_ptr()
     out = torch.empty(1, heads * vdim_s, dtype=cache.dtype, device=q.device)

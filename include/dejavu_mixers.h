@@ -122,7 +122,7 @@ typedef struct {
   const int* pos_dev;      /* position of query row 0 */
   int pos_host;
   void* out;               /* [n][H][vdim_s] */
-  float* part;             /* splits > 1 (at most 128): [n][H][splits][vdim_s + 2] scratch */
+  float* part;             /* splits > 1 (at most 128): n H splits (vdim_s + 2) floats of scratch */
   int splits;
   const float* fresh_k;    /* decode: this token's key / value rows (fp32), stored in their slots first */
   const float* fresh_v;
