@@ -2,7 +2,7 @@
 
 Steps come as JSON lines on standard input:
 
-    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
+    {"step": 0, "entries": [{"id": "s1", "tokens": [11, 4, 250, 9], "want": [3]}], "end": []}
 
 An entry brings the next tokens of a sequence (a new id starts one) and the places among them whose logits are wanted.
 ``OUT/<step>.f32`` gets those logits, little-endian fp32 [wanted, vocab], in the order of the entries and of ``want``;

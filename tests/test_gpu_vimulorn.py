@@ -246,6 +246,46 @@ def test_delta_rule_scan(heads, kv_heads, dim, vdim):
         close(St.view(heads, -1), S.transpose(0, 2, 1).reshape(heads, -1), 1e-5, "state")
 
 
+def test_delta_rule_scan_of_a_long_portion():
+    """More tokens than the kernels take at a time."""
+    from dejavu_amd import mixer_ops as ops
+
+    rng = np.random.default_rng(8)
+    T, dim, vdim = 4133, 8, 8
+    q, k = (host(dev(V.unit_norm(rng.normal(size=(T, 1, dim))))) for _ in range(2))
+    v, beta = host(dev(rng.normal(size=(T, 1, vdim)))), host(dev(V.sigmoid(rng.normal(size=(T, 1)))))
+    g = host(dev(np.exp(-np.exp(rng.normal(size=(T, 1, dim)) - 4))))
+    S = np.zeros((1, dim, vdim))
+    want = V.delta_rule(q, k, v, g, beta, S)
+    St = torch.zeros(1, vdim, dim, device="cuda")
+    got = ops.delta_scan(*(dev(a.reshape(T, -1)) for a in (q, k, v, g, beta)), St, 1, 1)
+    close(got.view(T, -1), want.reshape(T, -1), 1e-5, "read-outs")
+    close(St[0], S[0].T, 1e-5, "state")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,dim,rank,vdim,cap", [(20, 32, 200, 16, 300), (5, 64, 512, 72, 700), (33, 16, 520, 8, 260),
+                                                 (80, 8, 64, 8, 16500), (3, 8, 1032, 40, 130)])
+def test_latent_decode_at_many_sizes(H, dim, rank, vdim, cap, dtype):
+    """Latents of every width the kernels distinguish, many and few heads, positions at the edges of tiles and splits."""
+    from dejavu_amd import mixer_ops as ops
+
+    rng = np.random.default_rng(rank)
+    c, ku, vu = (host(dev(rng.normal(size=s) * f, dtype)) for s, f in
+                 (((cap, rank), 1.0), ((H * dim, rank), (rank * dim) ** -0.5), ((H * vdim, rank), rank ** -0.5)))
+    q, gate = host(dev(rng.normal(size=(1, H * dim)) * 3)), host(dev(rng.normal(size=H)))
+    ct, kt, vt = dev(c, dtype), dev(ku, dtype), dev(vu, dtype)
+    ql = np.einsum("hdr,hd->hr", ku.reshape(H, dim, rank), q.reshape(H, dim))
+    for pos in (0, 63, 64, 128, 129, cap - 1):
+        s = ql @ c[:pos + 1].T * 0.5
+        p = np.exp(s - s.max(-1, keepdims=True))
+        lat = (p / p.sum(-1, keepdims=True)) @ c[:pos + 1] * V.sigmoid(gate)[:, None]
+        want = np.einsum("hvr,hr->hv", vu.reshape(H, vdim, rank), lat)
+        where = torch.tensor([pos], dtype=torch.int32, device="cuda") if pos % 2 else None
+        got = ops.latent_attention_row(dev(q), kt, vt, ct, H, 0.5, dev(gate), where, 0 if pos % 2 else pos)
+        close(got, want.reshape(1, -1), OP_LIMIT[dtype], f"position {pos}")
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("name", sorted(U.CONFIGS))
 def test_mixers_alone(name, dtype):
@@ -306,8 +346,8 @@ def test_sequences_side_by_side_and_memory_used_again(dtype):
 
     cfg, P, model = model_of("mixed", dtype)
     pool = SequencePool(90)
-    for round_ in range(2):
-        seqs = {n: U.tokens(cfg, ln, seed=10 * round_ + ln) for n, ln in (("a", 90), ("b", 37), ("c", 1))}
+    for turn in range(2):
+        seqs = {n: U.tokens(cfg, ln, seed=10 * turn + ln) for n, ln in (("a", 90), ("b", 37), ("c", 1))}
         want = {n: V.forward(cfg, P, t) for n, t in seqs.items()}
         got = {n: [] for n in seqs}
         at = {n: 0 for n in seqs}
@@ -318,11 +358,11 @@ def test_sequences_side_by_side_and_memory_used_again(dtype):
                 part = seqs[n][at[n]:at[n] + sizes[i % len(sizes)]]
                 i += 1
                 if part:
-                    got[n].append(feed(model, pool.get(f"{n}{round_}"), part, [len(part)]))
+                    got[n].append(feed(model, pool.get(f"{n}{turn}"), part, [len(part)]))
                     at[n] += len(part)
         for n in seqs:
-            close(np.concatenate(got[n]), want[n], LIMIT[dtype], f"sequence {n}, turn {round_}")
-            pool.end(f"{n}{round_}")
+            close(np.concatenate(got[n]), want[n], LIMIT[dtype], f"sequence {n}, turn {turn}")
+            pool.end(f"{n}{turn}")
     assert len(pool.free) == 3 and not pool.live
 
 

@@ -42,8 +42,8 @@ CONFIGS = {
     "mixed": config(100, 213, [(window(4, 2, 20, 12, 4, 9), mlp(75, 1.5)), (delta(4, 2, 12, 20, 3), mlp(50, 3.0)),
                                (latent(3, 20, 28, 18, 44), None), (delta(2, 1, 40, 8, 2), mlp(64, 0.7))],
                     loop=(1, 4, 3), eps=3e-5),
-    # no loop, one key/value head, window of one tap and wide heads, a layer without feed-forward at the end
-    "plain": config(64, 96, [(latent(2, 8, 8, 16, 8, scale=0.5), mlp(32, 4.0)), (window(6, 1, 32, 64, 1, 70), None),
+    # no loop, one key/value head, one tap, a window longer than some sequences, layers without feed-forward
+    "plain": config(64, 96, [(latent(2, 8, 8, 16, 8, scale=0.5), mlp(32, 4.0)), (window(6, 1, 32, 64, 1, 100), None),
                              (delta(3, 3, 72, 24, 5), None)]),
     # loop from the first layer, longest taps first, a window of one token
     "loop0": config(48, 65, [(delta(2, 2, 16, 16, 4), mlp(40, 2.5)), (window(2, 2, 16, 8, 2, 1), mlp(24, 1.0)),
