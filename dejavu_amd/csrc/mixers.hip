@@ -51,7 +51,7 @@ int launch_lds(dim3 grid, dim3 block, size_t lds, hipStream_t s, A... args) {
 // ---- one row ---------------------------------------------------------------
 template <typename T, int BEFORE, int AFTER>
 int linear_row(const RowsArgs& a, hipStream_t s) {
-  constexpr int R = AFTER == DV_OUT_GLU ? 2 : 2, U = sizeof(T) == 2 ? 4 : 2;
+  constexpr int R = 2, U = sizeof(T) == 2 ? 4 : 2;
   const int ntasks = (a.M + R - 1) / R;
   int blocks = (ntasks + 3) / 4;
   if (blocks > 2048) blocks = 2048;
