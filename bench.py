@@ -796,8 +796,8 @@ def vimulorn_kernels(torch, model, prompt, context):
     elementwise("norm + residual + norm", lambda a: mo.residual(y, st, norm, norm), n * width * 12)
     gu = rnd(n, mlp.gate_up.shape[0])
     out = torch.empty(n, mlp.gate_up.shape[0] // 2, dtype=bf, device=dev)
-    elementwise("clamped gated unit", lambda a: mo.lib.dv_mix_clamped_glu(
-        0, gu.data_ptr(), out.numel(), 7.0, out.data_ptr(), mo._stream()), gu.numel() * 3)
+    elementwise("clamped gated unit", lambda a: mo.lib.dv_mix_glu(
+        0, gu.data_ptr(), out.numel(), 0, 7.0, out.data_ptr(), mo._stream()), gu.numel() * 3)
     p = rnd(n, win.channels)
     k, v, qq = torch.empty(n, G * hd, dtype=bf, device=dev), torch.empty(n, G * hd, dtype=bf, device=dev), torch.empty(n, H * hd, dtype=bf, device=dev)
     cst = win.new_state(context)["conv"]

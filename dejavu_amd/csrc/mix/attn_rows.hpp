@@ -7,13 +7,24 @@ namespace dv {
 
 using AttnArgs = dvAttnArgs;
 
-// By one wave: put(c, x[c] / rms(x)) for every entry, the mean over norm_dim entries (0: put(c, x[c])).
+// The oldest position that the query at `pos` sees.
+__device__ __forceinline__ int oldest_key(const AttnArgs& a, int pos) {
+  if (a.window > 0) return max(0, pos - a.window + 1);
+  return a.chunk > 0 ? pos - pos % a.chunk : 0;
+}
+
+// By one wave: put(c, x[c] / rms(x) * w[c]) for every entry, the mean over norm_dim entries (0: put(c, x[c])); w may be
+// null.
 template <typename T, typename F>
-__device__ __forceinline__ void normed_row(const T* __restrict__ x, int n, int norm_dim, float eps, int lane, F put) {
+__device__ __forceinline__ void normed_row(const T* __restrict__ x, int n, int norm_dim, float eps,
+                                           const float* __restrict__ w, int lane, F put) {
   constexpr int NX = 4;  // values a lane keeps; longer rows read the rest again
-  float v[NX];
+  float v[NX], wv[NX];
 #pragma unroll
-  for (int u = 0; u < NX; ++u) v[u] = to_f(x[min(lane + u * 64, n - 1)]);
+  for (int u = 0; u < NX; ++u) {
+    v[u] = to_f(x[min(lane + u * 64, n - 1)]);
+    wv[u] = w ? w[min(lane + u * 64, n - 1)] : 1.f;
+  }
   float s = 1.f;
   if (norm_dim > 0) {
     float ss = 0.f;
@@ -25,8 +36,8 @@ __device__ __forceinline__ void normed_row(const T* __restrict__ x, int n, int n
   }
 #pragma unroll
   for (int u = 0; u < NX; ++u)
-    if (lane + u * 64 < n) put(lane + u * 64, v[u] * s);
-  for (int c = lane + NX * 64; c < n; c += 64) put(c, to_f(x[c]) * s);
+    if (lane + u * 64 < n) put(lane + u * 64, v[u] * s * wv[u]);
+  for (int c = lane + NX * 64; c < n; c += 64) put(c, to_f(x[c]) * s * (w ? w[c] : 1.f));
 }
 
 // Partial sums of a split: `part` holds [n][H][splits][vdim_s] sums, then [n][H][splits][2] (maximum, denominator).
@@ -75,14 +86,14 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
   const int nh = min(RH, (g + 1) * rep - h0);
   const int row = blockIdx.z, split = blockIdx.x;
   const int pos = seq_position(a.pos_dev, a.pos_host) + row;
-  const int lo = a.window > 0 ? max(0, pos - a.window + 1) : 0;
+  const int lo = oldest_key(a, pos);
   const int nk = pos + 1 - lo;
   const int per = ((nk + a.splits - 1) / a.splits + kAttnKeys - 1) / kAttnKeys * kAttnKeys;
   const int j0 = lo + split * per, j1 = min(pos + 1, j0 + per);
   const int fresh = a.fresh_k ? pos : -1;
   const T* K = reinterpret_cast<const T*>(a.k) + (int64_t)g * a.k_head;
   const T* V = reinterpret_cast<const T*>(a.v) + (int64_t)g * a.v_head;
-  // keys of a split lie in consecutive slots but for one wrap (a ring holds at least the window)
+  // keys of a split lie in consecutive slots but for one wrap (a ring holds at least the window or chunk)
   const int s0 = a.ring > 0 ? j0 % a.ring : j0 - a.base;
   auto slot = [&](int j) -> int64_t {
     const int s = s0 + (j - j0);
@@ -95,8 +106,18 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
   const int grp = pow2 ? tid >> sh : tid / nc, chunk = pow2 ? tid & (nc - 1) : tid - grp * nc;
 
   constexpr int VU = 4;  // values a thread keeps of a tile (all of them with at least 16 key groups)
+  constexpr int RW = (RH + 3) / 4;  // heads whose softmax a wave does
   Pack8<T> kv[4], vv[VU];
+  float rb[RW];  // their biases for key `lane` of a tile
   auto load_tile = [&](int jt) {
+#pragma unroll
+    for (int u = 0; u < RW; ++u) {
+      rb[u] = 0.f;
+      if (a.rel) {
+        const int r = min(wave + u * 4, nh - 1), n = min(max(pos - jt - lane, 0), a.rel_len - 1);
+        rb[u] = a.rel[(int64_t)(h0 + r) * a.rel_len + n];
+      }
+    }
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
       const int j = min(jt + u * 16 + (tid >> 4), j1 - 1);
@@ -113,7 +134,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
   for (int r = wave; r < RH; r += 4) {
     const TQ* q = reinterpret_cast<const TQ*>(a.q) + (int64_t)row * a.ldq + (int64_t)(h0 + (r < nh ? r : 0)) * a.dim_s;
     const bool normed = a.norm_dim > 0;
-    normed_row(q, a.dim_s, normed ? a.norm_dim : 0, a.eps, lane,
+    normed_row(q, a.dim_s, normed ? a.norm_dim : 0, a.eps, a.q_w, lane,
                [&](int c, float x) { qs[r * a.dim_s + c] = r < nh ? x : 0.f; });
   }
   if (tid < RH) {
@@ -124,14 +145,17 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
     const bool first = h0 == g * rep;  // one of the workgroups of a key/value head stores the rows
     if (wave == 2) {
       T* o = const_cast<T*>(K) + slot(pos) * a.ldk;
-      normed_row(a.fresh_k + (int64_t)g * a.dim_s, a.dim_s, a.norm_dim, a.eps, lane, [&](int c, float x) {
+      normed_row(a.fresh_k + (int64_t)g * a.dim_s, a.dim_s, a.norm_dim, a.eps, a.k_w, lane, [&](int c, float x) {
         const T t = from_f<T>(x);
         kf[c] = t;
         if (first) o[c] = t;
       });
     } else if (wave == 3) {
       T* o = const_cast<T*>(V) + slot(pos) * a.ldv;
-      normed_row(a.fresh_v + (int64_t)g * a.vdim_s, a.vdim_s, 0, 0.f, lane, [&](int c, float x) {
+      const float* other = a.other_v ? a.other_v + (int64_t)g * a.vdim_s : nullptr;
+      const float lam = other ? *a.lambda : 0.f;
+      normed_row(a.fresh_v + (int64_t)g * a.vdim_s, a.vdim_s, 0, 0.f, nullptr, lane, [&](int c, float x) {
+        if (other) x = __builtin_fmaf(lam, other[c], (1.f - lam) * x);
         const T t = from_f<T>(x);
         vf[c] = t;
         if (first) o[c] = t;
@@ -183,9 +207,12 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnArgs a) {
         if (sub == (r & 15)) ps[r][u * 16 + (tid >> 4)] = d * a.scale;
       }
     __syncthreads();
-    for (int r = wave; r < RH; r += 4) {
+#pragma unroll
+    for (int u = 0; u < RW; ++u) {
+      const int r = wave + u * 4;
+      if (r >= RH) break;
       const bool in = jt + lane < j1;
-      const float sc = in ? ps[r][lane] : -INFINITY;
+      const float sc = in ? ps[r][lane] + rb[u] : -INFINITY;
       const float m0 = ms[r], m1 = fmaxf(m0, butterfly_max<64>(sc));
       const float p = in ? exp_f(sc - m1) : 0.f;
       const float sum = wave_sum(p), c = exp_f(m0 - m1);

@@ -1,5 +1,6 @@
 // Causal softmax attention of a portion of a prompt on the matrix cores (bf16 operands, fp32 scores and sums):
-// grouped key/value heads, different query/key and value sizes, optional sliding window, sink and output gate.
+// grouped key/value heads, different query/key and value sizes, optional sliding window or chunks, bias by distance,
+// sink and output gate.
 //
 // A workgroup takes 128 queries of one head, a wave 32 of them.  Scores are computed transposed (keys x queries),
 // so a lane holds the scores of ONE query: the softmax is lane-local but for one exchange between the half waves,
@@ -18,6 +19,7 @@ __global__ __launch_bounds__(256) void attn_tiles_kernel(AttnArgs a, int keys /*
   constexpr int DL = DT * 16 + 8, VL = kTileK + 4;  // LDS row lengths
   __shared__ __attribute__((aligned(16))) bf16_t ks[kTileK * DL];
   __shared__ __attribute__((aligned(16))) bf16_t vs[VT * 32 * VL];
+  __shared__ float rs[kTileQ + kTileK];  // biases of a tile: entry i is the distance off + q0 - k0 - (kTileK - 1) + i
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l32 = lane & 31, hh = lane >> 5;
   const int head = blockIdx.x % a.H, g = head / (a.H / a.G);
   const int nblk = (a.n + kTileQ - 1) / kTileQ;
@@ -39,15 +41,24 @@ __global__ __launch_bounds__(256) void attn_tiles_kernel(AttnArgs a, int keys /*
     }
   }
   const int qslot = off + qi;
+  auto oldest_slot = [&](int q) { return max(0, oldest_key(a, a.pos_host + q) - a.base); };
+  const int klo = oldest_slot(min(qi, a.n - 1));
+  const int wklo = __builtin_amdgcn_readfirstlane(klo);
+  const int wkhi = oldest_slot(min(q0 + wave * 32 + 31, a.n - 1));
   const int wlo = off + q0 + wave * 32, whi = min(off + q0 + wave * 32 + 31, off + a.n - 1);  // slots of the wave
-  const int blo = off + q0, bhi = min(off + q0 + kTileQ - 1, off + a.n - 1);
-  const int first = a.window > 0 ? max(0, blo - a.window + 1) / kTileK * kTileK : 0;
+  const int bhi = min(off + q0 + kTileQ - 1, off + a.n - 1);
+  const int first = oldest_slot(q0) / kTileK * kTileK;
+  const float* rel = a.rel ? a.rel + (int64_t)head * a.rel_len : nullptr;
+  constexpr float kLog2e = 1.44269504088896340736f;
+  const float rel_far = rel ? rel[a.rel_len - 1] * kLog2e : 0.f;
+  float rr = 0.f;
   const int last = bhi;
 
   constexpr int KV = (kTileK * DT * 2 + 255) / 256;       // 16-byte loads of K per thread
   constexpr int VV = (kTileK / 2 * VT * 4 + 255) / 256;   // pairs of 16-byte loads of V per thread
   uint4_t kr[KV], vr[VV][2];
   auto fetch = [&](int k0) {
+    if (rel) rr = rel[min(max(off + q0 - k0 - (kTileK - 1) + tid, 0), a.rel_len - 1)] * kLog2e;
     // past the last key the weights are zero; past the last channel the queries are, or nothing is stored
 #pragma unroll
     for (int i = 0; i < KV; ++i) {
@@ -62,6 +73,7 @@ __global__ __launch_bounds__(256) void attn_tiles_kernel(AttnArgs a, int keys /*
     }
   };
   auto put = [&]() {
+    if (rel && tid < kTileQ + kTileK) rs[tid] = rr;
 #pragma unroll
     for (int i = 0; i < KV; ++i) {
       const int at = i * 256 + tid, r = at / (DT * 2), d = at % (DT * 2) * 8;
@@ -87,7 +99,7 @@ __global__ __launch_bounds__(256) void attn_tiles_kernel(AttnArgs a, int keys /*
 #pragma unroll
     for (int i = 0; i < 16; ++i) o[t][i] = 0.f;
   float m = -1e30f, l = 0.f;  // l: this half wave's share
-  const float sc = a.scale * 1.44269504088896340736f;
+  const float sc = a.scale * kLog2e;
 
   fetch(first);
   for (int k0 = first; k0 <= last; k0 += kTileK) {
@@ -95,7 +107,7 @@ __global__ __launch_bounds__(256) void attn_tiles_kernel(AttnArgs a, int keys /*
     put();
     __syncthreads();
     if (k0 + kTileK <= last) fetch(k0 + kTileK);
-    const bool seen = k0 <= whi && (a.window <= 0 || k0 + kTileK - 1 > wlo - a.window);
+    const bool seen = k0 <= whi && k0 + kTileK - 1 >= wklo;
     if (!seen) continue;
     float16_t s[2];
 #pragma unroll
@@ -108,16 +120,28 @@ __global__ __launch_bounds__(256) void attn_tiles_kernel(AttnArgs a, int keys /*
         s[kt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, qf[t], s[kt], 0, 0, 0);
       }
     }
-    const bool full = k0 + kTileK - 1 <= wlo && (a.window <= 0 || k0 > whi - a.window);
+    const bool full = k0 + kTileK - 1 <= wlo && k0 >= wkhi;
+    if (rel && wlo - (k0 + kTileK - 1) < a.rel_len - 1) {
+      const float* rp = rs + wave * 32 + l32 + kTileK - 1 - 4 * hh;
+#pragma unroll
+      for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) s[kt][i] = __builtin_fmaf(s[kt][i], sc, rp[-(kt * 32 + 8 * (i >> 2) + (i & 3))]);
+    } else {  // no bias, or one for all
+#pragma unroll
+      for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) s[kt][i] = __builtin_fmaf(s[kt][i], sc, rel_far);
+    }
     float mx = -INFINITY;
 #pragma unroll
     for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
       for (int i = 0; i < 16; ++i) {
-        float x = s[kt][i] * sc;
+        float x = s[kt][i];
         if (!full) {
           const int key = k0 + kt * 32 + 8 * (i >> 2) + 4 * hh + (i & 3);
-          if (key > qslot || (a.window > 0 && key <= qslot - a.window)) x = -INFINITY;
+          if (key > qslot || key < klo) x = -INFINITY;
         }
         s[kt][i] = x;
         mx = fmaxf(mx, x);

@@ -48,6 +48,19 @@ __device__ __forceinline__ float to_f(bf16_t v) { return (float)v; }
 template <typename T>
 __device__ __forceinline__ T from_f(float v) { return (T)v; }
 
+// Four consecutive values in the storage type.
+template <typename T>
+__device__ __forceinline__ void store_quad(T* p, const float4_t& v) {
+  typedef T quad_t __attribute__((ext_vector_type(4)));
+  *reinterpret_cast<quad_t*>(p) = quad_t{from_f<T>(v[0]), from_f<T>(v[1]), from_f<T>(v[2]), from_f<T>(v[3])};
+}
+template <typename T>
+__device__ __forceinline__ float4_t load_quad(const T* p) {
+  typedef T quad_t __attribute__((ext_vector_type(4)));
+  const quad_t v = *reinterpret_cast<const quad_t*>(p);
+  return float4_t{to_f(v[0]), to_f(v[1]), to_f(v[2]), to_f(v[3])};
+}
+
 // Sum over the 16 lanes of a DPP row; every lane ends with the total.
 template <int CTRL>
 __device__ __forceinline__ float dpp_add(float v) {

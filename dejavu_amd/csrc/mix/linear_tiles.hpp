@@ -87,12 +87,16 @@ __global__ __launch_bounds__(256) void linear_tiles_kernel(TileArgs a) {
     const int tile = q >> 6, ln = q & 63;
     const int m = m0 + (tile / NT) * 16 + (ln >> 4) * 4, n = n0 + (tile % NT) * 16 + (ln & 15);
     if (n >= a.n) continue;
-    const float4_t v = red[0][tile][ln];
+    float4_t v = red[0][tile][ln];
+    if (AFTER != DV_OUT_GLU && a.bias) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] += to_f(reinterpret_cast<const bf16_t*>(a.bias)[min(m + e, a.M - 1)]);
+    }
     if constexpr (AFTER == DV_OUT_GLU) {
 #pragma unroll
       for (int e = 0; e < 4; e += 2)
         if (m + e + 1 < a.M)
-          reinterpret_cast<bf16_t*>(a.out)[(int64_t)n * a.ldo + ((m + e) >> 1)] = (bf16_t)clamped_glu_f(v[e], v[e + 1], a.limit);
+          reinterpret_cast<bf16_t*>(a.out)[(int64_t)n * a.ldo + ((m + e) >> 1)] = (bf16_t)glu_f(v[e], v[e + 1], a.act, a.limit);
     } else {
 #pragma unroll
       for (int e = 0; e < 4; ++e) {

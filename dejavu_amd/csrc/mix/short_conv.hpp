@@ -54,6 +54,9 @@ __global__ __launch_bounds__(256) void short_conv_kernel(ConvArgs a) {
 #pragma unroll
       for (int j = 0; j < TAPS; ++j) w[j][e] = wv[(e * TAPS + j) >> 2][(e * TAPS + j) & 3];
   }
+  float bias[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) bias[e] = a.b ? a.b[ch + e] : 0.f;
   const int t0 = blockIdx.y * kConvTokens, t1 = min(a.n, t0 + kConvTokens);
   Pack8<T> next[kConvTokens];
 #pragma unroll
@@ -79,7 +82,7 @@ __global__ __launch_bounds__(256) void short_conv_kernel(ConvArgs a) {
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
       u[TAPS - 1][e] = next[i].get(e);
-      float v = 0.f;
+      float v = bias[e];
 #pragma unroll
       for (int j = 0; j < TAPS; ++j) v = __builtin_fmaf(w[j][e], u[j][e], v);
       y[e] = a.silu ? silu_f(v) : v;
@@ -126,7 +129,7 @@ __global__ __launch_bounds__(256) void short_conv_any_kernel(ConvArgs a) {
   base += h * g.stride;
   auto value = [&](int c) {
     const int ch = base + c;
-    float y = 0.f;
+    float y = a.b ? a.b[ch] : 0.f;
     for (int j = 0; j < a.taps; ++j) {
       const int s = t - (a.taps - 1) + j;
       const float u = s >= 0 ? to_f(in[s * a.ldi + ch]) : a.state[(int64_t)ch * (a.taps - 1) + a.taps - 1 + s];

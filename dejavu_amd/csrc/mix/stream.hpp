@@ -75,16 +75,20 @@ __device__ __forceinline__ float clamped_glu_f(float g, float u, float limit) {
   return g * sigmoid_f(1.702f * g) * (u + 1.f);
 }
 
+__device__ __forceinline__ float glu_f(float g, float u, int act, float limit) {
+  return act == DV_GLU_RELU ? fmaxf(g, 0.f) * u : clamped_glu_f(g, u, limit);
+}
+
 // y[i] from gu[2 i] (gate) and gu[2 i + 1] (up); four outputs per thread, count % 4 == 0.
-template <typename T>
-__global__ __launch_bounds__(256) void clamped_glu_kernel(const T* __restrict__ gu, int64_t count, float limit,
-                                                          T* __restrict__ y) {
+template <typename T, int ACT>
+__global__ __launch_bounds__(256) void glu_kernel(const T* __restrict__ gu, int64_t count, float limit,
+                                                  T* __restrict__ y) {
   const int64_t i = ((int64_t)blockIdx.x * 256 + threadIdx.x) * 4;
   if (i >= count) return;
   Pack8<T> v;
   v.load(gu + 2 * i);
 #pragma unroll
-  for (int e = 0; e < 4; ++e) y[i + e] = from_f<T>(clamped_glu_f(v.get(2 * e), v.get(2 * e + 1), limit));
+  for (int e = 0; e < 4; ++e) y[i + e] = from_f<T>(glu_f(v.get(2 * e), v.get(2 * e + 1), ACT, limit));
 }
 
 // y = x / sqrt(mean(x^2) + eps) * w, the mean over the first `dim` entries (those up to `padded`, a multiple of 8, are

@@ -9,9 +9,11 @@
 #include "mix/attn_rows.hpp"
 #include "mix/attn_tiles.hpp"
 #include "mix/delta_rule.hpp"
+#include "mix/hyper.hpp"
 #include "mix/linear_rows.hpp"
 #include "mix/linear_tiles.hpp"
 #include "mix/short_conv.hpp"
+#include "mix/ssd.hpp"
 #include "mix/stream.hpp"
 
 using namespace dv;
@@ -67,9 +69,18 @@ int linear_row_any(int before, int after, const RowsArgs& a, hipStream_t s) {
       case DV_OUT_GLU: return linear_row<T, DV_ROW_PLAIN, DV_OUT_GLU>(a, s);
       case DV_OUT_RESIDUAL: return linear_row<T, DV_ROW_PLAIN, DV_OUT_RESIDUAL>(a, s);
       case DV_OUT_CONV: return linear_row<T, DV_ROW_PLAIN, DV_OUT_CONV>(a, s);
+      case DV_OUT_HYPER: return linear_row<T, DV_ROW_PLAIN, DV_OUT_HYPER>(a, s);
     }
-  } else if (before == DV_ROW_RMS && after == DV_OUT_F32) {
-    return linear_row<T, DV_ROW_RMS, DV_OUT_F32>(a, s);
+  } else if (before == DV_ROW_RMS) {
+    switch (after) {
+      case DV_OUT_F32: return linear_row<T, DV_ROW_RMS, DV_OUT_F32>(a, s);
+      case DV_OUT_GLU: return linear_row<T, DV_ROW_RMS, DV_OUT_GLU>(a, s);
+      case DV_OUT_CONV: return linear_row<T, DV_ROW_RMS, DV_OUT_CONV>(a, s);
+    }
+  } else if (before == DV_ROW_GROUPS && after == DV_OUT_HYPER) {
+    return linear_row<T, DV_ROW_GROUPS, DV_OUT_HYPER>(a, s);
+  } else if (before == DV_ROW_GROUPS && after == DV_OUT_T) {
+    return linear_row<T, DV_ROW_GROUPS, DV_OUT_T>(a, s);
   } else if (before == DV_ROW_HEADS && after == DV_OUT_RESIDUAL) {
     return linear_row<T, DV_ROW_HEADS, DV_OUT_RESIDUAL>(a, s);
   }
@@ -94,6 +105,7 @@ int short_conv_types(const ConvArgs& a, int heads, int widest, hipStream_t s) {
     hipLaunchKernelGGL((short_conv_any_kernel<T, TO>), dim3(blocks_of((int64_t)a.n * heads, 4)), dim3(256), 0, s, a);
     return launched();
   }
+  if (widest <= 8) return short_conv_lanes<T, TO, 1>(a, heads, s);
   if (widest <= 64) return short_conv_lanes<T, TO, 8>(a, heads, s);
   if (widest <= 128) return short_conv_lanes<T, TO, 16>(a, heads, s);
   if (widest <= 256) return short_conv_lanes<T, TO, 32>(a, heads, s);
@@ -162,13 +174,64 @@ int latent_tiles(const AttnArgs& a, hipStream_t s) {
 int attn_args_ok(const AttnArgs* a) {
   if (!a || !a->q || !a->k || !a->v || a->n < 1 || a->H < 1 || a->G < 1 || a->H % a->G || a->dim_s < 8 ||
       a->vdim_s < 8 || a->splits < 1 || a->splits > kMaxSplits || (a->splits > 1 && !a->part) || (a->splits == 1 && !a->out) ||
-      (!a->fresh_k != !a->fresh_v))
+      (!a->fresh_k != !a->fresh_v) || a->window < 0 || a->chunk < 0 || (a->window > 0 && a->chunk > 0) ||
+      (a->rel && a->rel_len < 1) || (a->other_v && (!a->lambda || !a->fresh_v)) || ((a->q_w || a->k_w) && a->norm_dim < 1))
     return DV_ERR_INVALID_ARG;
   if (a->dim_s % 8 || a->vdim_s % 8 || a->ldk % 8 || a->ldv % 8 || a->k_head % 8 || a->v_head % 8 || !al16(a->k) ||
       !al16(a->v) || !al16(a->q))
     return DV_ERR_ALIGNMENT;
   if (a->vdim_s > 2048 || a->n > 65535 || (int64_t)a->H > 65535) return DV_ERR_UNSUPPORTED;
   return DV_OK;
+}
+
+// ---- residual streams ------------------------------------------------------------
+int hyper_ok(const dvHyper* r, const dvRmsOut* norm) {
+  if (!r || !r->x || r->streams < 1 || r->streams > DV_HYPER_MAX || r->width < 4 || !norm || (!r->u && !norm->h) ||
+      (norm->h && (!norm->w || norm->dim < 1 || norm->dim > r->width)))
+    return DV_ERR_INVALID_ARG;
+  if (r->width % 8 || !al16(r->x) || !al16(r->u) || !al16(norm->h) || !al16(norm->w)) return DV_ERR_ALIGNMENT;
+  return DV_OK;
+}
+template <typename T, int SM, bool EMBED>
+int hyper_rows(const void* y, int n, const dvHyper& r, const dvEmbedArgs& e, const dvRmsOut& norm, hipStream_t s) {
+  const dim3 grid(n, norm.h ? 1 : (r.width + 1023) / 1024);
+  const size_t lds = norm.h ? (size_t)r.width * 4 : 0;
+  return launch_lds<hyper_rows_kernel<T, SM, EMBED>>(grid, dim3(256), lds, s, (const T*)y, r, e, norm);
+}
+
+// ---- Mamba-2 -----------------------------------------------------------------------
+constexpr int kSsdSegment = 4096;  // tokens whose chunk blocks are in memory at a time
+template <typename T, int NT>
+int ssd_scan(const SsdArgs& a, hipStream_t s) {
+  const size_t need = (size_t)((a.n < kSsdSegment ? a.n : kSsdSegment) + kSsdChunk - 1) / kSsdChunk * a.heads * SsdChunk::floats;
+  if ((size_t)a.tm_floats < need) return DV_ERR_WORKSPACE;
+  const int rep = a.heads / a.groups;
+  for (int t0 = 0; t0 < a.n; t0 += kSsdSegment) {
+    SsdArgs b = a;
+    b.xbc += (int64_t)t0 * a.ld;
+    b.dt = reinterpret_cast<const T*>(a.dt) + (int64_t)t0 * a.lddt;
+    b.y += (int64_t)t0 * a.ldy;
+    b.n = a.n - t0 < kSsdSegment ? a.n - t0 : kSsdSegment;
+    const int chunks = (b.n + kSsdChunk - 1) / kSsdChunk;
+    int hp = 1;  // heads per workgroup: as many as leave four workgroups per compute unit
+    while (hp < rep && (int64_t)a.heads * chunks / (2 * hp) >= 1024) hp *= 2;
+    if (hp > rep) hp = rep;
+    hipLaunchKernelGGL((ssd_chunk_kernel<T>), dim3((unsigned)(a.groups * ((rep + hp - 1) / hp)), chunks), dim3(256), 0, s, b, hp);
+    int rc = launched();
+    if (rc != DV_OK) return rc;
+    hipLaunchKernelGGL((ssd_scan_kernel<NT>), dim3((unsigned)(a.heads * ((a.vdim + kSsdCols - 1) / kSsdCols))), dim3(256), 0, s, b);
+    rc = launched();
+    if (rc != DV_OK) return rc;
+  }
+  return DV_OK;
+}
+template <typename T>
+int ssd_scan_any(const SsdArgs& a, hipStream_t s) {
+  if (a.state_s <= 64) return ssd_scan<T, 1>(a, s);
+  if (a.state_s <= 128) return ssd_scan<T, 2>(a, s);
+  if (a.state_s <= 192) return ssd_scan<T, 3>(a, s);
+  if (a.state_s <= 256) return ssd_scan<T, 4>(a, s);
+  return DV_ERR_UNSUPPORTED;
 }
 
 template <int DT, int VT>
@@ -212,14 +275,86 @@ int dv_mix_residual(int dtype, const void* y, int64_t n, int width, const dvResi
   return launched();
 }
 
-int dv_mix_clamped_glu(int dtype, const void* gu, int64_t count, float limit, void* y, void* stream) {
-  if (!dtype_ok(dtype) || !gu || !y || count < 4) return DV_ERR_INVALID_ARG;
+int dv_mix_glu(int dtype, const void* gu, int64_t count, int act, float limit, void* y, void* stream) {
+  if (!dtype_ok(dtype) || !gu || !y || count < 4 || (act != DV_GLU_CLAMPED && act != DV_GLU_RELU)) return DV_ERR_INVALID_ARG;
   if (count % 4 || !al16(gu)) return DV_ERR_ALIGNMENT;
   const dim3 grid(blocks_of(count, 1024));
+#define DV_GLU(T)                                                                                                          \
+  do {                                                                                                                     \
+    if (act == DV_GLU_RELU)                                                                                                \
+      hipLaunchKernelGGL((glu_kernel<T, DV_GLU_RELU>), grid, dim3(256), 0, st(stream), (const T*)gu, count, limit, (T*)y);    \
+    else                                                                                                                   \
+      hipLaunchKernelGGL((glu_kernel<T, DV_GLU_CLAMPED>), grid, dim3(256), 0, st(stream), (const T*)gu, count, limit, (T*)y); \
+  } while (0)
+  if (dtype == DV_BF16) DV_GLU(bf16_t);
+  else DV_GLU(float);
+#undef DV_GLU
+  return launched();
+}
+
+int dv_mix_hyper_embed(int dtype, const dvEmbedArgs* e, const dvHyper* r, const dvRmsOut* norm, void* stream) {
+  if (!dtype_ok(dtype) || !e || !e->tokens || !e->history || !e->embed || e->n < 1 || e->vocab < 1 || e->capacity < 1 ||
+      (e->bigram && e->buckets < 1) || (!e->pos_dev && (e->pos_host < 0 || e->pos_host + (int64_t)e->n > e->capacity)))
+    return DV_ERR_INVALID_ARG;
+  int rc = hyper_ok(r, norm);
+  if (rc != DV_OK) return rc;
+  if (!r->in) return DV_ERR_INVALID_ARG;
+  if (!al16(e->embed) || !al16(e->bigram)) return DV_ERR_ALIGNMENT;
+  return dtype == DV_BF16 ? hyper_rows<bf16_t, 16, true>(nullptr, e->n, *r, *e, *norm, st(stream))
+                          : hyper_rows<float, 16, true>(nullptr, e->n, *r, *e, *norm, st(stream));
+}
+
+int dv_mix_hyper_rows(int dtype, const void* y, int n, const dvHyper* r, const dvRmsOut* norm, void* stream) {
+  if (!dtype_ok(dtype) || n < 1) return DV_ERR_INVALID_ARG;
+  int rc = hyper_ok(r, norm);
+  if (rc != DV_OK) return rc;
+  if (!r->in || (y && (!r->mix || !r->out))) return DV_ERR_INVALID_ARG;
+  if (!al16(y)) return DV_ERR_ALIGNMENT;
+  const dvEmbedArgs none = {};
   if (dtype == DV_BF16)
-    hipLaunchKernelGGL((clamped_glu_kernel<bf16_t>), grid, dim3(256), 0, st(stream), (const bf16_t*)gu, count, limit, (bf16_t*)y);
-  else
-    hipLaunchKernelGGL((clamped_glu_kernel<float>), grid, dim3(256), 0, st(stream), (const float*)gu, count, limit, (float*)y);
+    return r->streams <= 4 ? hyper_rows<bf16_t, 4, false>(y, n, *r, none, *norm, st(stream))
+                           : hyper_rows<bf16_t, 16, false>(y, n, *r, none, *norm, st(stream));
+  return r->streams <= 4 ? hyper_rows<float, 4, false>(y, n, *r, none, *norm, st(stream))
+                         : hyper_rows<float, 16, false>(y, n, *r, none, *norm, st(stream));
+}
+
+int dv_mix_head_rows(int dtype, const dvHeadArgs* a, void* stream) {
+  if (!dtype_ok(dtype) || !a || !a->in || a->n < 1) return DV_ERR_INVALID_ARG;
+  if (a->ldi % 8 || !al16(a->in)) return DV_ERR_ALIGNMENT;
+  int heads = 0;
+  for (const dvHeadGroup& g : a->g) {
+    if (g.heads < 0) return DV_ERR_INVALID_ARG;
+    if (g.heads == 0) continue;
+    if (!g.out || g.stride < 8 || g.dim < 1 || g.dim > g.stride || (g.other && (g.w || !g.lambda))) return DV_ERR_INVALID_ARG;
+    if (g.stride % 8 || g.ld % 8 || !al16(g.out) || (g.other && (g.ldo % 8 || !al16(g.other)))) return DV_ERR_ALIGNMENT;
+    heads += g.heads;
+  }
+  if (heads == 0) return DV_ERR_INVALID_ARG;
+  const dim3 grid(blocks_of((int64_t)a->n * heads, 16));
+  if (dtype == DV_BF16) hipLaunchKernelGGL((head_rows_kernel<bf16_t>), grid, dim3(256), 0, st(stream), *a);
+  else hipLaunchKernelGGL((head_rows_kernel<float>), grid, dim3(256), 0, st(stream), *a);
+  return launched();
+}
+
+int dv_mix_gated_group_norm(int dtype, const float* y, int64_t ldy, const void* z, int64_t ldz, int64_t rows, int dim,
+                            int groups, int padded, const float* w, float eps, void* out, void* stream) {
+  if (!dtype_ok(dtype) || !y || !z || !w || !out || rows < 1 || dim < 1 || groups < 1 || dim % groups || padded < dim)
+    return DV_ERR_INVALID_ARG;
+  if (padded % 8 || ldy % 4 || ldz % 8 || !al16(y) || !al16(z) || !al16(w) || !al16(out)) return DV_ERR_ALIGNMENT;
+  const int gs = dim / groups;
+#define DV_GROUP(T, W, VEC)                                                                                          \
+  hipLaunchKernelGGL((gated_group_norm_kernel<T, W, VEC>), dim3(blocks_of(rows * groups, 4 / W)), dim3(256), 0, st(stream), \
+                     y, ldy, (const T*)z, ldz, rows, dim, gs, padded, w, eps, (T*)out)
+#define DV_GROUPS(T)                                  \
+  do {                                                \
+    if (gs % 4) DV_GROUP(T, 1, false);                \
+    else if (gs <= 1024) DV_GROUP(T, 1, true);        \
+    else DV_GROUP(T, 4, true);                        \
+  } while (0)
+  if (dtype == DV_BF16) DV_GROUPS(bf16_t);
+  else DV_GROUPS(float);
+#undef DV_GROUPS
+#undef DV_GROUP
   return launched();
 }
 
@@ -251,7 +386,7 @@ int dv_mix_gated_head_norm(int dtype, const float* o, const void* gate, int64_t 
 int dv_mix_linear_row(int dtype, int before, int after, const dvRowArgs* a, void* stream) {
   if (!dtype_ok(dtype) || !a || !a->x || !a->W || a->M < 1 || a->K < 8) return DV_ERR_INVALID_ARG;
   if (a->K % 8 || a->ldw % 8 || !al16(a->W) || !al16(a->x)) return DV_ERR_ALIGNMENT;
-  if (after != DV_OUT_RESIDUAL && !a->out) return DV_ERR_INVALID_ARG;
+  if (after != DV_OUT_RESIDUAL && after != DV_OUT_HYPER && !a->out) return DV_ERR_INVALID_ARG;
   if (after == DV_OUT_GLU && a->M % 2) return DV_ERR_INVALID_ARG;
   if (after == DV_OUT_RESIDUAL && (!a->res.x || !a->res.post.w || (a->res.h && !a->res.pre.w))) return DV_ERR_INVALID_ARG;
   if (after == DV_OUT_CONV && (!a->conv_w || a->taps < 1 || (a->taps > 1 && !a->conv_state) || a->conv_rows > a->M))
@@ -261,6 +396,13 @@ int dv_mix_linear_row(int dtype, int before, int after, const dvRowArgs* a, void
                                  a->K % a->head_stride ||
                                  a->norm_dim < 1 || a->norm_dim > a->head_stride))
     return DV_ERR_INVALID_ARG;
+  if (before == DV_ROW_GROUPS && (!a->xw || a->x_dim < 1 || a->x_dim > a->K || a->norm_dim < 1 || a->x_dim % a->norm_dim))
+    return DV_ERR_INVALID_ARG;
+  if ((before == DV_ROW_RMS || before == DV_ROW_GROUPS) && !al16(a->xw)) return DV_ERR_ALIGNMENT;
+  if (after == DV_OUT_HYPER && (!a->hyper.x || !a->hyper.mix || !a->hyper.out || (a->hyper.u && !a->hyper.in) ||
+                                a->hyper.streams < 1 || a->hyper.streams > DV_HYPER_ROW_MAX || a->hyper.width != a->M))
+    return DV_ERR_INVALID_ARG;
+  if (after == DV_OUT_GLU && a->bias) return DV_ERR_INVALID_ARG;
   if (a->side_x && (!a->side_w || !a->side_out || a->side_dim < 1)) return DV_ERR_INVALID_ARG;
   return dtype == DV_BF16 ? linear_row_any<bf16_t>(before, after, *a, st(stream))
                           : linear_row_any<float>(before, after, *a, st(stream));
@@ -455,6 +597,29 @@ int dv_mix_delta_step(int dtype, const dvDeltaStepArgs* a, void* stream) {
   if (dtype == DV_BF16) DV_STEP(bf16_t);
   else DV_STEP(float);
 #undef DV_STEP
+  return launched();
+}
+
+int dv_mix_ssd_scan(int dtype, const dvSsdArgs* a, void* stream) {
+  if (!dtype_ok(dtype) || !a || !a->xbc || !a->dt || !a->A_log || !a->dt_bias || !a->D || !a->S || !a->y || !a->tm || a->n < 1 ||
+      a->heads < 1 || a->groups < 1 || a->heads % a->groups || a->vdim < 1 || a->state_s < 8)
+    return DV_ERR_INVALID_ARG;
+  if (a->state_s % 8 || a->ld % 4 || a->off_b % 4 || a->off_c % 4 || !al16(a->xbc) || !al16(a->S) || !al16(a->tm))
+    return DV_ERR_ALIGNMENT;
+  return dtype == DV_BF16 ? ssd_scan_any<bf16_t>(*a, st(stream)) : ssd_scan_any<float>(*a, st(stream));
+}
+
+int dv_mix_ssd_step(const dvSsdStepArgs* a, void* stream) {
+  if (!a || !a->p || !a->A_log || !a->dt_bias || !a->D || !a->S || !a->y || a->heads < 1 || a->groups < 1 ||
+      a->heads % a->groups || a->vdim < 1 || a->state_s < 8)
+    return DV_ERR_INVALID_ARG;
+  if (a->state_s % 8 || a->off_b % 4 || a->off_c % 4 || !al16(a->p) || !al16(a->S)) return DV_ERR_ALIGNMENT;
+  const dim3 grid((unsigned)(a->heads * ((a->vdim + kSsdCols - 1) / kSsdCols)));
+  if (a->state_s <= 64) hipLaunchKernelGGL((ssd_step_kernel<1>), grid, dim3(256), 0, st(stream), *a);
+  else if (a->state_s <= 128) hipLaunchKernelGGL((ssd_step_kernel<2>), grid, dim3(256), 0, st(stream), *a);
+  else if (a->state_s <= 192) hipLaunchKernelGGL((ssd_step_kernel<3>), grid, dim3(256), 0, st(stream), *a);
+  else if (a->state_s <= 256) hipLaunchKernelGGL((ssd_step_kernel<4>), grid, dim3(256), 0, st(stream), *a);
+  else return DV_ERR_UNSUPPORTED;
   return launched();
 }
 

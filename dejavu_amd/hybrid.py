@@ -1,11 +1,14 @@
-"""Decoders whose layers differ in how they mix tokens (latent attention, gated delta rule, windowed attention).
+"""Decoders whose layers differ in how they mix tokens (attention of several kinds, recurrences).
 
-``Vimulorn`` is the family that is registered: sandwich dynamic-tanh norms (before and after every sublayer), a
-clamped gated feed-forward, and optionally a stretch of layers that runs several times with the same weights, where
-every pass but the first adds the embedding output again and every pass keeps its own cache or state.
+Two families are registered.  ``Vimulorn``: one residual stream between sandwich dynamic-tanh norms (before and after
+every sublayer), a clamped gated feed-forward, and optionally a stretch of layers that runs several times with the same
+weights, where every pass but the first adds the embedding output again and every pass keeps its own cache or state.
+``Varolorn``: several residual streams that every sublayer reads as a weighted sum and joins through a matrix, RMS norms
+before the sublayers, a relu-gated feed-forward, an embedding of every token with its predecessor, and a head that is
+the embedding table.
 
-A layer is: h -> mixer -> output projection (with norm, residual add and the next norm behind it) -> feed-forward ->
-down projection (likewise).  No norm has a launch of its own.
+A layer is: h -> mixer -> output projection (with what the residual does and the next norm behind it) -> feed-forward ->
+down projection (likewise).  At decode no norm has a launch of its own.
 """
 from __future__ import annotations
 
@@ -19,7 +22,8 @@ from . import mixer_ops as ops
 from .generation import CausalLMOutput, GreedyDecoding
 from .inference import InferenceParams
 from .mixer_ops import padded
-from .mixers import ChannelDelta, ClampedGLU, DynamicTanh, LatentAttention, StepInfo, WindowAttention
+from .mixers import (ChannelDelta, ChunkAttention, ClampedGLU, DynamicTanh, HyperConnection, LatentAttention, Mamba2,
+                     ReluGLU, RMSNorm, StepInfo, WindowAttention)
 
 
 @dataclass
@@ -32,12 +36,24 @@ class LayerSpec:
 
 
 @dataclass
+class EmbeddingSpec:
+    """embed[token] scale + bigram[(previous mul_prev + token mul_cur) mod buckets]; buckets 0: no second table."""
+
+    scale: float = 1.0
+    buckets: int = 0
+    mul_prev: int = 0
+    mul_cur: int = 0
+
+
+@dataclass
 class HybridConfig:
     width: int
     vocab: int
     layers: List[LayerSpec]
     norm_eps: float = 1e-5
     loop: Optional[Tuple[int, int, int]] = None  # layers start .. stop - 1 run `times` times
+    streams: Optional[int] = None                # None: one stream and sandwich norms; else that many, pre-norm
+    embedding: Optional[EmbeddingSpec] = None    # of models with streams; their head is the embedding table
 
     @classmethod
     def from_dict(cls, config: dict, shapes: Optional[Dict[str, tuple]] = None) -> "HybridConfig":
@@ -76,6 +92,51 @@ class HybridConfig:
                    vocab=config.get("vocab", shapes.get("embed", (0, 0))[0]), layers=layers,
                    norm_eps=float(config["norm"]["eps"]), loop=loop or None)
 
+    @classmethod
+    def from_dict_streams(cls, config: dict, shapes: Optional[Dict[str, tuple]] = None) -> "HybridConfig":
+        """The same for models with several residual streams (Varolorn)."""
+        shapes = shapes or {}
+
+        def size(name, axis=0):
+            return shapes[name][axis] if name in shapes else None
+
+        layers, values = [], "first"
+        for i, entry in enumerate(config["layers"]):
+            kind, mix, mlp, pre = entry["type"], dict(entry["mixer"]), entry.get("mlp"), f"l{i}.mix."
+            if kind == "attention":
+                kind = "chunk_attention"
+                mix.setdefault("heads", size(pre + "g"))
+                mix.setdefault("dim", size(pre + "q.norm"))
+                if pre + "k" in shapes:
+                    mix.setdefault("kv_heads", size(pre + "k") // mix["dim"])
+                    mix.setdefault("vdim", size(pre + "v") // mix["kv_heads"])
+                    mix["bias_rows"] = size(pre + "rel")
+                mix["chunk"] = (mix.get("mask") or {}).get("size")
+                mix["values"] = None
+                if mix.get("v_mix"):  # the first layer that says so is the source of the others
+                    mix["values"], values = values, "mixed"
+            elif kind == "mamba2":
+                mix.setdefault("heads", size(pre + "A_log"))
+                mix.setdefault("conv", size(pre + "conv", 1))
+                if pre + "o" in shapes:
+                    mix.setdefault("vdim", size(pre + "o", 1) // mix["heads"])
+            else:
+                raise ValueError(f"layer {i}: unknown mixer {kind!r}")
+            if mlp is not None:
+                if mlp.get("kind", "dense") != "dense":
+                    raise ValueError(f"layer {i}: unknown feed-forward {mlp['kind']!r}")
+                mlp = dict(mlp)
+                mlp.setdefault("ff", size(f"l{i}.mlp.gate"))
+            layers.append(LayerSpec(kind, mix, mlp))
+        emb = config.get("embedding") or {}
+        big = emb.get("bigram")
+        spec = EmbeddingSpec(scale=float(emb.get("scale", 1.0)))
+        if big:
+            buckets = big.get("buckets", (size("bigram") or 1) - 1)
+            spec = EmbeddingSpec(spec.scale, int(buckets), int(big["mul_prev"]), int(big["mul_cur"]))
+        return cls(width=config.get("width", size("embed", 1)), vocab=config.get("vocab", size("embed")), layers=layers,
+                   norm_eps=float(config["norm"]["eps"]), streams=int(config.get("streams", 1)), embedding=spec)
+
     def runs(self) -> List[Tuple[int, bool]]:
         """(layer, does it start a repeated pass) in the order of execution."""
         order = list(range(len(self.layers)))
@@ -99,10 +160,17 @@ def create_mixer(spec: LayerSpec, width: int, eps: float, dtype=None, device=Non
     if spec.type == "attention":
         return WindowAttention(width, m["heads"], m["kv_heads"], m["dim"], m["vdim"], m["conv"], m["mask"]["size"],
                                m["scale"], **kw)
+    if spec.type == "chunk_attention":
+        return ChunkAttention(width, m["heads"], m["kv_heads"], m["dim"], m["vdim"], m["chunk"], m["scale"],
+                              m["bias_rows"], m["bias_max"], m["values"], **kw)
+    if spec.type == "mamba2":
+        return Mamba2(width, m["heads"], m["groups"], m["vdim"], m["state"], m["conv"], m["norm_groups"], **kw)
     raise ValueError(f"unknown mixer {spec.type!r}")
 
 
 class HybridBlock(nn.Module):
+    """One residual stream, a norm before and after every sublayer."""
+
     def __init__(self, spec: LayerSpec, width: int, eps: float, dtype=None, device=None):
         super().__init__()
         self.norm1 = DynamicTanh(width, device=device)
@@ -113,6 +181,11 @@ class HybridBlock(nn.Module):
             self.norm2 = DynamicTanh(width, device=device)
             self.mlp = ClampedGLU(width, spec.mlp["ff"], spec.mlp["limit"], dtype=dtype, device=device)
             self.norm2b = DynamicTanh(width, device=device)
+
+    @property
+    def entry(self):
+        """What makes the layer's input of the residual."""
+        return self.norm1
 
     def forward(self, h, stream: ops.ResidualStream, state: dict, step: StepInfo, pre, add_start: bool = False):
         """h: norm1 of the stream.  Adds both sublayers to the stream (then, with ``add_start``, the stream's start
@@ -129,6 +202,32 @@ class HybridBlock(nn.Module):
         return ops.linear_residual(self.mlp(h), self.mlp.out_weight, stream, self.norm2b, pre, add_start)
 
 
+class StreamsBlock(nn.Module):
+    """Several residual streams, a norm before every sublayer."""
+
+    def __init__(self, spec: LayerSpec, width: int, eps: float, streams: int, dtype=None, device=None):
+        super().__init__()
+        self.norm1, self.hyper1 = RMSNorm(width, eps, device=device), HyperConnection(streams, device=device)
+        self.mixer = create_mixer(spec, width, eps, dtype=dtype, device=device)
+        self.mlp = None
+        if spec.mlp is not None:
+            self.norm2, self.hyper2 = RMSNorm(width, eps, device=device), HyperConnection(streams, device=device)
+            self.mlp = ReluGLU(width, spec.mlp["ff"], dtype=dtype, device=device)
+
+    @property
+    def entry(self):
+        return ops.StreamRead(self.norm1, self.hyper1.weights)
+
+    def forward(self, h, stream: ops.HyperStream, state: dict, step: StepInfo, following, add_start: bool = False):
+        """h: this layer's ``entry`` of the streams.  Both sublayers join the streams; returns ``following`` of them."""
+        assert not add_start
+        middle = following if self.mlp is None else ops.StreamRead(self.norm2, self.hyper2.weights)
+        h = stream.update(self.mixer(h, state, step), self.mixer.out_weight, self.mixer.out_bias, self.hyper1, middle)
+        if self.mlp is None:
+            return h
+        return stream.update(self.mlp(h), self.mlp.out_weight, None, self.hyper2, following)
+
+
 class HybridLMHeadModel(GreedyDecoding, nn.Module):
     decode_period = 8  # steps per captured graph
 
@@ -137,11 +236,24 @@ class HybridLMHeadModel(GreedyDecoding, nn.Module):
         assert dtype in (torch.bfloat16, torch.float32), "weights and activations in bf16 or fp32"
         self.config = config
         width = padded(config.width)
-        self.embeddings = nn.Parameter(torch.zeros(config.vocab, width, dtype=dtype, device=device), requires_grad=False)
-        self.layers = nn.ModuleList([HybridBlock(s, config.width, config.norm_eps, dtype=dtype, device=device)
-                                     for s in config.layers])
-        self.final_norm = DynamicTanh(config.width, device=device)
-        self.lm_head = nn.Parameter(torch.zeros(config.vocab, width, dtype=dtype, device=device), requires_grad=False)
+
+        def table(rows):
+            return nn.Parameter(torch.zeros(rows, width, dtype=dtype, device=device), requires_grad=False)
+
+        kw = dict(dtype=dtype, device=device)
+        self.embeddings = table(config.vocab)
+        if config.streams is None:
+            self.layers = nn.ModuleList([HybridBlock(s, config.width, config.norm_eps, **kw) for s in config.layers])
+            self.final_norm = DynamicTanh(config.width, device=device)
+            self.lm_head = table(config.vocab)
+        else:
+            assert config.loop is None, "one stream only"
+            self.bigram = table(config.embedding.buckets + 1) if config.embedding.buckets else None
+            self.layers = nn.ModuleList([StreamsBlock(s, config.width, config.norm_eps, config.streams, **kw)
+                                         for s in config.layers])
+            self.final_norm = RMSNorm(config.width, config.norm_eps, device=device)
+            self.register_buffer("_ones", torch.ones(config.streams, device=device), persistent=False)
+            self.lm_head = self.embeddings
         self.runs = config.runs()
         self.keeps_start = any(again for _, again in self.runs)
         # when a list, every forward appends the residual stream after every layer run
@@ -154,6 +266,26 @@ class HybridLMHeadModel(GreedyDecoding, nn.Module):
             if key not in memory:
                 memory[key] = self.layers[i].mixer.new_state(inference_params.max_sequence_len)
         return [memory[key] for key in range(len(self.runs))]
+
+    def _history(self, inference_params: InferenceParams) -> torch.Tensor:
+        """The sequence's tokens by position (an embedding reads the one before a portion)."""
+        state = inference_params.key_value_memory_dict.setdefault("embedding", {})
+        if "tokens" not in state:
+            state["tokens"] = torch.zeros(inference_params.max_sequence_len, dtype=torch.long,
+                                          device=self.embeddings.device)
+        return state["tokens"]
+
+    def _exit(self):
+        """What makes the head's input of the residual."""
+        return self.final_norm if self.config.streams is None else ops.StreamRead(self.final_norm, self._ones)
+
+    def _embed(self, tokens, ip: InferenceParams, step: StepInfo):
+        first = self.layers[self.runs[0][0]].entry
+        if self.config.streams is None:
+            return ops.embed(tokens, self.embeddings, first, self.keeps_start)
+        e = self.config.embedding
+        return ops.hyper_embed(tokens, self.embeddings, e.scale, self.bigram, e.mul_prev, e.mul_cur, self._history(ip),
+                               step.pos_dev, step.pos, self.config.streams, first)
 
     @torch.no_grad()
     def forward(self, input_ids, position_ids=None, inference_params=None, last_token_only=False, rows=None):
@@ -170,20 +302,22 @@ class HybridLMHeadModel(GreedyDecoding, nn.Module):
         assert pos + n <= ip.max_sequence_len, "the sequence does not fit its memory"
         step = StepInfo(pos, ip.lengths_per_sample if n == 1 else None)
         states = self._states(ip)
-        stream, h = ops.embed(input_ids.reshape(-1), self.embeddings, self.layers[self.runs[0][0]].norm1,
-                              self.keeps_start)
+        stream, h = self._embed(input_ids.reshape(-1), ip, step)
         for key, (i, _) in enumerate(self.runs):
             if key + 1 < len(self.runs):
                 following, again = self.runs[key + 1]
-                pre = self.layers[following].norm1
+                pre = self.layers[following].entry
             else:
-                pre, again = self.final_norm, False
+                pre, again = self._exit(), False
             if self.record is None:
                 h = self.layers[i](h, stream, states[key], step, pre, again)
-            else:
+            elif self.config.streams is None:
                 self.layers[i](h, stream, states[key], step, None)
                 self.record.append(stream.x[:, :self.config.width].clone())
                 h = ops.residual(None, stream, None, pre, again)
+            else:
+                h = self.layers[i](h, stream, states[key], step, pre)
+                self.record.append(stream.total()[:, :self.config.width])
         if rows is not None:
             if len(rows) == 0:
                 return CausalLMOutput(logits=None)

@@ -1,4 +1,4 @@
-"""Checkpoint formats: HuggingFace OPT weights, trained sparsity predictors, Vimulorn weights.
+"""Checkpoint formats: HuggingFace OPT weights, trained sparsity predictors, Vimulorn and Varolorn weights.
 
 Mirrors what the reference does before ``model.load_state_dict``
 (Dejavu/src/utils/dejavu_util.py:12-234 ``remap_state_dict_opt`` / ``shard_state_dict_tp``,
@@ -154,12 +154,21 @@ def load_checkpoint_folder(folder: str) -> dict:
     return load_checkpoint_file(os.path.join(folder, "pytorch_model.bin"))
 
 
-# ---- Vimulorn ---------------------------------------------------------------------
+# ---- Vimulorn, Varolorn -------------------------------------------------------------
 def _pad(x: torch.Tensor, *sizes: int) -> torch.Tensor:
     """Zero padding at the end of the leading dimensions up to ``sizes``."""
     out = x.new_zeros(*sizes, *x.shape[len(sizes):])
     out[tuple(slice(0, n) for n in x.shape[:len(sizes)])] = x
     return out
+
+
+def _pad_cols(x: torch.Tensor, size: int) -> torch.Tensor:
+    return _pad(x.t(), size).t()
+
+
+def _head_rows(x: torch.Tensor, heads: int, dim: int, stride: int) -> torch.Tensor:
+    """(heads * dim, ...) -> rows padded to ``stride`` per head."""
+    return _pad(x.reshape(heads, dim, *x.shape[1:]), heads, stride).reshape(heads * stride, *x.shape[1:])
 
 
 def remap_state_dict_vimulorn(state_dict: Mapping[str, torch.Tensor], config) -> "OrderedDict[str, torch.Tensor]":
@@ -177,10 +186,10 @@ def remap_state_dict_vimulorn(state_dict: Mapping[str, torch.Tensor], config) ->
     ws = padded(width)
 
     def cols(x):  # an input of the model's width
-        return _pad(x.t(), ws).t()
+        return _pad_cols(x, ws)
 
-    def head_rows(x, heads, dim):  # (heads * dim, ...) -> rows padded per head
-        return _pad(x.reshape(heads, dim, *x.shape[1:]), heads, padded(dim)).reshape(heads * padded(dim), *x.shape[1:])
+    def head_rows(x, heads, dim):
+        return _head_rows(x, heads, dim, padded(dim))
 
     def head_cols(x, heads, dim):
         return head_rows(x.t(), heads, dim).t()
@@ -239,6 +248,91 @@ def remap_state_dict_vimulorn(state_dict: Mapping[str, torch.Tensor], config) ->
             gate, up = (_pad(cols(t.pop(f"{src}mlp.{n}")), fs) for n in ("gate", "up"))
             out[dst + "mlp.gate_up"] = torch.stack([gate, up], dim=1).reshape(2 * fs, ws)
             out[dst + "mlp.down"] = _pad(_pad(t.pop(f"{src}mlp.down"), ws).t(), fs).t()
+    for name in t:  # what is left has no place in this family: reported by the caller
+        out[name] = t[name]
+    return out
+
+
+def remap_state_dict_varolorn(state_dict: Mapping[str, torch.Tensor], config) -> "OrderedDict[str, torch.Tensor]":
+    """Varolorn checkpoint names -> parameters of ``dejavu_amd.hybrid.HybridLMHeadModel`` with several streams.
+
+    * the projections that read a mixer's input become one matrix (rows in the order the mixer documents), their
+      biases one vector; gate and up rows of the feed-forward alternate
+    * norm weights stored around zero become 1 + w; the table of biases by bucket becomes one by distance
+    * sizes along vectorised dimensions are padded to multiples of 8 with zeros: per head in attention, behind the last
+      head in the recurrence (B and C: per group)
+    """
+    from .mixer_ops import padded
+    from .mixers import bias_distances, distance_buckets
+
+    t = dict(state_dict)
+    out: "OrderedDict[str, torch.Tensor]" = OrderedDict()
+    ws, S = padded(config.width), config.streams
+
+    def cols(x):  # an input of the model's width
+        return _pad_cols(x, ws)
+
+    def norm(src, dst):
+        out[dst + ".weight"] = _pad(1.0 + t.pop(src).float(), ws)
+
+    def hyper(src, dst):
+        for name, to in (("in", "weights"), ("out", "out"), ("mix", "mix")):
+            out[f"{dst}.{to}"] = t.pop(f"{src}.{name}").float()
+
+    out["embeddings"] = cols(t.pop("embed"))
+    out["lm_head"] = out["embeddings"]
+    if config.embedding.buckets:
+        out["bigram"] = cols(t.pop("bigram"))
+    norm("final.norm", "final_norm")
+    for i, spec in enumerate(config.layers):
+        src, dst, m = f"l{i}.", f"layers.{i}.", spec.mixer
+        mix = dst + "mixer."
+
+        def take(name, src=src):
+            return t.pop(src + "mix." + name)
+
+        norm(src + "norm1", dst + "norm1")
+        hyper(src + "hc1", dst + "hyper1")
+        H, vdim = m["heads"], m["vdim"]
+        if spec.type == "chunk_attention":
+            G, dim, ds, vs = m["kv_heads"], m["dim"], padded(m["dim"]), padded(vdim)
+            groups = (("q", H, dim, ds), ("k", G, dim, ds), ("v", G, vdim, vs))
+            gate = _pad(take("g"), padded(H))
+            out[mix + "in_proj"] = cols(torch.cat([_head_rows(take(n), *size) for n, *size in groups] + [gate]))
+            bias = [_head_rows(take(n + ".b"), *size) for n, *size in groups]
+            out[mix + "in_bias"] = torch.cat(bias + [bias[0].new_zeros(padded(H))])
+            out[mix + "q_norm"], out[mix + "k_norm"] = (_pad(take(n + ".norm").float(), ds) for n in "qk")
+            table = take("rel").float()
+            rows = distance_buckets(bias_distances(table.shape[0], m["bias_max"], m["chunk"]), table.shape[0], m["bias_max"])
+            out[mix + "rel"] = table[rows].t().contiguous()
+            # the layer that is the source of the values (and one that mixes none) has no use for it
+            lam = t.pop(src + "mix.vmix", None)
+            out[mix + "vmix"] = (torch.zeros(1) if lam is None else lam).float().reshape(1)
+            out[mix + "out_proj"] = _pad(_head_rows(take("o").t(), H, vdim, vs).t(), ws)
+            out[mix + "out_bias"] = _pad(take("o.b"), ws)
+        else:
+            G, N, inner = m["groups"], m["state"], H * vdim
+            ns, inner_s = padded(N), padded(H * vdim)
+
+            def xbc(x):  # rows of x, B, C
+                x, B, C = x.split([inner, G * N, G * N])
+                return [_pad(x, inner_s), _head_rows(B, G, N, ns), _head_rows(C, G, N, ns)]
+
+            z, conv_in, dt = take("in").split([inner, inner + 2 * G * N, H])
+            out[mix + "in_proj"] = cols(torch.cat(xbc(conv_in) + [_pad(z, inner_s), _pad(dt, padded(H))]))
+            out[mix + "conv"] = torch.cat(xbc(take("conv").float()))
+            out[mix + "conv_bias"] = torch.cat(xbc(take("conv.b").float()))
+            for name in ("A_log", "dt_bias", "D"):
+                out[mix + name] = take(name).float()
+            out[mix + "norm"] = _pad(take("norm").float(), inner_s)
+            out[mix + "out_proj"] = _pad(_pad_cols(take("o"), inner_s), ws)
+        if spec.mlp is not None:
+            norm(src + "norm2", dst + "norm2")
+            hyper(src + "hc2", dst + "hyper2")
+            fs = padded(spec.mlp["ff"])
+            gate, up = (_pad(cols(t.pop(f"{src}mlp.{n}")), fs) for n in ("gate", "up"))
+            out[dst + "mlp.gate_up"] = torch.stack([gate, up], dim=1).reshape(2 * fs, ws)
+            out[dst + "mlp.down"] = _pad_cols(_pad(t.pop(f"{src}mlp.down"), ws), fs)
     for name in t:  # what is left has no place in this family: reported by the caller
         out[name] = t[name]
     return out

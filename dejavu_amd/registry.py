@@ -34,7 +34,7 @@ def _vimulorn_config(config, shapes):
     return HybridConfig.from_dict(config, shapes)
 
 
-def _vimulorn_class():
+def _hybrid_class():
     from .hybrid import HybridLMHeadModel
 
     return HybridLMHeadModel
@@ -44,6 +44,18 @@ def _vimulorn_remap(state_dict, config):
     from .loaders import remap_state_dict_vimulorn
 
     return remap_state_dict_vimulorn(state_dict, config)
+
+
+def _varolorn_config(config, shapes):
+    from .hybrid import HybridConfig
+
+    return HybridConfig.from_dict_streams(config, shapes)
+
+
+def _varolorn_remap(state_dict, config):
+    from .loaders import remap_state_dict_varolorn
+
+    return remap_state_dict_varolorn(state_dict, config)
 
 
 def _opt_config(config, shapes):
@@ -77,8 +89,10 @@ def _opt_remap(state_dict, config):
 
 
 FAMILIES: Dict[str, Family] = {
-    "Vimulorn": Family((build.MIXERS_LIB_NAME,), (torch.bfloat16, torch.float32), _vimulorn_config, _vimulorn_class,
+    "Vimulorn": Family((build.MIXERS_LIB_NAME,), (torch.bfloat16, torch.float32), _vimulorn_config, _hybrid_class,
                        _vimulorn_remap, takes_portions=True),
+    "Varolorn": Family((build.MIXERS_LIB_NAME,), (torch.bfloat16, torch.float32), _varolorn_config, _hybrid_class,
+                       _varolorn_remap, takes_portions=True),
     "OPTForCausalLM": Family((build.LIB_NAME,), (torch.float16,), _opt_config, _opt_class, _opt_remap,
                              takes_portions=False),
 }

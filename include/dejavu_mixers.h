@@ -1,6 +1,7 @@
 /*
  * C ABI of libdejavu_mixers.so: gfx950 kernels for decoders that mix tokens with latent attention, a gated delta
- * rule or sliding-window attention around dynamic-tanh norms (see dejavu_amd/mixers.py for the modules).
+ * rule, a Mamba-2 recurrence, or sliding-window or chunk-local attention, around dynamic-tanh norms and one residual
+ * stream or around RMS norms and several streams (see dejavu_amd/mixers.py for the modules).
  *
  * Conventions
  *  - every pointer is a DEVICE pointer; the structs themselves live on the host and are copied by the call;
@@ -38,15 +39,42 @@ typedef struct {
   dvDynTanh post, pre;
 } dvResidual;
 
+/* Several residual streams x [n][streams][width] around a sublayer with result y:
+ * x_t <- sum_s mix[s][t] x_s + out[t] y, all at once; then u = sum_t in[t] x_t for the next sublayer (in null: none). */
+#define DV_HYPER_MAX 16        /* streams                                                    */
+#define DV_HYPER_ROW_MAX 4     /* streams in the epilogue of dv_mix_linear_row               */
+typedef struct {
+  float* x;
+  const float* mix;        /* [streams][streams], from, to */
+  const float* out;        /* [streams] */
+  const float* in;         /* [streams] */
+  float* u;                /* [n][width] or null */
+  int streams, width;
+} dvHyper;
+
+/* An RMS norm that follows: h = u / rms(u) * w, the mean over dim entries, eps inside the root (h null: none). */
+typedef struct {
+  const float* w;
+  float eps;
+  int dim;
+  void* h;
+} dvRmsOut;
+
+/* Gated units of a feed-forward. */
+#define DV_GLU_CLAMPED 0   /* g = min(gate, limit), u = clamp(up, limit): g sigmoid(1.702 g) (u + 1) */
+#define DV_GLU_RELU 1      /* max(gate, 0) up                                                         */
+
 /* How a row enters dv_mix_linear_row, and what happens to the products. */
 #define DV_ROW_PLAIN 0   /* x: elements of `dtype`                                                        */
 #define DV_ROW_RMS 1     /* x: fp32, divided by its root mean square over norm_dim, times xw              */
 #define DV_ROW_HEADS 2   /* x: fp32 heads of head_stride entries, each RMS-normed, times xw, times gate   */
+#define DV_ROW_GROUPS 3  /* x: fp32, groups of norm_dim entries (x_dim in all) each RMS-normed, times xw  */
 #define DV_OUT_F32 0     /* fp32 store                                                                    */
 #define DV_OUT_T 1       /* store in `dtype`                                                              */
-#define DV_OUT_GLU 2     /* rows 2 i (gate) and 2 i + 1 (up) -> clamped gated unit, in `dtype`             */
+#define DV_OUT_GLU 2     /* rows 2 i (gate) and 2 i + 1 (up) -> gated unit `act`, in `dtype`               */
 #define DV_OUT_RESIDUAL 3 /* dvResidual                                                                   */
 #define DV_OUT_CONV 4    /* fp32; the first conv_rows rows pass a short convolution (and silu)            */
+#define DV_OUT_HYPER 5   /* dvHyper, at most DV_HYPER_ROW_MAX streams                                     */
 
 typedef struct {
   const void* x;
@@ -56,11 +84,15 @@ typedef struct {
   const float* xw;
   const float* gate;       /* [K] factors of DV_ROW_HEADS */
   float eps;
-  int norm_dim, head_stride;
+  int norm_dim, head_stride, x_dim;
+  const void* bias;        /* [M] in `dtype` or null; added to the products (not with DV_OUT_GLU) */
   void* out;
+  int act;
   float limit;
   dvResidual res;
+  dvHyper hyper;
   const float* conv_w;     /* [conv_rows][taps] */
+  const float* conv_b;     /* [conv_rows] or null */
   float* conv_state;       /* [conv_rows][taps - 1], oldest first, moved on by one token */
   int conv_rows, taps, silu;
   /* a second fp32 row that one extra workgroup RMS-norms and stores at row `position` of side_out (null: none) */
@@ -80,8 +112,10 @@ typedef struct {
   const void* W;
   int64_t ldw;
   int n, M, K;
+  const void* bias;        /* [M] or null (not with DV_OUT_GLU) */
   void* out;               /* DV_OUT_F32 / DV_OUT_T: [n][ldo]; DV_OUT_GLU: [n][ldo], M / 2 columns */
   int64_t ldo;
+  int act;
   float limit;
   dvResidual res;          /* DV_OUT_RESIDUAL: x, x0, h are [n][M] */
 } dvTileArgs;
@@ -99,9 +133,28 @@ typedef struct {
   int64_t ldi;
   int n, taps, silu;
   const float* w;          /* [channels][taps] */
+  const float* b;          /* [channels] or null */
   const float* state;      /* [channels][taps - 1] */
   dvConvGroup g[3];
 } dvConvArgs;
+
+/* One group of heads of a projection's rows: RMS-normed per head with a weight, or mixed with other rows. */
+typedef struct {
+  int heads, stride, dim;
+  const float* w;          /* [stride]: x / rms(x) * w, the mean over dim; null: no norm */
+  float eps;
+  const void* other;       /* no norm: (1 - *lambda) x + *lambda other (null: x) */
+  int64_t ldo;
+  const float* lambda;
+  void* out;               /* [n][heads][stride], ld elements between tokens */
+  int64_t ld;
+} dvHeadGroup;
+typedef struct {
+  const void* in;          /* [n][ldi], the groups' channels one after the other */
+  int64_t ldi;
+  int n;
+  dvHeadGroup g[3];
+} dvHeadArgs;
 
 /* Softmax attention of n query rows; scores (q . k) * scale, fp32. */
 typedef struct {
@@ -117,6 +170,10 @@ typedef struct {
   const void* gate;        /* [n][ldg] logits or null: outputs times sigmoid(gate[., head]) */
   int64_t ldg;
   int window;              /* > 0: a query sees the newest `window` tokens up to itself */
+  int chunk;               /* > 0 (without a window): a query sees the tokens of its own chunk up to itself; chunks
+                            * are counted from position 0 */
+  const float* rel;        /* [H][rel_len] or null: added to the scaled score by distance, the last entry beyond */
+  int rel_len;
   int ring;                /* > 0: token j lies in row j % ring of k and v, else in row j - base */
   int base;
   const int* pos_dev;      /* position of query row 0 */
@@ -128,6 +185,10 @@ typedef struct {
   const float* fresh_v;
   int norm_dim;            /* > 0: q and fresh_k are divided by their root mean square over norm_dim */
   float eps;
+  const float* q_w;        /* [dim_s] or null: weights of these norms */
+  const float* k_w;
+  const float* other_v;    /* fp32 [G][vdim_s] or null: fresh_v <- (1 - *lambda) fresh_v + *lambda other_v */
+  const float* lambda;
 } dvAttnArgs;
 
 typedef struct {
@@ -158,13 +219,67 @@ typedef struct {
   float* gate;             /* [heads][vdim_s]: sigmoid of the output gate */
 } dvDeltaStepArgs;
 
+/* Mamba-2 recurrence over n tokens: S <- exp(-exp(A_log) dt) S + dt B x^T, y = S^T C + D x per head, where
+ * dt = softplus(logit + dt_bias); head h uses group h / (heads / groups) of B and C. */
+typedef struct {
+  const float* xbc;        /* [n][ld]: x [heads][vdim], then from off_b on B and from off_c on C, [groups][state_s] */
+  int64_t ld;
+  int off_b, off_c;
+  const void* dt;          /* [n][lddt] logits in `dtype`, a column per head */
+  int64_t lddt;
+  const float* A_log;      /* [heads] each */
+  const float* dt_bias;
+  const float* D;
+  float* S;                /* [heads][vdim][state_s] */
+  float* y;                /* [n][ldy], [heads][vdim] */
+  int64_t ldy;
+  float* tm;               /* scratch of tm_floats: ceil(min(n, 4096) / 64) * heads * 2688 */
+  int64_t tm_floats;
+  int n, heads, groups, vdim, state_s;
+} dvSsdArgs;
+
+/* One decode token of it from the fp32 projection row p (x, B, C after convolution and silu; z and dt logits);
+ * y [heads][vdim] is also multiplied by silu(z). */
+typedef struct {
+  const float* p;
+  int off_b, off_c, off_z, off_dt;
+  const float* A_log;
+  const float* dt_bias;
+  const float* D;
+  float* S;
+  float* y;
+  int heads, groups, vdim, state_s;
+} dvSsdStepArgs;
+
+/* Embedding of a token and its predecessor: embed[token] scale + bigram[row], row = (previous mul_prev + token
+ * mul_cur) mod buckets, or `buckets` for the first token of a sequence; every stream starts with it. */
+typedef struct {
+  const void* tokens;      /* [n] int64 */
+  void* history;           /* [capacity] int64: the sequence's tokens by position, written here */
+  int64_t capacity, vocab;
+  const void* embed;       /* [vocab][width] */
+  float scale;
+  const void* bigram;      /* [buckets + 1][width] or null */
+  int64_t buckets, mul_prev, mul_cur;
+  const int* pos_dev;
+  int pos_host, n;
+} dvEmbedArgs;
+
 /* x = x0 = embed[token] (x0 may be null), h = norm(x). */
 DV_API int dv_mix_embed(int dtype, const void* tokens, int64_t vocab, const void* embed, int n, int width, float* x,
                         float* x0, const dvDynTanh* norm, void* h, void* stream);
 /* Residual step of n x width values y (null: only x += x0 and h = pre(x)). */
 DV_API int dv_mix_residual(int dtype, const void* y, int64_t n, int width, const dvResidual* r, void* stream);
-/* y [n][ff] from gu [n][2 ff] (gate and up interleaved): g = min(g, limit), u = clamp(u), g sigmoid(1.702 g) (u + 1). */
-DV_API int dv_mix_clamped_glu(int dtype, const void* gu, int64_t count, float limit, void* y, void* stream);
+/* y [n][ff] from gu [n][2 ff] (gate and up interleaved): the gated unit `act` (DV_GLU_*). */
+DV_API int dv_mix_glu(int dtype, const void* gu, int64_t count, int act, float limit, void* y, void* stream);
+/* Streams: start of a portion (r->mix, r->out are not read). */
+DV_API int dv_mix_hyper_embed(int dtype, const dvEmbedArgs* e, const dvHyper* r, const dvRmsOut* norm, void* stream);
+/* Streams: what follows a sublayer with n x width values y (null: only u and h, the streams stay). */
+DV_API int dv_mix_hyper_rows(int dtype, const void* y, int n, const dvHyper* r, const dvRmsOut* norm, void* stream);
+DV_API int dv_mix_head_rows(int dtype, const dvHeadArgs* args, void* stream);
+/* out = t / rms(t) * w per group of `dim / groups` entries, t = y silu(z); entries dim .. padded - 1 become 0. */
+DV_API int dv_mix_gated_group_norm(int dtype, const float* y, int64_t ldy, const void* z, int64_t ldz, int64_t rows,
+                                   int dim, int groups, int padded, const float* w, float eps, void* out, void* stream);
 /* y = x / rms(x) * w, row by row; w has `padded` entries, the mean runs over `dim`. */
 DV_API int dv_mix_rms_rows(int dtype, const void* x, int64_t ldx, int64_t rows, int dim, int padded, const float* w,
                            float eps, void* y, int64_t ldy, void* stream);
@@ -193,6 +308,8 @@ DV_API int dv_mix_delta_gates(int dtype, const void* z, int64_t ldz, const void*
                               const float* dt_bias, int n, int heads, int dim_s, float* g, float* beta, void* stream);
 DV_API int dv_mix_delta_scan(const dvDeltaArgs* args, void* stream);
 DV_API int dv_mix_delta_step(int dtype, const dvDeltaStepArgs* args, void* stream);
+DV_API int dv_mix_ssd_scan(int dtype, const dvSsdArgs* args, void* stream);
+DV_API int dv_mix_ssd_step(const dvSsdStepArgs* args, void* stream);
 /* dv_greedy_advance_f16 for fp32 logits. */
 DV_API int dv_mix_greedy_advance(const float* logits, int vocab, void* token, void* position, void* seq_pos,
                                  void* sequences, int64_t seq_capacity, void* out_index, float* scores,
