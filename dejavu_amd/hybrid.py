@@ -323,7 +323,7 @@ class HybridLMHeadModel(GreedyDecoding, nn.Module):
                 return CausalLMOutput(logits=None)
             if list(rows) != list(range(n)):
                 h = h[torch.as_tensor(rows, device=h.device)]
-        elif last_token_only:
+        elif last_token_only and n > 1:
             h = h[-1:]
         return CausalLMOutput(logits=ops.linear(h, self.lm_head, f32=True)[None])
 

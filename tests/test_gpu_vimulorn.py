@@ -9,31 +9,11 @@ import torch
 
 from oracle import vimulorn_oracle as V
 from tests import vimulorn_utils as U
+from tests.mixer_utils import DTYPES, LIMIT, OP_LIMIT, close, dev, feed, host
 
 pytestmark = pytest.mark.gpu
 
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
-DTYPES = [torch.float32, torch.bfloat16]
-# largest rms difference of a row over the rms of the rows: fp32 rounding; bf16 operands and activations
-LIMIT = {torch.float32: 2e-5, torch.bfloat16: 3e-2}
-# a single mechanism on its own
-OP_LIMIT = {torch.float32: 1e-5, torch.bfloat16: 1.5e-2}
-
-
-def dev(a, dtype=torch.float32):
-    return torch.as_tensor(np.asarray(a), dtype=torch.float32).to(dtype).cuda()
-
-
-def host(t):
-    return t.detach().float().cpu().numpy().astype(np.float64)
-
-
-def close(got, want, limit, what):
-    s = U.spread(host(got) if torch.is_tensor(got) else got, want)
-    print(f"{what}: {s:.2e} (limit {limit:.0e})", flush=True)
-    assert s <= limit, what
-
-
 _models = {}
 
 
@@ -46,18 +26,6 @@ def model_of(name, dtype, seed=0, **kw):
         t = U.weights(cfg, seed=seed, ranks=U.RANKS[name], **kw)
         _models[key] = (cfg, U.as_numpy(t), build_model(cfg, t, dtype=dtype))
     return _models[key]
-
-
-def feed(model, params, tokens, cuts):
-    """Logits of all tokens, given in portions of the sizes in ``cuts`` (the last one repeated)."""
-    out, at, i = [], 0, 0
-    while at < len(tokens):
-        n = min(cuts[min(i, len(cuts) - 1)], len(tokens) - at)
-        ids = torch.tensor([tokens[at:at + n]], device="cuda")
-        out.append(model(ids, inference_params=params).logits[0])
-        params.sequence_len_offset += n
-        at, i = at + n, i + 1
-    return host(torch.cat(out))
 
 
 # ---- mechanisms ---------------------------------------------------------------------------------
