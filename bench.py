@@ -822,6 +822,34 @@ def vimulorn_kernels(torch, model, prompt, context):
     return table
 
 
+def generation_throughput(torch, model, vocab, prompts, decode_prompt, new_tokens, warmup):
+    """Prompt times of ``generate``, and its decode rate from HIP graphs behind a prompt of ``decode_prompt`` tokens."""
+    ids = torch.randint(0, vocab, (1, max(prompts + (decode_prompt,))), device="cuda")
+
+    def run(n, length, cg):
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        model.generate(ids[:, :n], max_length=length, cg=cg)
+        torch.cuda.synchronize()
+        return time.perf_counter() - t0
+
+    length = decode_prompt + new_tokens
+    for _ in range(max(1, warmup)):
+        run(decode_prompt, length, True)
+    total = min(run(decode_prompt, length, True) for _ in range(3))
+    out = {"prompt_ms": {}, "prompt_tokens_per_s": {}}
+    for n in prompts:
+        run(n, n + 1, False)
+        t = min(run(n, n + 1, False) for _ in range(3))
+        out["prompt_ms"][str(n)] = round(t * 1e3, 3)
+        out["prompt_tokens_per_s"][str(n)] = round(n / t)
+    run(decode_prompt, decode_prompt + 1, False)
+    t_prompt = min(run(decode_prompt, decode_prompt + 1, False) for _ in range(3))
+    out["decode_tokens_per_s"] = round((new_tokens - 1) / (total - t_prompt), 1)
+    out["decode_ms_per_token"] = round((total - t_prompt) / (new_tokens - 1) * 1e3, 4)
+    return out
+
+
 def vimulorn_bench(args):
     """Vimulorn at the layer sizes of real models (random weights): prompt and decode throughput beside an OPT-shaped
     sparse model of the same width, layers and feed-forward weights, and every kernel beside its like.  A step is one
@@ -837,39 +865,13 @@ def vimulorn_bench(args):
     new_tokens, decode_prompt = args.steps, 1024
     prompts = (128, 2048, 8192)
 
-    def throughput(model, vocab, prompts):
-        ids = torch.randint(0, vocab, (1, max(prompts + (decode_prompt,))), device="cuda")
-
-        def run(n, length, cg):
-            torch.cuda.synchronize()
-            t0 = time.perf_counter()
-            model.generate(ids[:, :n], max_length=length, cg=cg)
-            torch.cuda.synchronize()
-            return time.perf_counter() - t0
-
-        length = decode_prompt + new_tokens
-        for _ in range(max(1, args.warmup)):
-            run(decode_prompt, length, True)
-        total = min(run(decode_prompt, length, True) for _ in range(3))
-        out = {"prompt_ms": {}, "prompt_tokens_per_s": {}}
-        for n in prompts:
-            run(n, n + 1, False)
-            t = min(run(n, n + 1, False) for _ in range(3))
-            out["prompt_ms"][str(n)] = round(t * 1e3, 3)
-            out["prompt_tokens_per_s"][str(n)] = round(n / t)
-        run(decode_prompt, decode_prompt + 1, False)
-        t_prompt = min(run(decode_prompt, decode_prompt + 1, False) for _ in range(3))
-        out["decode_tokens_per_s"] = round((new_tokens - 1) / (total - t_prompt), 1)
-        out["decode_ms_per_token"] = round((total - t_prompt) / (new_tokens - 1) * 1e3, 4)
-        return out
-
     results = {}
     with torch.no_grad():
         for name in args.vimulorn:
             cfg = VIMULORN_CONFIGS[name]
             model = HybridLMHeadModel(HybridConfig.from_dict(cfg), device="cuda", dtype=torch.bfloat16).eval()
             init_vimulorn_synthetic(model, 1)
-            r = throughput(model, cfg["vocab"], prompts)
+            r = generation_throughput(torch, model, cfg["vocab"], prompts, decode_prompt, new_tokens, args.warmup)
             runs = [model.layers[i] for i, _ in model.runs]
             nbytes = model.lm_head.numel() * 2 + sum(
                 p.numel() * 2 for layer in runs for p in layer.parameters() if p.dtype == torch.bfloat16)
@@ -889,7 +891,7 @@ def vimulorn_bench(args):
             for emb in (opt.transformer.embeddings.word_embeddings, opt.transformer.embeddings.position_embeddings):
                 emb.weight.normal_(0.0, 0.02)
             opt.tie_weights()
-            o = throughput(opt, cfg["vocab"], prompts)
+            o = generation_throughput(torch, opt, cfg["vocab"], prompts, decode_prompt, new_tokens, args.warmup)
             d, hd, K, Hk, rk = width, 128, ffn // 4, heads // 2, 1000
             pred = (2 * d * rk + rk * ffn + rk * heads) * 2
             nb = (4 * d * d + 2 * d * ffn) * 2 + pred + (layers - 1) * ((4 * Hk * hd * d + 2 * K * d) * 2 + pred) + cfg["vocab"] * d * 2
@@ -906,6 +908,260 @@ def vimulorn_bench(args):
         "unit": "tokens/s", "n_gpus": 1, "steps": new_tokens, "warmup": args.warmup,
         "ms_per_step": lead["decode_ms_per_token"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
         "dtype": "bf16", "data": "synthetic", "config": {"workload": "vimulorn", "models": args.vimulorn,
+                                                        "decode_prompt": decode_prompt, "prompts": prompts},
+        "models": results}))
+
+
+def varolorn_kernels(torch, model, near, prompt, context):
+    """Every kernel of the design at the sizes of ``model`` beside the like kernel of ``near``, a Vimulorn model of the
+    same width: time per launch (HIP graph of launches over several sets of operands, so that no cache holds them), the
+    bytes or flops that have to be moved or done, and the fraction of the peak.  ``like``: the Vimulorn side."""
+    from dejavu_amd import mixer_ops as mo
+    from dejavu_amd.mixers import ChannelDelta, ChunkAttention, Mamba2, WindowAttention
+
+    dev, bf, f32, table = "cuda", torch.bfloat16, torch.float32, {}
+    width = model.embeddings.shape[1]
+    gen = torch.Generator(device=dev)
+    gen.manual_seed(3)
+
+    def rnd(*shape, dtype=bf):
+        return torch.randn(*shape, dtype=f32, device=dev, generator=gen).to(dtype)
+
+    def copies(W, least=600e6):
+        count = max(2, min(24, int(least // (W.numel() * W.element_size())) + 1))
+        return [W.detach().clone() for _ in range(count)]
+
+    def put(name, us, like_us, work, like_work, like, flops=False):
+        def entry(t, w):
+            if flops:
+                return {"us": round(t, 2), "TFLOPS": round(w / t / 1e6, 1), "frac": round(w / t / 1e6 / MFMA_PEAK_TFLOPS, 4)}
+            return {"us": round(t, 2), "GB/s": round(w / t / 1e3, 1), "frac": round(w / t / 1e3 / HBM_PEAK_GBPS, 4)}
+        row, other = entry(us, work), entry(like_us, like_work)
+        table[name] = dict(row, like=dict(other, kernel=like), ratio=round(other["frac"] / max(row["frac"], 1e-9), 2))
+
+    mixer = {}
+    for m in (model, near):
+        for layer in m.layers:
+            mixer.setdefault(type(layer.mixer), layer)
+    att, mam = mixer[ChunkAttention].mixer, mixer[Mamba2].mixer
+    win, dlt = mixer[WindowAttention].mixer, mixer[ChannelDelta].mixer
+    block, S = mixer[ChunkAttention], model.config.streams
+    mlp, read, dyn = block.mlp, block.entry, near.final_norm
+    eps = read.norm.eps
+
+    def streams(n):
+        return mo.HyperStream(rnd(n, S, width, dtype=f32), bf)
+
+    def plain_stream(n):
+        return mo.ResidualStream(rnd(n, width, dtype=f32), None, bf)
+
+    # ---- one token: products ----
+    u1 = mo.RmsRow(rnd(1, width, dtype=f32), read.norm.weight, width, eps, bf)
+    x1, s1, r1 = rnd(1, width), streams(1), plain_stream(1)
+    state = torch.zeros(mam.channels, 3, device=dev)
+
+    def row_product(name, W, fn, like, like_fn):
+        Ws = copies(W)
+        put("decode: " + name, time_kernel(torch, fn, Ws), time_kernel(torch, like_fn, Ws), W.numel() * 2, W.numel() * 2, like)
+
+    row_product("norm + attention projections + bias", att.in_proj, lambda w: mo.linear(u1, w, att.in_bias, f32=True),
+                "projections", lambda w: mo.linear(x1, w, f32=True))
+    row_product("norm + Mamba-2 projections + short convolution", mam.in_proj,
+                lambda w: mo.row_conv(u1, w, mam.conv, state, True, mam.conv_bias),
+                "projections + short convolution", lambda w: mo.row_conv(x1, w, mam.conv, state, True))
+    row_product("norm + gate / up + relu unit", mlp.gate_up, lambda w: mo.relu_glu(u1, w),
+                "gate / up + clamped unit", lambda w: mo.clamped_glu(x1, w, 7.0))
+    xf, xo = rnd(1, mlp.down.shape[1]), rnd(1, att.out_proj.shape[1])
+    row_product("down + streams", mlp.down, lambda w: s1.update(xf, w, None, block.hyper1, read),
+                "down + norm + residual + norm", lambda w: mo.linear_residual(xf, w, r1, dyn, dyn))
+    row_product("output projection + bias + streams", att.out_proj,
+                lambda w: s1.update(xo, w, att.out_bias, block.hyper1, read),
+                "output projection + norm + residual + norm", lambda w: mo.linear_residual(xo, w, r1, dyn, dyn))
+    y1 = rnd(1, mam.inner_s, dtype=f32)
+    grouped = mo.GroupedRow(y1, mam.norm, mam.inner, mam.norm_groups, eps, bf)
+    heads = mo.GatedHeads(y1, torch.rand(mam.inner_s, device=dev), dlt.norm, dlt.vdim, eps)
+    row_product("grouped norm + output projection + streams", mam.out_proj,
+                lambda w: s1.update(grouped, w, None, block.hyper1, read),
+                "head norm + gate + output projection + norm + residual + norm",
+                lambda w: heads.linear_residual(w, r1, dyn, dyn))
+    row_product("norm + head", model.lm_head, lambda w: mo.linear(u1, w, f32=True),
+                "head", lambda w: mo.linear(x1, w, f32=True))
+
+    # ---- one token: attention and recurrence ----
+    pos = att.chunk - 1  # a full chunk
+    H, G, ds, vs = att.heads, att.kv_heads, att.dim_s, att.vdim_s
+    row, sink = rnd(1, att.in_proj.shape[0], dtype=f32), torch.zeros(H, device=dev)
+    sets = [att.new_state(att.chunk) for _ in range(24)]
+    nb = (sets[0]["k"].numel() + sets[0]["v"].numel()) * 2
+    mix = (rnd(G * vs, dtype=f32), att.vmix)
+    us = time_kernel(torch, lambda st: mo.ring_attention_row(
+        row, st["k"], st["v"], H, G, att.dim, att.scale, eps, None, pos, chunk=att.chunk, rel=att.rel, q_weight=att.q_norm,
+        k_weight=att.k_norm, mix_v=mix, gate=row[0, att.off_g:]), sets)
+    like_us = time_kernel(torch, lambda st: mo.window_attention_row(row, st["k"], st["v"], H, G, att.dim, att.scale, eps, sink,
+                                                                    att.chunk, None, pos), sets)
+    put(f"decode: attention, chunk of {att.chunk}", us, like_us, nb, nb, "windowed attention, the same sizes")
+    row = rnd(1, mam.in_proj.shape[0], dtype=f32)
+    rule = (mam.A_log, mam.dt_bias, mam.D)
+    sets = [mam.new_state(1)["S"] for _ in range(24)]
+    us = time_kernel(torch, lambda st: mo.ssd_step(row, *rule, st, mam.groups, mam.off_b, mam.off_c, mam.off_z, mam.off_dt,
+                                                   mam.inner_s), sets)
+    drow = rnd(1, dlt.in_proj.shape[0], dtype=f32)
+    dsets = [(dlt.new_state(1)["S"], dlt.decay_up.clone(), dlt.gate_up.clone()) for _ in range(24)]
+    like_us = time_kernel(torch, lambda st: mo.delta_row(drow, dlt.offsets, dlt.heads, dlt.kv_heads, dlt.dim, st[1], st[2],
+                                                         dlt.A_log, dlt.dt_bias, st[0]), dsets)
+    put("decode: recurrence", us, like_us, sets[0].numel() * 8,
+        dsets[0][0].numel() * 8 + (dlt.decay_up.numel() + dlt.gate_up.numel()) * 2, "delta rule step with its low-rank products")
+    ids = torch.randint(0, model.config.vocab, (1, prompt), device=dev)
+    e, history = model.config.embedding, torch.zeros(prompt, dtype=torch.long, device=dev)
+
+    def embed(n):
+        return lambda a: mo.hyper_embed(ids[0, :n], model.embeddings, e.scale, model.bigram, e.mul_prev, e.mul_cur, history,
+                                        None, 0, S, read)
+
+    def like_embed(n):
+        return lambda a: mo.embed(ids[0, :n], near.embeddings, dyn, False)
+
+    put("decode: embedding", time_kernel(torch, embed(1), [0]), time_kernel(torch, like_embed(1), [0]),
+        width * (4 + 4 * S + 4), width * (2 + 4 + 2), "embedding + norm")
+
+    # ---- portions of a few rows ----
+    for n in (16, 64):
+        xn = rnd(n, width)
+        for name, W, fn, like, like_fn in (
+                ("gate / up + relu unit", mlp.gate_up, lambda w: mo.relu_glu(xn, w), "gate / up + clamped unit",
+                 lambda w: mo.clamped_glu(xn, w, 7.0)),
+                ("product + bias", att.in_proj, lambda w: mo.linear(xn, w, att.in_bias), "plain product",
+                 lambda w: mo.linear(xn, w))):
+            Ws = copies(W)
+            put(f"portion of {n}: {name}", time_kernel(torch, fn, Ws), time_kernel(torch, like_fn, Ws), W.numel() * 2,
+                W.numel() * 2, like)
+        sn, rn, yn = streams(n), plain_stream(n), rnd(n, width)
+        eye, code = block.hyper1, mo._DTYPES[bf]
+
+        def rows(a, sn=sn, yn=yn, n=n):
+            r, o, h = sn._structs(read, True)
+            r.mix, r.out = eye.mix.data_ptr(), eye.out.data_ptr()
+            mo.check(mo.lib.dv_mix_hyper_rows(code, yn.data_ptr(), n, mo._ref(r), mo._ref(o), mo._stream()), "hyper_rows")
+
+        put(f"portion of {n}: streams + norm", time_kernel(torch, rows, [0]),
+            time_kernel(torch, lambda a: mo.residual(yn, rn, dyn, dyn), [0]), n * width * (8 * S + 4), n * width * 12,
+            "norm + residual + norm")
+
+    # ---- prompt ----
+    n, c = prompt, min(att.chunk, prompt)
+    q, k, v = rnd(n, H * ds), rnd(n, G * ds), rnd(n, G * vs)
+    gate = rnd(n, (H + 7) // 8 * 8)
+    pairs = n // c * c * (c + 1) / 2.0
+    wpairs = c * n - c * (c - 1) / 2.0
+    us = time_kernel(torch, lambda a: mo.portion_attention(q, k, v, H, G, att.scale, 0, 0, gate=gate, chunk=c, rel=att.rel),
+                     [0], launches=10)
+    like_us = time_kernel(torch, lambda a: mo.portion_attention(q, k, v, H, G, att.scale, 0, 0, sink=sink, window=c), [0],
+                          launches=10)
+    put(f"prompt of {n}: attention, chunk of {c}", us, like_us, 2.0 * H * (ds + vs) * pairs, 2.0 * H * (ds + vs) * wpairs,
+        f"windowed attention, window {c}", flops=True)
+
+    def elementwise(name, fn, nbytes, like, like_fn, like_bytes):
+        put(f"prompt of {n}: {name}", time_kernel(torch, fn, [0]), time_kernel(torch, like_fn, [0]), nbytes, like_bytes, like)
+
+    y, sn, rn = rnd(n, width), streams(n), plain_stream(n)
+
+    def rows(a):
+        r, o, h = sn._structs(read, True)
+        r.mix, r.out = block.hyper1.mix.data_ptr(), block.hyper1.out.data_ptr()
+        mo.check(mo.lib.dv_mix_hyper_rows(0, y.data_ptr(), n, mo._ref(r), mo._ref(o), mo._stream()), "hyper_rows")
+
+    elementwise("streams + norm", rows, n * width * (8 * S + 4), "norm + residual + norm",
+                lambda a: mo.residual(y, rn, dyn, dyn), n * width * 12)
+    elementwise("embedding + streams + norm", embed(n), n * width * (4 + 4 * S + 2), "embedding + norm", like_embed(n),
+                n * width * (2 + 4 + 2))
+    gu = rnd(n, mlp.gate_up.shape[0])
+    out = torch.empty(n, mlp.gate_up.shape[0] // 2, dtype=bf, device=dev)
+
+    def glu(act):
+        return lambda a: mo.lib.dv_mix_glu(0, gu.data_ptr(), out.numel(), act, 7.0, out.data_ptr(), mo._stream())
+
+    elementwise("relu unit", glu(1), gu.numel() * 3, "clamped unit", glu(0), gu.numel() * 3)
+    p = rnd(n, att.in_proj.shape[0])
+    vf = rnd(n, G * vs)
+    hw, hs = win.channels, win.new_state(1)["conv"]
+    wp = rnd(n, hw)
+    wq, wk, wv = (torch.empty(n, w, dtype=bf, device=dev) for w in (win.heads * ds, win.kv_heads * ds, win.kv_heads * vs))
+    elementwise("head norms + mixed values",
+                lambda a: mo.head_rows(p, [(H, ds, att.dim, (att.q_norm, eps), q), (G, ds, att.dim, (att.k_norm, eps), k),
+                                           (G, vs, att.vdim, (vf, att.vmix), v)]),
+                n * (att.off_g * 4 + G * vs * 2), "short convolution + head RMS norm",
+                lambda a: mo.short_conv(wp, win.conv, hs, [(win.heads, ds, win.dim, 1, eps, 1.0, wq),
+                                                           (win.kv_heads, ds, win.dim, 1, eps, 1.0, wk),
+                                                           (win.kv_heads, vs, win.vdim, 0, 0.0, 1.0, wv)], False), n * hw * 4)
+    p = rnd(n, mam.in_proj.shape[0])
+    xbc = torch.empty(n, mam.channels, dtype=f32, device=dev)
+    dp = rnd(n, dlt.in_proj.shape[0])
+    dg, dh = dlt.kv_heads, dlt.heads
+    dq, dk, dvv = (torch.empty(n, w, dtype=f32, device=dev) for w in (dg * dlt.dim_s, dg * dlt.dim_s, dh * dlt.vdim_s))
+    dcs = dlt.new_state(1)["conv"]
+    elementwise("short convolution",
+                lambda a: mo.short_conv(p, mam.conv, state, [(mam.channels // 8, 8, 8, 0, 0.0, 1.0, xbc)], True, mam.conv_bias),
+                n * mam.channels * 6, "short convolution + unit norms (delta rule)",
+                lambda a: mo.short_conv(dp, dlt.conv, dcs, [(dg, dlt.dim_s, dlt.dim, 2, 0.0, 1.0, dq),
+                                                            (dg, dlt.dim_s, dlt.dim, 2, 0.0, 1.0, dk),
+                                                            (dh, dlt.vdim_s, dlt.vdim, 0, 0.0, 1.0, dvv)], True),
+                n * dlt.channels * 6)
+    St, dS = mam.new_state(1)["S"], dlt.new_state(1)["S"]
+    dz, db = rnd(n, dh * dlt.dim_s), rnd(n, 64)
+    g, beta = mo.delta_gates(dz, db, dlt.A_log, dlt.dt_bias, dh)
+    scan = lambda a: mo.ssd_scan(xbc, p[:, mam.off_dt:mam.off_dt + mam.heads], *rule, St, mam.groups, mam.off_b,  # noqa: E731
+                                 mam.off_c, mam.inner_s)
+    elementwise("recurrence", scan, 4 * n * (mam.channels + mam.inner_s), "delta rule scan",
+                lambda a: mo.delta_scan(dq, dk, dvv, g, beta, dS, dh, dg),
+                4 * n * (2 * dg * dlt.dim_s + 2 * dh * dlt.vdim_s + dh * dlt.dim_s))
+    ys, z = scan(0), p[:, mam.off_z:mam.off_dt]
+    od, gt = rnd(n, dh, dlt.vdim_s, dtype=f32), rnd(n, dh * dlt.vdim_s)
+    elementwise("gated group norm", lambda a: mo.gated_group_norm(ys, z, mam.norm, mam.inner, mam.norm_groups, eps),
+                n * mam.inner * 8, "gated head norm", lambda a: mo.gated_head_norm(od, gt, dlt.norm, dlt.vdim, eps),
+                n * dh * dlt.vdim_s * 8)
+    return table
+
+
+def varolorn_bench(args):
+    """Varolorn at the layer sizes of real models (random weights): prompt and decode throughput beside a Vimulorn model
+    of the same width, layer runs, feed-forward and vocabulary, and every kernel beside its like.  A step is one
+    generated token; prints its own JSON line."""
+    import torch
+
+    from dejavu_amd.hybrid import HybridConfig, HybridLMHeadModel
+    from dejavu_amd.workloads import VAROLORN_CONFIGS, VIMULORN_CONFIGS, init_varolorn_synthetic, init_vimulorn_synthetic
+
+    torch.cuda.set_device(0)
+    decode_prompt, prompts, results = 1024, (128, 2048, 8192), {}
+
+    def measured(model, vocab):
+        r = generation_throughput(torch, model, vocab, prompts, decode_prompt, args.steps, args.warmup)
+        nbytes = model.lm_head.numel() * 2 + sum(p.numel() * 2 for i, _ in model.runs for p in model.layers[i].parameters()
+                                                 if p.dtype == torch.bfloat16)
+        r["weight_MB_per_token"] = round(nbytes / 1e6, 1)
+        r["weight_frac_of_hbm_peak"] = round(nbytes / r["decode_ms_per_token"] / 1e6 / HBM_PEAK_GBPS, 4)
+        return r
+
+    with torch.no_grad():
+        for name in args.varolorn:
+            cfg, other = VAROLORN_CONFIGS[name], VIMULORN_CONFIGS["vimulorn-" + name.split("-")[1]]
+            model = HybridLMHeadModel(HybridConfig.from_dict_streams(cfg), device="cuda", dtype=torch.bfloat16).eval()
+            near = HybridLMHeadModel(HybridConfig.from_dict(other), device="cuda", dtype=torch.bfloat16).eval()
+            init_varolorn_synthetic(model, 1)
+            init_vimulorn_synthetic(near, 1)
+            r = measured(model, cfg["vocab"])
+            r["vimulorn_of_equal_size"] = measured(near, other["vocab"])
+            if not args.no_kernels:
+                r["kernels"] = varolorn_kernels(torch, model, near, 2048, 4096)
+            results[name] = r
+            del model, near
+            torch.cuda.empty_cache()
+    lead = results[args.varolorn[0]]
+    print(json.dumps({
+        "metric": f"tokens_per_s, greedy decode, {args.varolorn[0]}, batch 1", "value": lead["decode_tokens_per_s"],
+        "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+        "ms_per_step": lead["decode_ms_per_token"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+        "dtype": "bf16", "data": "synthetic", "config": {"workload": "varolorn", "models": args.varolorn,
                                                         "decode_prompt": decode_prompt, "prompts": prompts},
         "models": results}))
 
@@ -1028,13 +1284,16 @@ def main():
                     help="batch sizes of --workload mlp")
     ap.add_argument("--K", type=int, default=None,
                     help="--workload mlp: active neurons (default: the configuration's K; K = ffn is the dense block)")
-    ap.add_argument("--workload", default="layer", choices=["layer", "decode", "mlp", "vimulorn"],
+    ap.add_argument("--workload", default="layer", choices=["layer", "decode", "mlp", "vimulorn", "varolorn"],
                     help="layer: the headline sparse decode layer; decode: end-to-end greedy generation "
                          "(40-layer OPT-13B shape, --steps = new tokens, default 256); vimulorn: prompt and decode "
-                         "throughput and the kernels of Vimulorn models beside OPT ones of equal size")
+                         "throughput and the kernels of Vimulorn models beside OPT ones of equal size; varolorn: the "
+                         "same of Varolorn models beside Vimulorn ones")
     ap.add_argument("--vimulorn", nargs="+", default=["vimulorn-4k", "vimulorn-2k"],
                     help="model sizes of --workload vimulorn (workloads.VIMULORN_CONFIGS)")
-    ap.add_argument("--no-kernels", action="store_true", help="--workload vimulorn: throughput only")
+    ap.add_argument("--varolorn", nargs="+", default=["varolorn-4k", "varolorn-2k"],
+                    help="model sizes of --workload varolorn (workloads.VAROLORN_CONFIGS)")
+    ap.add_argument("--no-kernels", action="store_true", help="--workload vimulorn / varolorn: throughput only")
     ap.add_argument("--decode-layers", type=int, default=40)
     ap.add_argument("--no-other-workloads", action="store_true",
                     help="default run only: skip the batched-layer (batch 8 / 16 / 32) and greedy-decode legs")
@@ -1068,10 +1327,10 @@ def main():
     from dejavu_amd.workloads import CONFIGS
 
     dv_modules.USE_SIDE_STREAM = args.side_stream
-    if args.workload == "vimulorn":
+    if args.workload in ("vimulorn", "varolorn"):
         args.steps = 256 if args.steps is None else args.steps
         args.warmup = 1 if args.warmup is None else args.warmup
-        return vimulorn_bench(args)
+        return (vimulorn_bench if args.workload == "vimulorn" else varolorn_bench)(args)
     if args.workload == "decode":
         args.steps = 256 if args.steps is None else args.steps
         args.warmup = 1 if args.warmup is None else args.warmup

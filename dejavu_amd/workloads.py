@@ -93,6 +93,48 @@ VIMULORN_CONFIGS = {
 }
 
 
+# Varolorn decoders of the same width, depth and feed-forward: [chunk attention, Mamba-2, Mamba-2] three times
+def varolorn_config(width: int, ff: int, heads: int, chunk: int, streams: int = 4, vocab: int = 32768) -> dict:
+    hd, inner = 128, 2 * width
+    mlp = {"kind": "dense", "ff": ff}
+    attention = {"type": "attention", "mlp": mlp,
+                 "mixer": dict(heads=heads, kv_heads=heads // 4, dim=hd, vdim=hd, bias_max=128, bias_rows=32, v_mix=True,
+                               mask={"size": chunk}, scale=hd ** -0.5)}
+    mamba = {"type": "mamba2", "mlp": mlp,
+             "mixer": dict(heads=inner // 64, groups=8, vdim=64, state=128, conv=4, norm_groups=8)}
+    return {"architecture": "Varolorn", "width": width, "vocab": vocab, "norm": {"eps": 1e-5}, "streams": streams,
+            "embedding": {"scale": width ** 0.5, "bigram": {"buckets": 65521, "mul_prev": 8191, "mul_cur": 31}},
+            "layers": [attention, mamba, mamba] * 3}
+
+
+VAROLORN_CONFIGS = {
+    "varolorn-4k": varolorn_config(4096, 11008, 32, 2048),
+    "varolorn-2k": varolorn_config(2048, 5632, 16, 1024),
+}
+
+
+@torch.no_grad()
+def init_varolorn_synthetic(model, seed: int = 0) -> None:
+    """Seeded random weights in place: matrices ~ N(0, 1 / columns), norm weights and D 1, streams read evenly and kept
+    as they are, everything else small."""
+    dev = next(model.parameters()).device
+    gen = torch.Generator(device=dev)
+    gen.manual_seed(seed)
+    for name, p in model.named_parameters():
+        leaf = name.rsplit(".", 1)[-1]
+        if leaf in ("weight", "norm", "q_norm", "k_norm", "D", "out"):
+            p.fill_(1.0)
+        elif leaf == "weights":
+            p.fill_(1.0 / p.numel())
+        elif leaf == "mix":
+            p.copy_(torch.eye(p.shape[0], device=dev))
+        elif leaf in ("A_log", "dt_bias"):
+            p.fill_(-1.0)
+        else:
+            tmp = torch.empty(p.shape, dtype=torch.float32, device=dev)
+            p.copy_(tmp.normal_(0.0, p.shape[-1] ** -0.5 if p.dim() == 2 else 0.1, generator=gen))
+
+
 @torch.no_grad()
 def init_vimulorn_synthetic(model, seed: int = 0) -> None:
     """Seeded random weights in place: matrices ~ N(0, 1 / columns), norm weights 1, everything else small."""

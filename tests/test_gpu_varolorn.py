@@ -301,9 +301,9 @@ def rel_of(table, far, chunk, T):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("T,H,G,dim,vdim,chunk,rows,far", [
-    (150, 4, 2, 24, 40, None, 8, 30), (300, 3, 3, 64, 32, 64, 32, 120), (70, 6, 1, 72, 104, 3, 4, 6),
+    (150, 4, 2, 24, 40, None, 8, 30), (300, 3, 3, 64, 32, 64, 32, 100), (70, 6, 1, 72, 104, 3, 4, 6),
     (330, 2, 2, 136, 136, 65, 6, 9), (270, 2, 1, 232, 248, 128, 16, 200), (65, 9, 1, 16, 8, 1, 2, 3),
-    (90, 2, 1, 264, 40, 20, 5, 9), (400, 1, 1, 48, 64, 300, 10, 40)])
+    (90, 2, 1, 264, 40, 20, 5, 9), (400, 1, 1, 56, 64, 300, 10, 40)])
 def test_attention_in_chunks_with_a_bias(T, H, G, dim, vdim, chunk, rows, far, dtype):
     """Prompt, portions cut inside chunks, and decoding from rings with norms, mixed values and gates."""
     from dejavu_amd import mixer_ops as ops
@@ -374,7 +374,7 @@ def test_a_single_key_at_the_edge_of_a_chunk(at, key, chunk, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("rows,far", [(32, 120), (8, 30), (5, 9)])
+@pytest.mark.parametrize("rows,far", [(32, 100), (8, 30), (5, 9)])
 def test_every_distance_has_its_bias(rows, far, dtype):
     """Equal keys, a large bias on one row of the table at a time: the weight goes to the distances of that row."""
     from dejavu_amd import mixer_ops as ops

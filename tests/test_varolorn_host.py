@@ -26,7 +26,7 @@ def test_recurrence_of_the_oracle_matches_its_sum():
             np.testing.assert_allclose(y[t, h], want, atol=1e-12)
 
 
-@pytest.mark.parametrize("rows,far", [(32, 120), (8, 12), (6, 20), (5, 9), (2, 3), (7, 64), (16, 128), (20, 11), (12, 5)])
+@pytest.mark.parametrize("rows,far", [(32, 100), (8, 12), (6, 20), (5, 9), (2, 3), (7, 64), (16, 128), (20, 11), (12, 5)])
 def test_distance_buckets(rows, far):
     """Against the logarithm where that is not within rounding of a step, and the two statements of it against each
     other; the last row is reached at ``far`` and kept."""

@@ -37,7 +37,7 @@ _LAYERS = {
               (attention(6, 2, 28, 12, 33, 6, 20), None), (attention(3, 3, 16, 24, 70, 12, 40, v_mix=False), ff(33)),
               (mamba(3, 1, 8, 40, 2, 1), None), (attention(2, 2, 8, 12, 64, 5, 9, scale=0.5), ff(24))],
     # one stream, the recurrence first, one tap, heads that are no multiple of anything, chunks longer than sequences
-    "one": [(mamba(3, 3, 10, 8, 1, 3), ff(32)), (attention(2, 1, 32, 64, 200, 32, 120), None),
+    "one": [(mamba(3, 3, 10, 8, 1, 3), ff(32)), (attention(2, 1, 32, 64, 200, 32, 100), None),
             (mamba(5, 1, 7, 24, 3, 1), ff(16))],
     # more streams than the fused epilogue takes, five taps, chunks of one token, bias rows that end before the chunk
     "many": [(attention(2, 2, 16, 8, 1, 4, 6), ff(40)), (mamba(6, 2, 12, 72, 5, 4), ff(24)),
