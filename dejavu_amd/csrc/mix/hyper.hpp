@@ -35,12 +35,12 @@ using RmsOut = dvRmsOut;
 
 // One workgroup per token (several for one token without a norm: grid.y).  EMBED: the streams start with the embedding;
 // else y joins them (null: they stay).  Four channels per thread; u is kept in LDS for the norm (dynamic, width floats).
-// SM: streams kept in registers (>= streams).
-template <typename T, int SM, bool EMBED>
-__global__ __launch_bounds__(256) void hyper_rows_kernel(const T* __restrict__ y, HyperArgs a, EmbedArgs em, RmsOut norm) {
+// SM: streams kept in registers (>= streams).  TH: threads.
+template <typename T, int SM, bool EMBED, int TH>
+__global__ __launch_bounds__(TH) void hyper_rows_kernel(const T* __restrict__ y, HyperArgs a, EmbedArgs em, RmsOut norm) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem_raw[];
   float* us = reinterpret_cast<float*>(smem_raw);
-  __shared__ float coef[SM * (SM + 2)], red[4];
+  __shared__ float coef[SM * (SM + 2)], red[TH / 64];
   const int tid = threadIdx.x, S = a.streams;
   const int64_t row = blockIdx.x;
   float* x = a.x + row * S * a.width;
@@ -61,28 +61,38 @@ __global__ __launch_bounds__(256) void hyper_rows_kernel(const T* __restrict__ y
     }
     if (tid == 0 && blockIdx.y == 0 && pos < em.capacity) history[pos] = tok;  // no workgroup of this call reads it
   }
-  hyper_coefficients(a, coef, tid, 256);
+  // the first values are requested before the coefficients are there
+  float4_t old[SM], add[2];
+  auto load = [&](int c) {
+    if constexpr (EMBED) {
+      add[0] = add[1] = float4_t{0.f, 0.f, 0.f, 0.f};
+      if (e0) add[0] = load_quad(e0 + c);
+      if (e1) add[1] = load_quad(e1 + c);
+    } else {
+#pragma unroll
+      for (int s = 0; s < SM; ++s)
+        if (s < S) old[s] = *reinterpret_cast<const float4_t*>(x + (int64_t)s * a.width + c);
+      if (y) add[0] = load_quad(y + row * a.width + c);
+    }
+  };
+  const int c0 = (blockIdx.y * TH + tid) * 4, step = gridDim.y * TH * 4;
+  if (c0 < a.width) load(c0);
+  hyper_coefficients(a, coef, tid, TH);
   __syncthreads();
   float ss = 0.f;
-  for (int c = (blockIdx.y * 256 + tid) * 4; c < a.width; c += gridDim.y * 1024) {
+  for (int c = c0; c < a.width; c += step) {
     float4_t u = {0.f, 0.f, 0.f, 0.f};
+    if (c != c0) load(c);
     if constexpr (EMBED) {
-      float4_t v = {0.f, 0.f, 0.f, 0.f};
-      if (e0) v = load_quad(e0 + c) * em.scale;
-      if (e1) v += load_quad(e1 + c);
+      const float4_t v = add[0] * em.scale + add[1];
       for (int s = 0; s < S; ++s) {
         *reinterpret_cast<float4_t*>(x + (int64_t)s * a.width + c) = v;
         u += v * coef[s];
       }
     } else {
-      float4_t old[SM];
-#pragma unroll
-      for (int s = 0; s < SM; ++s)
-        if (s < S) old[s] = *reinterpret_cast<const float4_t*>(x + (int64_t)s * a.width + c);
       if (y) {
-        const float4_t yv = load_quad(y + row * a.width + c);
         for (int t = 0; t < S; ++t) {
-          float4_t v = yv * coef[S + t];
+          float4_t v = add[0] * coef[S + t];
 #pragma unroll
           for (int s = 0; s < SM; ++s)
             if (s < S) v += old[s] * coef[2 * S + s * S + t];
@@ -107,9 +117,12 @@ __global__ __launch_bounds__(256) void hyper_rows_kernel(const T* __restrict__ y
   ss = wave_sum(ss);
   if ((tid & 63) == 0) red[tid >> 6] = ss;
   __syncthreads();
-  const float s = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / norm.dim + norm.eps);
+  ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < TH / 64; ++i) ss += red[i];
+  const float s = 1.f / sqrtf(ss / norm.dim + norm.eps);
   T* h = reinterpret_cast<T*>(norm.h) + row * a.width;
-  for (int c = tid * 4; c < a.width; c += 1024)  // the entries this thread has written
+  for (int c = c0; c < a.width; c += step)  // the entries this thread has written
     store_quad(h + c, *reinterpret_cast<const float4_t*>(us + c) * s * *reinterpret_cast<const float4_t*>(norm.w + c));
 }
 
@@ -121,11 +134,11 @@ using HeadArgs = dvHeadArgs;
 template <typename T>
 __global__ __launch_bounds__(256) void head_rows_kernel(HeadArgs a) {
   const int heads = a.g[0].heads + a.g[1].heads + a.g[2].heads;
-  const int64_t unit = (int64_t)blockIdx.x * 16 + (threadIdx.x >> 4);
+  const unsigned unit = blockIdx.x * 16 + (threadIdx.x >> 4);
   const int sub = threadIdx.x & 15;
-  const bool ok = unit < (int64_t)a.n * heads;  // whole rows of lanes: the sum below stays inside one
-  const int64_t row = ok ? unit / heads : 0;
-  int h = ok ? (int)(unit % heads) : 0, base = 0, gi = 0;
+  const bool ok = unit < (unsigned)a.n * (unsigned)heads;  // whole rows of lanes: the sum below stays inside one
+  const int64_t row = ok ? unit / (unsigned)heads : 0;
+  int h = ok ? (int)(unit % (unsigned)heads) : 0, base = 0, gi = 0;
   if (h >= a.g[0].heads) {
     h -= a.g[0].heads;
     base = a.g[0].heads * a.g[0].stride;
@@ -141,9 +154,14 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HeadArgs a) {
   const T* other = g.other ? reinterpret_cast<const T*>(g.other) + row * g.ldo + (int64_t)h * g.stride : nullptr;
   T* out = reinterpret_cast<T*>(g.out) + row * g.ld + (int64_t)h * g.stride;
   const float lam = other ? *g.lambda : 0.f;
-  Pack8<T> v;
+  Pack8<T> v, o0;
+  Pack8<float> w0;
   v.zero();
-  if (sub * 8 < g.stride) v.load(in + sub * 8);
+  if (sub * 8 < g.stride) {
+    v.load(in + sub * 8);
+    if (g.w) w0.load(g.w + sub * 8);
+    if (other) o0.load(other + sub * 8);
+  }
   float ss = 0.f;
 #pragma unroll
   for (int e = 0; e < 8; ++e) ss = __builtin_fmaf(v.get(e), v.get(e), ss);  // entries from dim on are zero
@@ -157,17 +175,22 @@ __global__ __launch_bounds__(256) void head_rows_kernel(HeadArgs a) {
   if (!ok) return;
   const float s = g.w ? 1.f / sqrtf(ss / g.dim + g.eps) : 1.f;
   for (int c = sub * 8; c < g.stride; c += 128) {
-    Pack8<T> t = v, o;
+    Pack8<T> t = v;
     if (c >= 128) t.load(in + c);
-    o.zero();
-    if (other) o.load(other + c);
     __attribute__((aligned(16))) T r[8];
+    if (g.w) {
+      Pack8<float> w = w0;
+      if (c >= 128) w.load(g.w + c);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      float x = t.get(e) * s;
-      if (g.w) x *= g.w[c + e];
-      if (other) x = __builtin_fmaf(lam, o.get(e), (1.f - lam) * x);
-      r[e] = from_f<T>(x);
+      for (int e = 0; e < 8; ++e) r[e] = from_f<T>(t.get(e) * s * w.get(e));
+    } else if (other) {
+      Pack8<T> o = o0;
+      if (c >= 128) o.load(other + c);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) r[e] = from_f<T>(__builtin_fmaf(lam, o.get(e), (1.f - lam) * t.get(e)));
+    } else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) r[e] = from_f<T>(t.get(e));
     }
     *reinterpret_cast<Pack8<T>*>(out + c) = *reinterpret_cast<const Pack8<T>*>(r);
   }
@@ -183,10 +206,10 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __re
   constexpr int TH = 64 * W, NX = 4, V = VEC ? 4 : 1;
   __shared__ float red[4];
   const int groups = dim / gs, t = threadIdx.x % TH;
-  const int64_t unit = (int64_t)blockIdx.x * (4 / W) + threadIdx.x / TH;
+  const unsigned unit = blockIdx.x * (4 / W) + threadIdx.x / TH;
   const bool ok = unit < rows * groups;  // whole waves
-  const int64_t row = ok ? unit / groups : 0;
-  const int g = ok ? (int)(unit % groups) : 0;
+  const int64_t row = ok ? unit / (unsigned)groups : 0;
+  const int g = ok ? (int)(unit % (unsigned)groups) : 0;
   const float* yr = y + row * ldy + g * gs;
   const T* zr = z + row * ldz + g * gs;
   auto value = [&](int c) {

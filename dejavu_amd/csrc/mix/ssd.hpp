@@ -126,15 +126,17 @@ __global__ __launch_bounds__(256) void ssd_chunk_kernel(SsdArgs a, int hp) {
 // accumulators of the 16x16x4 products (element i of a lane: channel 4 (lane / 16) + i of a tile, column lane % 16),
 // which is also the operand layout of the product with C when its channels are taken in that order; the waves exchange
 // the state through LDS once per chunk, then every wave makes 16 tokens of Y and its own channels of the next state.
+// Operands are loaded by the lanes that use them, a chunk ahead: those of the state's own part as soon as it is done with
+// them, those of the product with the state after that product.
 template <int NT>
 struct SsdOperands {
-  float4_t c[4 * NT], m[4], e[4], p0;
+  float4_t c[4 * NT], p0, m[4], e[4];
   float b[NT][4][4], x[4][4], total;
 };
 
 // Grid: heads * ceil(vdim / 16), head fastest.
 template <int NT>
-__global__ __launch_bounds__(256) void ssd_scan_kernel(SsdArgs a) {
+__global__ __launch_bounds__(256, NT <= 2 ? 2 : 1) void ssd_scan_kernel(SsdArgs a) {
   constexpr int C = kSsdChunk;
   __shared__ __attribute__((aligned(16))) float4_t state[2][4 * NT][64];
   const int head = blockIdx.x % a.heads, tile = blockIdx.x / a.heads;
@@ -154,15 +156,12 @@ __global__ __launch_bounds__(256) void ssd_scan_kernel(SsdArgs a) {
   const float* Bg = a.xbc + a.off_b + group * N;
   const float* Cg = a.xbc + a.off_c + group * N;
   const int chunks = (a.n + C - 1) / C;
-  auto load = [&](SsdOperands<NT>& o, int c) {
+  SsdOperands<NT> o;
+  // channels past the state meet zeros of S, tokens past the end zeros of M and e (rows of Y are not stored)
+  auto load_own = [&](int c) {
     const float* src = a.tm + ((int64_t)c * a.heads + head) * SsdChunk::floats;
-    // channels past the state meet zeros of S, tokens past the end zeros of M and e (rows of Y are not stored)
-    const float* cr = Cg + (int64_t)min(c * C + wave * 16 + l16, a.n - 1) * a.ld;
-#pragma unroll
-    for (int t = 0; t < 4 * NT; ++t) o.c[t] = *reinterpret_cast<const float4_t*>(cr + min(t * 16 + q4 * 4, N - 4));
 #pragma unroll
     for (int k = 0; k < 4; ++k) {
-      o.m[k] = *reinterpret_cast<const float4_t*>(src + SsdChunk::m + (wave * (wave + 1) / 2 + min(k, wave)) * 256 + lane * 4);
       o.e[k] = *reinterpret_cast<const float4_t*>(src + SsdChunk::e + k * 16 + q4 * 4);
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
@@ -171,24 +170,33 @@ __global__ __launch_bounds__(256) void ssd_scan_kernel(SsdArgs a) {
 #pragma unroll
         for (int t = 0; t < NT; ++t) o.b[t][k][i] = Bg[row + min((wave * NT + t) * 16 + l16, N - 1)];
       }
+      o.m[k] = *reinterpret_cast<const float4_t*>(src + SsdChunk::m + (wave * (wave + 1) / 2 + min(k, wave)) * 256 + lane * 4);
     }
-    o.p0 = *reinterpret_cast<const float4_t*>(src + SsdChunk::p0 + wave * 16 + q4 * 4);
     o.total = src[SsdChunk::p0 + C - 1];
   };
-  auto step = [&](const SsdOperands<NT>& o, int c, int par) {
+  auto load_read = [&](int c) {
+    const float* cr = Cg + (int64_t)min(c * C + wave * 16 + l16, a.n - 1) * a.ld;
+#pragma unroll
+    for (int t = 0; t < 4 * NT; ++t) o.c[t] = *reinterpret_cast<const float4_t*>(cr + min(t * 16 + q4 * 4, N - 4));
+    o.p0 = *reinterpret_cast<const float4_t*>(a.tm + ((int64_t)c * a.heads + head) * SsdChunk::floats + SsdChunk::p0 +
+                                              wave * 16 + q4 * 4);
+  };
+  load_own(0);
+  load_read(0);
+  for (int c = 0; c < chunks; ++c) {
+    const int par = c & 1, next = min(c + 1, chunks - 1);
 #pragma unroll
     for (int t = 0; t < NT; ++t) state[par][wave * NT + t][lane] = S[t];
     // the next state needs only this wave's own part of the last one
-    float4_t add[NT];
 #pragma unroll
-    for (int t = 0; t < NT; ++t) add[t] = S[t] * o.total;
+    for (int t = 0; t < NT; ++t) S[t] *= o.total;
 #pragma unroll
     for (int k = 0; k < 4; ++k)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const float xe = o.x[k][i] * o.e[k][i];
 #pragma unroll
-        for (int t = 0; t < NT; ++t) add[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.b[t][k][i], xe, add[t], 0, 0, 0);
+        for (int t = 0; t < NT; ++t) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.b[t][k][i], xe, S[t], 0, 0, 0);
       }
     float4_t mx = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -197,6 +205,10 @@ __global__ __launch_bounds__(256) void ssd_scan_kernel(SsdArgs a) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) mx = __builtin_amdgcn_mfma_f32_16x16x4f32(o.m[k][i], o.x[k][i], mx, 0, 0, 0);
       }
+#pragma unroll
+    for (int t = 0; t < NT; ++t)  // channels past the state stay zero
+      if ((wave * NT + t) * 16 + q4 * 4 >= N) S[t] = float4_t{0.f, 0.f, 0.f, 0.f};
+    load_own(next);
     __syncthreads();
     float4_t y[2];
     y[0] = y[1] = float4_t{0.f, 0.f, 0.f, 0.f};
@@ -207,25 +219,11 @@ __global__ __launch_bounds__(256) void ssd_scan_kernel(SsdArgs a) {
       for (int i = 0; i < 4; ++i) y[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.c[t][i], s[i], y[t & 1], 0, 0, 0);
     }
     const float4_t out = (y[0] + y[1]) * o.p0 + mx;
+    load_read(next);
     const int t0 = c * C + wave * 16 + q4 * 4;
 #pragma unroll
     for (int i = 0; i < 4; ++i)
       if (col_ok && t0 + i < a.n) a.y[(int64_t)(t0 + i) * a.ldy + head * a.vdim + col] = out[i];
-#pragma unroll
-    for (int t = 0; t < NT; ++t) {
-      // channels past the state stay zero
-      S[t] = (wave * NT + t) * 16 + q4 * 4 < N ? add[t] : float4_t{0.f, 0.f, 0.f, 0.f};
-    }
-  };
-  SsdOperands<NT> even, odd;
-  load(even, 0);
-  for (int c = 0; c < chunks; c += 2) {
-    if (c + 1 < chunks) load(odd, c + 1);
-    step(even, c, 0);
-    if (c + 1 < chunks) {
-      if (c + 2 < chunks) load(even, c + 2);
-      step(odd, c + 1, 1);
-    }
   }
 #pragma unroll
   for (int t = 0; t < NT; ++t) {

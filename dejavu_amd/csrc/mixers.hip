@@ -196,7 +196,9 @@ template <typename T, int SM, bool EMBED>
 int hyper_rows(const void* y, int n, const dvHyper& r, const dvEmbedArgs& e, const dvRmsOut& norm, hipStream_t s) {
   const dim3 grid(n, norm.h ? 1 : (r.width + 1023) / 1024);
   const size_t lds = norm.h ? (size_t)r.width * 4 : 0;
-  return launch_lds<hyper_rows_kernel<T, SM, EMBED>>(grid, dim3(256), lds, s, (const T*)y, r, e, norm);
+  if (norm.h && n <= 512 && r.width > 1024)  // few rows: more threads for each
+    return launch_lds<hyper_rows_kernel<T, SM, EMBED, 1024>>(grid, dim3(1024), lds, s, (const T*)y, r, e, norm);
+  return launch_lds<hyper_rows_kernel<T, SM, EMBED, 256>>(grid, dim3(256), lds, s, (const T*)y, r, e, norm);
 }
 
 // ---- Mamba-2 -----------------------------------------------------------------------
@@ -330,6 +332,7 @@ int dv_mix_head_rows(int dtype, const dvHeadArgs* a, void* stream) {
     heads += g.heads;
   }
   if (heads == 0) return DV_ERR_INVALID_ARG;
+  if ((int64_t)a->n * heads >= (int64_t)1 << 31) return DV_ERR_UNSUPPORTED;
   const dim3 grid(blocks_of((int64_t)a->n * heads, 16));
   if (dtype == DV_BF16) hipLaunchKernelGGL((head_rows_kernel<bf16_t>), grid, dim3(256), 0, st(stream), *a);
   else hipLaunchKernelGGL((head_rows_kernel<float>), grid, dim3(256), 0, st(stream), *a);
@@ -341,6 +344,7 @@ int dv_mix_gated_group_norm(int dtype, const float* y, int64_t ldy, const void* 
   if (!dtype_ok(dtype) || !y || !z || !w || !out || rows < 1 || dim < 1 || groups < 1 || dim % groups || padded < dim)
     return DV_ERR_INVALID_ARG;
   if (padded % 8 || ldy % 4 || ldz % 8 || !al16(y) || !al16(z) || !al16(w) || !al16(out)) return DV_ERR_ALIGNMENT;
+  if (rows * groups >= (int64_t)1 << 31) return DV_ERR_UNSUPPORTED;
   const int gs = dim / groups;
 #define DV_GROUP(T, W, VEC)                                                                                          \
   hipLaunchKernelGGL((gated_group_norm_kernel<T, W, VEC>), dim3(blocks_of(rows * groups, 4 / W)), dim3(256), 0, st(stream), \
