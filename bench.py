@@ -1094,7 +1094,7 @@ def varolorn_kernels(torch, model, near, prompt, context):
                                                            (win.kv_heads, ds, win.dim, 1, eps, 1.0, wk),
                                                            (win.kv_heads, vs, win.vdim, 0, 0.0, 1.0, wv)], False), n * hw * 4)
     p = rnd(n, mam.in_proj.shape[0])
-    xbc = torch.empty(n, mam.channels, dtype=f32, device=dev)
+    xbc = mo.ssd_rows(n, mam.channels, dev)
     dp = rnd(n, dlt.in_proj.shape[0])
     dg, dh = dlt.kv_heads, dlt.heads
     dq, dk, dvv = (torch.empty(n, w, dtype=f32, device=dev) for w in (dg * dlt.dim_s, dg * dlt.dim_s, dh * dlt.vdim_s))

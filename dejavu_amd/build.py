@@ -1,7 +1,7 @@
 """Builds the kernel libraries in-tree with hipcc for gfx950.
 
     libdejavu_hip.so     csrc/dejavu_hip.hip   contextual-sparsity decode path
-    libdejavu_mixers.so  csrc/mixers.hip       latent attention, gated delta rule, windowed attention
+    libdejavu_mixers.so  csrc/mixers.hip       latent, windowed and chunk-local attention, gated delta rule, Mamba-2
 
 Run as ``python -m dejavu_amd.build``; tests and benchmarks only load the
 libraries that this step leaves next to the package.

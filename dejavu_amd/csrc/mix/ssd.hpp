@@ -122,114 +122,200 @@ __global__ __launch_bounds__(256) void ssd_chunk_kernel(SsdArgs a, int hp) {
   }
 }
 
-// Chunk after chunk for 16 columns of a head.  Wave w owns channels [16 NT w, 16 NT (w + 1)) of the state as
-// accumulators of the 16x16x4 products (element i of a lane: channel 4 (lane / 16) + i of a tile, column lane % 16),
-// which is also the operand layout of the product with C when its channels are taken in that order; the waves exchange
+// Chunk after chunk for 16 TC columns of a head.  Wave w owns channels [16 NT w, 16 NT (w + 1)) of the state as
+// accumulators of the 16x16x4 products: row r of tile t is channel NT r + t of them, column l of tile c is column
+// TC l + c, so that a lane's operands of all tiles lie side by side in memory.  Element i of a lane is row 4 (lane / 16) +
+// i, which is also the operand layout of the product with C when its channels are taken in that order; the waves exchange
 // the state through LDS once per chunk, then every wave makes 16 tokens of Y and its own channels of the next state.
-// Operands are loaded by the lanes that use them, a chunk ahead: those of the state's own part as soon as it is done with
-// them, those of the product with the state after that product.
-template <int NT>
+// Operands are loaded by the lanes that use them, a chunk ahead; there are at most 63 loads per chunk, what the counter of
+// outstanding loads holds.
+template <int NT, int TC>
 struct SsdOperands {
-  float4_t c[4 * NT], p0, m[4], e[4];
-  float b[NT][4][4], x[4][4], total;
+  float c[4][4 * NT];  // by owner of the channels: element NT i + t is step i of tile t
+  float b[4][4][NT], x[4][4][TC];
+  float4_t p0, m[4], e[4];
+  float total;
 };
 
-// Grid: heads * ceil(vdim / 16), head fastest.
-template <int NT>
-__global__ __launch_bounds__(256, NT <= 2 ? 2 : 1) void ssd_scan_kernel(SsdArgs a) {
+template <int W>
+__device__ __forceinline__ void load_floats(float* dst, const float* __restrict__ p) {
+  typedef float vec_t __attribute__((ext_vector_type(W), aligned(4)));
+  if constexpr (W == 1) {
+    dst[0] = *p;
+  } else {
+    const vec_t v = *reinterpret_cast<const vec_t*>(p);
+#pragma unroll
+    for (int i = 0; i < W; ++i) dst[i] = v[i];
+  }
+}
+
+// Grid: heads * ceil(vdim / (16 TC)).  Workgroups go to the eight XCDs in turn: neighbouring heads, which share B and C,
+// are kept on one of them when heads % 8 == 0.  vdim % TC == 0.
+template <int NT, int TC>
+__global__ __launch_bounds__(256) void ssd_scan_kernel(SsdArgs a) {
+  static_assert(NT == 1 || NT == 2 || NT == 4, "a lane's channels are one aligned load");
   constexpr int C = kSsdChunk;
-  __shared__ __attribute__((aligned(16))) float4_t state[2][4 * NT][64];
-  const int head = blockIdx.x % a.heads, tile = blockIdx.x / a.heads;
+  __shared__ __attribute__((aligned(16))) float4_t state[2][TC][4 * NT][64];
+  const int xcds = a.heads % 8 == 0 ? 8 : 1, per = a.heads / xcds, item = blockIdx.x / xcds;
+  const int head = blockIdx.x % xcds * per + item % per, tile = item / per;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int l16 = lane & 15, q4 = lane >> 4, N = a.state_s;
   const int group = head / (a.heads / a.groups);
-  const int col = tile * kSsdCols + l16;
+  const int col = (tile * kSsdCols + l16) * TC;
   const bool col_ok = col < a.vdim;
+  const bool part = N != 64 * NT;  // some channels are not there
+  const int n0 = (wave * 16 + q4 * 4) * NT;  // channel n0 + NT i + t is element i of tile t
   float* sp = a.S + ((int64_t)head * a.vdim + (col_ok ? col : 0)) * N;
-  float4_t S[NT];
+  float4_t S[TC][NT];
 #pragma unroll
-  for (int t = 0; t < NT; ++t) {
-    const int n = (wave * NT + t) * 16 + q4 * 4;
-    S[t] = (col_ok && n < N) ? *reinterpret_cast<const float4_t*>(sp + n) : float4_t{0.f, 0.f, 0.f, 0.f};
-  }
-  const float* xcol = a.xbc + head * a.vdim + min(col, a.vdim - 1);
-  const float* Bg = a.xbc + a.off_b + group * N;
-  const float* Cg = a.xbc + a.off_c + group * N;
-  const int chunks = (a.n + C - 1) / C;
-  SsdOperands<NT> o;
-  // channels past the state meet zeros of S, tokens past the end zeros of M and e (rows of Y are not stored)
-  auto load_own = [&](int c) {
-    const float* src = a.tm + ((int64_t)c * a.heads + head) * SsdChunk::floats;
+  for (int c = 0; c < TC; ++c)
 #pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      o.e[k] = *reinterpret_cast<const float4_t*>(src + SsdChunk::e + k * 16 + q4 * 4);
+    for (int t = 0; t < NT; ++t)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const int64_t row = (int64_t)min(c * C + k * 16 + q4 * 4 + i, a.n - 1) * a.ld;
-        o.x[k][i] = xcol[row];
-#pragma unroll
-        for (int t = 0; t < NT; ++t) o.b[t][k][i] = Bg[row + min((wave * NT + t) * 16 + l16, N - 1)];
+        const int n = n0 + i * NT + t;
+        S[c][t][i] = col_ok && n < N ? sp[c * N + n] : 0.f;
       }
-      o.m[k] = *reinterpret_cast<const float4_t*>(src + SsdChunk::m + (wave * (wave + 1) / 2 + min(k, wave)) * 256 + lane * 4);
+  const int chunks = (a.n + C - 1) / C;
+  // A load is a uniform address (on the scalar unit) plus what this lane adds to it in every chunk, in bytes.
+  auto at = [](const float* base, unsigned bytes) {
+    return reinterpret_cast<const float*>(reinterpret_cast<const char*>(base) + bytes);
+  };
+  const unsigned row4 = 4 * (unsigned)a.ld;
+  const unsigned xoff = q4 * 4 * row4 + 4 * (unsigned)min(col, a.vdim - TC);
+  const unsigned boff = q4 * 4 * row4 + 4 * (unsigned)min((wave * 16 + l16) * NT, N - NT);
+  unsigned coff[4][NT];
+#pragma unroll
+  for (int w = 0; w < 4; ++w)
+#pragma unroll
+    for (int u = 0; u < NT; ++u) coff[w][u] = l16 * row4 + 4 * (unsigned)min((w * 16 + q4 * 4) * NT + u * 4, N - 4);
+  const float* Xh = a.xbc + head * a.vdim;
+  const float* Bg = a.xbc + a.off_b + group * N;
+  const float* Cg = a.xbc + a.off_c + group * N + (int64_t)wave * 16 * a.ld;
+  const unsigned yoff = q4 * 16 * (unsigned)a.ldy + 4 * col;
+  // channels past the state meet zeros of S, tokens past the end zeros of M and e (rows of Y are not stored)
+  auto load_xb = [&](SsdOperands<NT, TC>& o, int c, int k, int i) {
+    const int64_t row = ((int64_t)c * C + k * 16 + i) * a.ld;
+    load_floats<TC>(o.x[k][i], at(Xh + row, xoff));
+    load_floats<NT>(o.b[k][i], at(Bg + row, boff));
+  };
+  auto load_c = [&](SsdOperands<NT, TC>& o, int c, int w, int u) {
+    load_floats<4>(&o.c[w][u * 4], at(Cg + (int64_t)c * C * a.ld, coff[w][u]));
+  };
+  auto load_me = [&](SsdOperands<NT, TC>& o, int c, int k) {
+    const float* src = a.tm + ((int64_t)c * a.heads + head) * SsdChunk::floats;
+    o.m[k] = *reinterpret_cast<const float4_t*>(
+        at(src + SsdChunk::m + (wave * (wave + 1) / 2 + min(k, wave)) * 256, lane * 16));
+    o.e[k] = *reinterpret_cast<const float4_t*>(at(src + SsdChunk::e + k * 16, q4 * 16));
+    if (k == 0) {
+      o.p0 = *reinterpret_cast<const float4_t*>(at(src + SsdChunk::p0 + wave * 16, q4 * 16));
+      o.total = src[SsdChunk::p0 + C - 1];
     }
-    o.total = src[SsdChunk::p0 + C - 1];
   };
-  auto load_read = [&](int c) {
-    const float* cr = Cg + (int64_t)min(c * C + wave * 16 + l16, a.n - 1) * a.ld;
-#pragma unroll
-    for (int t = 0; t < 4 * NT; ++t) o.c[t] = *reinterpret_cast<const float4_t*>(cr + min(t * 16 + q4 * 4, N - 4));
-    o.p0 = *reinterpret_cast<const float4_t*>(a.tm + ((int64_t)c * a.heads + head) * SsdChunk::floats + SsdChunk::p0 +
-                                              wave * 16 + q4 * 4);
-  };
-  load_own(0);
-  load_read(0);
-  for (int c = 0; c < chunks; ++c) {
-    const int par = c & 1, next = min(c + 1, chunks - 1);
-#pragma unroll
-    for (int t = 0; t < NT; ++t) state[par][wave * NT + t][lane] = S[t];
+  // One chunk; the loads of chunk `next` are spread between the products, so that issuing them does not hold those up.
+  auto step = [&](const SsdOperands<NT, TC>& o, SsdOperands<NT, TC>& x, int ch, int next, int par) {
     // the next state needs only this wave's own part of the last one
 #pragma unroll
-    for (int t = 0; t < NT; ++t) S[t] *= o.total;
+    for (int c = 0; c < TC; ++c)
+#pragma unroll
+      for (int t = 0; t < NT; ++t) {
+        state[par][c][wave * NT + t][lane] = S[c][t];
+        S[c][t] *= o.total;
+      }
+    float4_t mx[TC];
+#pragma unroll
+    for (int c = 0; c < TC; ++c) mx[c] = float4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int k = 0; k < 4; ++k)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const float xe = o.x[k][i] * o.e[k][i];
 #pragma unroll
-        for (int t = 0; t < NT; ++t) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.b[t][k][i], xe, S[t], 0, 0, 0);
+        for (int c = 0; c < TC; ++c) {
+          const float xe = o.x[k][i][c] * o.e[k][i];
+#pragma unroll
+          for (int t = 0; t < NT; ++t)
+            S[c][t] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.b[k][i][t], xe, S[c][t], 0, 0, 0);
+        }
+        load_xb(x, next, k, i);
+        __builtin_amdgcn_sched_group_barrier(0x008, TC * NT, 0);  // matrix instructions
+        __builtin_amdgcn_sched_group_barrier(0x020, 2, 0);        // loads
       }
-    float4_t mx = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int k = 0; k < 4; ++k)
       if (k <= wave) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) mx = __builtin_amdgcn_mfma_f32_16x16x4f32(o.m[k][i], o.x[k][i], mx, 0, 0, 0);
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+          for (int c = 0; c < TC; ++c)
+            mx[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.m[k][i], o.x[k][i][c], mx[c], 0, 0, 0);
+      }
+    if (part) {  // channels past the state stay zero
+#pragma unroll
+      for (int c = 0; c < TC; ++c)
+#pragma unroll
+        for (int t = 0; t < NT; ++t)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) S[c][t][i] = n0 + i * NT + t < N ? S[c][t][i] : 0.f;
+    }
+    __syncthreads();
+    float4_t y[TC];
+#pragma unroll
+    for (int c = 0; c < TC; ++c) y[c] = float4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int w = 0; w < 4; ++w)
+#pragma unroll
+      for (int t = 0; t < NT; ++t) {
+        float4_t s[TC];
+#pragma unroll
+        for (int c = 0; c < TC; ++c) s[c] = state[par][c][w * NT + t][lane];
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+          for (int c = 0; c < TC; ++c)
+            y[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.c[w][i * NT + t], s[c][i], y[c], 0, 0, 0);
+        load_c(x, next, w, t);
+        if (t == 0) load_me(x, next, w);
+        __builtin_amdgcn_sched_group_barrier(0x008, TC * 4, 0);
+        __builtin_amdgcn_sched_group_barrier(0x020, 1, 0);
+        if (t == 0) __builtin_amdgcn_sched_group_barrier(0x020, 2, 0);
       }
 #pragma unroll
-    for (int t = 0; t < NT; ++t)  // channels past the state stay zero
-      if ((wave * NT + t) * 16 + q4 * 4 >= N) S[t] = float4_t{0.f, 0.f, 0.f, 0.f};
-    load_own(next);
-    __syncthreads();
-    float4_t y[2];
-    y[0] = y[1] = float4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int t = 0; t < 4 * NT; ++t) {
-      const float4_t s = state[par][t][lane];
-#pragma unroll
-      for (int i = 0; i < 4; ++i) y[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(o.c[t][i], s[i], y[t & 1], 0, 0, 0);
-    }
-    const float4_t out = (y[0] + y[1]) * o.p0 + mx;
-    load_read(next);
-    const int t0 = c * C + wave * 16 + q4 * 4;
+    for (int c = 0; c < TC; ++c) y[c] = y[c] * o.p0 + mx[c];
+    const int t0 = ch * C + wave * 16;
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-      if (col_ok && t0 + i < a.n) a.y[(int64_t)(t0 + i) * a.ldy + head * a.vdim + col] = out[i];
+      if (col_ok && t0 + q4 * 4 + i < a.n) {
+        float* yp = const_cast<float*>(at(a.y + (int64_t)(t0 + i) * a.ldy + head * a.vdim, yoff));
+        if constexpr (TC == 2) {
+          typedef float vec_t __attribute__((ext_vector_type(2), aligned(4)));
+          *reinterpret_cast<vec_t*>(yp) = vec_t{y[0][i], y[1][i]};
+        } else {
+          *yp = y[0][i];
+        }
+      }
+  };
+  SsdOperands<NT, TC> even, odd;
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) load_xb(even, 0, k, i);
+#pragma unroll
+    for (int u = 0; u < NT; ++u) load_c(even, 0, k, u);
+    load_me(even, 0, k);
+  }
+  for (int c = 0; c < chunks; c += 2) {
+    step(even, odd, c, min(c + 1, chunks - 1), 0);
+    if (c + 1 < chunks) step(odd, even, c + 1, min(c + 2, chunks - 1), 1);
   }
 #pragma unroll
-  for (int t = 0; t < NT; ++t) {
-    const int n = (wave * NT + t) * 16 + q4 * 4;
-    if (col_ok && n < N) *reinterpret_cast<float4_t*>(sp + n) = S[t];
-  }
+  for (int c = 0; c < TC; ++c)
+#pragma unroll
+    for (int t = 0; t < NT; ++t)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int n = n0 + i * NT + t;
+        if (col_ok && n < N) sp[c * N + n] = S[c][t][i];
+      }
 }
 
 // One decode token.  A workgroup owns 16 columns of a head, a row of 16 lanes a column.  Grid: heads * ceil(vdim / 16).

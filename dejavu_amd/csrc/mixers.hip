@@ -221,7 +221,14 @@ int ssd_scan(const SsdArgs& a, hipStream_t s) {
     hipLaunchKernelGGL((ssd_chunk_kernel<T>), dim3((unsigned)(a.groups * ((rep + hp - 1) / hp)), chunks), dim3(256), 0, s, b, hp);
     int rc = launched();
     if (rc != DV_OK) return rc;
-    hipLaunchKernelGGL((ssd_scan_kernel<NT>), dim3((unsigned)(a.heads * ((a.vdim + kSsdCols - 1) / kSsdCols))), dim3(256), 0, s, b);
+    // 32 columns per workgroup read B, C and M half as often, if that leaves about a workgroup per compute unit (and
+    // the operands of two chunks fit the registers)
+    constexpr int TC = NT <= 2 ? 2 : 1;
+    const int wide = (a.vdim + TC * kSsdCols - 1) / (TC * kSsdCols), narrow = (a.vdim + kSsdCols - 1) / kSsdCols;
+    if (a.vdim % TC == 0 && a.heads * wide >= 192)
+      hipLaunchKernelGGL((ssd_scan_kernel<NT, TC>), dim3((unsigned)(a.heads * wide)), dim3(256), 0, s, b);
+    else
+      hipLaunchKernelGGL((ssd_scan_kernel<NT, 1>), dim3((unsigned)(a.heads * narrow)), dim3(256), 0, s, b);
     rc = launched();
     if (rc != DV_OK) return rc;
   }
@@ -231,7 +238,6 @@ template <typename T>
 int ssd_scan_any(const SsdArgs& a, hipStream_t s) {
   if (a.state_s <= 64) return ssd_scan<T, 1>(a, s);
   if (a.state_s <= 128) return ssd_scan<T, 2>(a, s);
-  if (a.state_s <= 192) return ssd_scan<T, 3>(a, s);
   if (a.state_s <= 256) return ssd_scan<T, 4>(a, s);
   return DV_ERR_UNSUPPORTED;
 }

@@ -574,16 +574,29 @@ def delta_row(row, offsets, heads, kv_heads, dim, decay_up, gate_up, A_log, dt_b
     return o, gate
 
 
+SSD_CHUNK = 64
+
+
+def ssd_rows(n: int, channels: int, device) -> torch.Tensor:
+    """(n, channels) fp32 for ``ssd_scan``: zeros follow up to the end of the last chunk."""
+    rows = torch.empty((n + SSD_CHUNK - 1) // SSD_CHUNK * SSD_CHUNK, channels, dtype=torch.float32, device=device)
+    if rows.shape[0] > n:
+        rows[n:].zero_()
+    return rows[:n]
+
+
 def ssd_scan(xbc, dt, A_log, dt_bias, D, S, groups: int, off_b: int, off_c: int, width: int) -> torch.Tensor:
-    """The Mamba-2 recurrence over n tokens; xbc fp32 (n, channels): x of all heads, B from column off_b and C from
+    """The Mamba-2 recurrence over n tokens; xbc fp32 (n, channels) from ``ssd_rows``: x of all heads, B from column off_b and C from
     off_c on; dt (n, heads) logits of the step sizes.  S (heads, vdim, state) is updated.  Returns fp32 (n, width), of
     which the first heads * vdim columns are written."""
     _f32(xbc, A_log, dt_bias, D, S)
     n, (heads, vdim, state) = xbc.shape[0], S.shape
+    chunks = (n + SSD_CHUNK - 1) // SSD_CHUNK
+    assert xbc.untyped_storage().nbytes() >= 4 * (xbc.storage_offset() + chunks * SSD_CHUNK * xbc.stride(0)), "ssd_rows"
     assert dt.shape == (n, heads) and dt.stride(1) == 1 and heads * vdim <= width
     assert heads * vdim <= off_b and off_b + groups * state <= off_c and off_c + groups * state <= xbc.shape[1]
     y = torch.empty(n, width, dtype=torch.float32, device=xbc.device)
-    tm = torch.empty((min(n, 4096) + 63) // 64 * heads * 2688, dtype=torch.float32, device=xbc.device)
+    tm = torch.empty(min(chunks, 64) * heads * 2688, dtype=torch.float32, device=xbc.device)
     a = L.SsdArgs(xbc=xbc.data_ptr(), ld=xbc.stride(0), off_b=off_b, off_c=off_c, dt=dt.data_ptr(), lddt=dt.stride(0),
                   A_log=A_log.data_ptr(), dt_bias=dt_bias.data_ptr(), D=D.data_ptr(), S=S.data_ptr(), y=y.data_ptr(),
                   ldy=width, tm=tm.data_ptr(), tm_floats=tm.numel(), n=n, heads=heads, groups=groups, vdim=vdim,

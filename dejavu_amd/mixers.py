@@ -344,7 +344,7 @@ class Mamba2(nn.Module):
             y = ops.ssd_step(row, *rule, self.off_z, self.off_dt, self.inner_s)
             return ops.GroupedRow(y, self.norm, self.inner, self.norm_groups, self.eps, h.dtype)
         p = ops.linear(h, self.in_proj)
-        xbc = torch.empty(n, self.channels, dtype=torch.float32, device=h.device)
+        xbc = ops.ssd_rows(n, self.channels, h.device)
         per = 8 if self.taps <= 4 else self.channels  # channels that the convolution kernel takes together
         ops.short_conv(p, self.conv, state["conv"], [(self.channels // per, per, per, ops.NORM_NONE, 0.0, 1.0, xbc)],
                        silu=True, conv_b=self.conv_bias)

@@ -222,7 +222,8 @@ typedef struct {
 /* Mamba-2 recurrence over n tokens: S <- exp(-exp(A_log) dt) S + dt B x^T, y = S^T C + D x per head, where
  * dt = softplus(logit + dt_bias); head h uses group h / (heads / groups) of B and C. */
 typedef struct {
-  const float* xbc;        /* [n][ld]: x [heads][vdim], then from off_b on B and from off_c on C, [groups][state_s] */
+  const float* xbc;        /* [n][ld]: x [heads][vdim], then from off_b on B and from off_c on C, [groups][state_s];
+                            * rows n .. up to the next multiple of 64 are readable and finite */
   int64_t ld;
   int off_b, off_c;
   const void* dt;          /* [n][lddt] logits in `dtype`, a column per head */
