@@ -112,6 +112,7 @@ class HybridConfig:
                     mix.setdefault("vdim", size(pre + "v") // mix["kv_heads"])
                     mix["bias_rows"] = size(pre + "rel")
                 mix["chunk"] = (mix.get("mask") or {}).get("size")
+                mix["bias_max"] = int(mix["bias_max"])
                 mix["values"] = None
                 if mix.get("v_mix"):  # the first layer that says so is the source of the others
                     mix["values"], values = values, "mixed"
